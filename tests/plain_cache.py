@@ -39,9 +39,12 @@ class PlainCache:
     chunk of group g (None: no chunks): a query reads only keys of its own chunk."""
 
     def __init__(self, windows: Sequence[Optional[int]], page_size: int, num_pages: int,
-                 max_requests: int, chunks: Optional[Sequence[Optional[int]]] = None):
+                 max_requests: int, chunks: Optional[Sequence[Optional[int]]] = None,
+                 keeps: Optional[Sequence[int]] = None):
         self.windows = list(windows)
         self.chunks = list(chunks) if chunks is not None else [None] * len(self.windows)
+        # the first positions that every query of the group reads
+        self.keeps = list(keeps) if keeps is not None else [0] * len(self.windows)
         self.ps = page_size
         self.pools = [PlainPool(num_pages) for _ in windows]
         self.slots = PlainPool(max_requests)
@@ -113,7 +116,8 @@ class PlainCache:
             if w is None and self.chunks[g] is None:
                 continue
             table = r["tables"][g]
-            gone = [i for i in range(min(self._first_needed(g, new_len), len(table)))
+            gone = [i for i in range(self._pages_for(self.keeps[g]),
+                                     min(self._first_needed(g, new_len), len(table)))
                     if table[i] != NO_PAGE]
             self._give_back(g, [table[i] for i in gone])
             for i in gone:

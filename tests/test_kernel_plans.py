@@ -166,6 +166,8 @@ TESTED_AGAINST = {
     "streams_step": "plain_kugisun.py:stream_step",
     "short_conv": "plain_kugisun.py:short_convolution",
     "delta_recurrence": "plain_kugisun.py:delta_rule",
+    "rotation_table": "plain_fumanex.py:rotate", "fixed_decay": "plain_fumanex.py:decayed_sums",
+    "bias_act_rows": "plain_fumanex.py:gelu_tanh", "add_row": "plain_fumanex.py:linear",
 }
 
 

@@ -120,6 +120,8 @@ class CacheManager:
         for g, need in enumerate(by_need):
             if need.chunk is not None:
                 self._raise(self._lib.zc_set_chunk(self._core, g, int(need.chunk)))
+            if need.keep_first:
+                self._raise(self._lib.zc_set_keep(self._core, g, int(need.keep_first)))
         self._where: Dict[int, Tuple[int, int]] = {}     # schedule position -> (group, run)
         for need, runs in by_need.items():
             g = len(self.groups)
@@ -228,7 +230,8 @@ class CacheManager:
     def pages_at_most(self, n_tokens: int, portion: int) -> List[int]:
         """Upper bound, per group, of the pages a request of ``n_tokens`` tokens holds at any
         one time when it runs in portions of at most ``portion`` tokens: a group with a window
-        keeps only the window and the portion being written."""
+        keeps only the window and the portion being written (and the first positions its need
+        names)."""
         out = []
         for grp in self.groups:
             n = n_tokens
@@ -236,6 +239,9 @@ class CacheManager:
                 n = min(n, grp.need.window + portion + self.page_size)
             if grp.need.chunk is not None:
                 n = min(n, grp.need.chunk + portion + self.page_size)
+            if n < n_tokens:
+                kept = (grp.need.keep_first + self.page_size - 1) // self.page_size
+                n = min(n_tokens, n + kept * self.page_size)
             out.append((n + self.page_size - 1) // self.page_size)
         return out
 

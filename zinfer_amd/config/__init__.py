@@ -15,3 +15,5 @@ from .lodenex import LodenexConfig
 from .nupovik import NupovikConfig
 from .specs import GatedDeltaRuleSpec, ParallelMixerSpec, StreamBlockSpec
 from .kugisun import KugisunConfig
+from .specs import DistanceBiasSpec, FixedDecayAttentionSpec
+from .fumanex import FumanexConfig

@@ -14,9 +14,11 @@ from typing import List, Optional, Tuple
 
 @dataclass(frozen=True)
 class RmsNormSpec:
-    """n = x * w / sqrt(mean(x^2) + eps) over ``width`` elements."""
+    """n = x * w / sqrt(mean(x^2) + eps) over ``width`` elements; the gain is the tensor
+    ``prefix + weight_name``."""
     width: int
     eps: float
+    weight_name: str = "weight"
 
 
 @dataclass(frozen=True)
@@ -97,6 +99,17 @@ class LeadingRotarySpec:
 
 
 @dataclass(frozen=True)
+class DistanceBiasSpec:
+    """A learned number a head and bucket of distances n = i - j, added to the score: the tensor
+    ``name`` [buckets, heads] (``buckets`` None: as many as the file holds).  Half of the B buckets
+    hold one distance each, n < B/2; from there on bucket B/2 + floor(ln(n / (B/2)) / ln(far /
+    (B/2)) * (B - B/2)), at most B - 1 (``config.distance`` computes it)."""
+    far: float
+    buckets: Optional[int] = None
+    name: str = "rel"
+
+
+@dataclass(frozen=True)
 class MaskedGqaAttentionSpec:
     """Causal grouped-query attention with separate key and value sizes and these options:
     ``qk_norm_eps``: an RMS norm over the whole q projection and one over the whole k projection
@@ -108,7 +121,15 @@ class MaskedGqaAttentionSpec:
     multiplied by sigmoid(W_g h)_h, one number a head.  ``qk_norm_per_head``: the norm of q and
     of k runs over every head on its own instead, with one gain of ``head_dim`` for all heads.
     ``bias``: q, k and v have biases (``bias_suffix`` behind the matrix's name), added before
-    the norm.  The ``*_name`` fields are the tensor names below the mixer's prefix."""
+    the norm.  ``qk_unit_eps``: q and k are instead divided by their root mean square, every
+    head on its own, without a gain.  ``keep_first``: the first so many positions are seen from
+    everywhere, whatever window and chunk say.  ``distance_bias``: a ``DistanceBiasSpec``; its
+    number joins the score behind scale and cap.  ``output_bias``: the output projection has a
+    bias.  ``value_mix``: "source": the values (biased) are kept for later layers of the same
+    step; "blend": v <- (1 - lambda) v + lambda v1, v1 the source's values of the same token and
+    lambda the tensor ``value_mix_name`` (one number), ahead of the cache ("idle": the layer
+    does neither, but may bring the number, as a source may).  The ``*_name`` fields
+    are the tensor names below the mixer's prefix."""
     hidden_size: int
     n_heads: int
     n_kv_heads: int
@@ -117,6 +138,12 @@ class MaskedGqaAttentionSpec:
     scale: float
     qk_norm_eps: Optional[float] = None
     qk_norm_per_head: bool = False
+    qk_unit_eps: Optional[float] = None
+    keep_first: int = 0
+    distance_bias: Optional[DistanceBiasSpec] = None
+    output_bias: bool = False
+    value_mix: Optional[str] = None
+    value_mix_name: str = "vmix"
     bias: bool = False
     bias_suffix: str = ".b"
     rotary: Optional[LeadingRotarySpec] = None
@@ -175,10 +202,13 @@ class LatentAttentionSpec:
 @dataclass(frozen=True)
 class DenseMlpSpec:
     """down(act(up(x))), no gate: ``activation`` is "gelu" (the exact form with erf),
-    "gelu_tanh", "silu" or "relu2" (the square of max(x, 0))."""
+    "gelu_tanh", "silu" or "relu2" (the square of max(x, 0)).  ``bias``: both projections have
+    one (``bias_suffix`` behind the matrix's name)."""
     hidden_size: int
     intermediate_size: int
     activation: str = "gelu"
+    bias: bool = False
+    bias_suffix: str = ".b"
     up_name: str = "up_proj.weight"
     down_name: str = "down_proj.weight"
 
@@ -209,6 +239,35 @@ class GatedLinearAttentionSpec:
     decay_down_name: str = "a1"
     decay_up_name: str = "a2"
     decay_bias_name: str = "a2.b"
+
+
+@dataclass(frozen=True)
+class FixedDecayAttentionSpec:
+    """A mixer whose memory is one matrix a head, S [head_dim, value_dim], carried from token to
+    token in 32-bit with a decay that is one fixed number a head: S_t = g S_(t-1) + k_t v_t^T,
+    o_t = S_t^T q_t, without soft-max or denominator.  q = W_q h, k = W_k h, v = W_v h, each
+    through silu (``silu``); then ``rotary`` (a ``LeadingRotarySpec`` or None) on q and k and a
+    factor ``k_scale`` on k.  ``norm`` "head": every head's o is divided by its root mean square;
+    "row": the concatenated heads are normed together.  ``norm_name``: the norm's gain [n_heads *
+    value_dim], None: it has none.  Then times ``gate``(W_g h), "silu" or "sigmoid", then W_o.
+    The ``*_name`` fields are the tensor names below the mixer's prefix."""
+    hidden_size: int
+    n_heads: int
+    head_dim: int
+    value_dim: int
+    decay: Tuple[float, ...]
+    norm_eps: float
+    silu: bool = False
+    rotary: Optional[LeadingRotarySpec] = None
+    k_scale: float = 1.0
+    norm: str = "head"
+    norm_name: Optional[str] = None
+    gate: str = "silu"
+    q_name: str = "q"
+    k_name: str = "k"
+    v_name: str = "v"
+    gate_name: str = "g"
+    o_name: str = "o"
 
 
 @dataclass(frozen=True)
@@ -412,8 +471,8 @@ class PostNormBlockSpec:
 @dataclass(frozen=True)
 class ParallelBlockSpec:
     """x += mixer(norm1(x)) + ff(norm2(x)): both sublayers read the same x, each through a norm
-    of its own.  ``feed_forward`` None: the layer is its mixer alone (and declares no
-    ``ff_norm``)."""
+    of its own, or (``ff_norm`` None) both through norm1.  ``feed_forward`` None: the layer is its
+    mixer alone (and declares no ``ff_norm``)."""
     mixer: object
     feed_forward: Optional[object]
     mixer_norm: object

@@ -580,6 +580,86 @@ extern "C" int zf_activation(const void* x, void* out, int dtype, long long n, i
   ZF_CHECK_LAUNCH();
 }
 
+// The same over rows with a bias a column, on a slice of columns of wider rows: out[t, i] =
+// act(x[t, i] + bias[i]) for i < n, and behind them `tail` columns of which the first `ones`
+// are 1 and the rest 0 (what a product whose matrix carries its own biases as further columns
+// multiplies them with).  grid (blocks of columns, rows); V neighbouring columns a thread.
+// tanh in bfloat16 rows through one exponential (1 - 2 / (e^2u + 1)), else the library's.
+template <typename T>
+__device__ __forceinline__ float bias_act_value(float z, int kind) {
+  if (sizeof(T) == 2 && kind == 1) {
+    const float u = 0.79788456080286535588f * (z + 0.044715f * z * z * z);
+    const float e = __builtin_amdgcn_exp2f(u * 2.8853900817779268f);
+    return 0.5f * z * (2.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f));
+  }
+  return activation_value(z, kind);
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(256) void bias_act_rows_kernel(
+    const T* __restrict__ x, long long x_stride, const float* __restrict__ bias,
+    T* __restrict__ out, long long out_stride, int n, int kind, int tail, int ones) {
+  const T* xr = x + (size_t)blockIdx.y * x_stride;
+  T* orow = out + (size_t)blockIdx.y * out_stride;
+  if (blockIdx.x == 0)
+    for (int i = threadIdx.x; i < tail; i += blockDim.x)
+      store_from_float<T>(orow + n + i, i < ones ? 1.f : 0.f);
+  const int i = (blockIdx.x * blockDim.x + threadIdx.x) * V;
+  if (i >= n) return;
+  if (V == 8) {
+    const uint4 v = *(const uint4*)(xr + i);
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+    float b[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (bias != nullptr) {
+      const float4 b0 = *(const float4*)(bias + i), b1 = *(const float4*)(bias + i + 4);
+      b[0] = b0.x; b[1] = b0.y; b[2] = b0.z; b[3] = b0.w;
+      b[4] = b1.x; b[5] = b1.y; b[6] = b1.z; b[7] = b1.w;
+    }
+    uint32_t o[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      o[e] = pack_bf16x2(bias_act_value<T>(__uint_as_float(w[e] << 16) + b[2 * e], kind),
+                         bias_act_value<T>(__uint_as_float(w[e] & 0xffff0000u) + b[2 * e + 1], kind));
+    *(uint4*)(orow + i) = make_uint4(o[0], o[1], o[2], o[3]);
+  } else {
+    const float b = bias != nullptr ? bias[i] : 0.f;
+    store_from_float<T>(orow + i, bias_act_value<T>(load_as_float<T>(xr + i) + b, kind));
+  }
+}
+
+extern "C" int zf_bias_act_rows(const void* x, int dtype, long long x_stride, const float* bias,
+                                void* out, long long out_stride, int T, int n, int kind, int tail,
+                                int ones, hipStream_t stream) {
+  if (T <= 0 || n <= 0) return 0;
+  if (kind < 0 || kind > 4 || tail < 0 || ones < 0 || ones > tail) return -2;
+  const bool vec = dtype == ZF_BF16 && n % 8 == 0 && x_stride % 8 == 0 && out_stride % 8 == 0 &&
+                   (uintptr_t)x % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)bias % 16 == 0;
+  const dim3 grid((unsigned)((n / (vec ? 8 : 1) + 255) / 256), T);
+  if (vec)
+    hipLaunchKernelGGL((bias_act_rows_kernel<bf16_t, 8>), grid, dim3(256), 0, stream,
+                       (const bf16_t*)x, x_stride, bias, (bf16_t*)out, out_stride, n, kind, tail, ones);
+  else if (dtype == ZF_BF16)
+    hipLaunchKernelGGL((bias_act_rows_kernel<bf16_t, 1>), grid, dim3(256), 0, stream,
+                       (const bf16_t*)x, x_stride, bias, (bf16_t*)out, out_stride, n, kind, tail, ones);
+  else
+    hipLaunchKernelGGL((bias_act_rows_kernel<float, 1>), grid, dim3(256), 0, stream,
+                       (const float*)x, x_stride, bias, (float*)out, out_stride, n, kind, tail, ones);
+  ZF_CHECK_LAUNCH();
+}
+
+// x[t, i] += bias[i] for float32 rows
+__global__ __launch_bounds__(256) void add_row_kernel(float* __restrict__ x,
+                                                      const float* __restrict__ bias, int n) {
+  const int i = blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) x[(size_t)blockIdx.y * n + i] += bias[i];
+}
+extern "C" int zf_add_row(float* x, const float* bias, int T, int n, hipStream_t stream) {
+  if (T <= 0 || n <= 0) return 0;
+  hipLaunchKernelGGL(add_row_kernel, dim3((unsigned)((n + 255) / 256), T), dim3(256), 0, stream, x,
+                     bias, n);
+  ZF_CHECK_LAUNCH();
+}
+
 // ---------------------------------------------------------------- cast and poison
 // out[i] = in[i] in the other storage type (bfloat16 -> float32 is exact, float32 -> bfloat16
 // rounds to nearest even): weights stored in one type for a build in the other are converted

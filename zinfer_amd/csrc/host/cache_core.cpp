@@ -83,6 +83,7 @@ struct Request {
 struct Group {
   int window;      // -1: every key is kept
   int chunk = -1;  // > 0: a query reads only keys of its own chunk of this many positions
+  int keep = 0;    // the first `keep` positions are read by every query, whatever the window
   PagePool pages;
   std::vector<int> freed;      // what the last call gave back, in the order it was freed
   Group(int w, int n) : window(w), pages(n) {}
@@ -105,6 +106,8 @@ struct Core {
     if (g.chunk > 0) first = std::max(first, length / g.chunk * g.chunk);
     return first / page_size;
   }
+  // how many of a request's first pages never go back before its end
+  int kept_pages(const Group& g) const { return pages_for(g.keep); }
   static bool keeps_all(const Group& g) { return g.window < 0 && g.chunk <= 0; }
   int missing(const Group& g, const std::vector<int>& table, int length, int new_len) const {
     const int last = pages_for(new_len);
@@ -157,6 +160,15 @@ int zc_set_chunk(void* h, int group, int chunk) {
   if (group < 0 || group >= (int)c->groups.size() || chunk < 1 || !c->requests.empty())
     return fail(BAD, "zc_set_chunk: a group of the core, a chunk of at least 1, no live request");
   c->groups[(size_t)group].chunk = chunk;
+  return OK;
+}
+// a group whose queries also read the first `keep` positions of their request, however far behind
+// the window they lie, keeps the pages that hold them; set before any request is added
+int zc_set_keep(void* h, int group, int keep) {
+  Core* c = (Core*)h;
+  if (group < 0 || group >= (int)c->groups.size() || keep < 0 || !c->requests.empty())
+    return fail(BAD, "zc_set_keep: a group of the core, no negative count, no live request");
+  c->groups[(size_t)group].keep = keep;
   return OK;
 }
 void zc_destroy(void* h) { delete (Core*)h; }
@@ -253,7 +265,7 @@ int zc_commit(void* h, long long rid, int new_len) {
     std::vector<int>& table = r.tables[g];
     const int first = std::min(c->first_needed(grp, new_len), (int)table.size());
     std::vector<int> gone;
-    for (int i = 0; i < first; ++i)
+    for (int i = c->kept_pages(grp); i < first; ++i)
       if (table[(size_t)i] != NO_PAGE) {
         gone.push_back(table[(size_t)i]);
         table[(size_t)i] = NO_PAGE;

@@ -5,6 +5,9 @@
 //   key j is seen by query i when j <= i and
 //       i - j < window                         (window 0: no window)
 //       floor(i / chunk) == floor(j / chunk)   (chunk 0: no chunks; counted from position 0)
+//   or when j <= i and j < keep                  (the first keep positions are seen from everywhere)
+//   with a table of distances, s_ij = s_ij + bias[head, i - j] behind the cap (the last entry for
+//   every distance beyond the table)
 //   a_ij = exp(s_ij) / (exp(sink_h) + sum_j exp(s_ij))   sink: one learned number a head that
 //                                                        has no key and no value (null: none)
 //   o_i  = sum_j a_ij v_j;  then o_i * sigmoid(gate) with one gate an element or one a head
@@ -19,7 +22,8 @@
 //  * project_rows: the rows of a projection, segment by segment: a bias, an RMS norm over the
 //    whole segment or over every head on its own, a rotation of some leading elements of every
 //    head by the token's position (angle = position * frequency in 32-bit, pairs (i, i + dims /
-//    2) or neighbours (2i, 2i + 1)), then to plain rows or into the pools at slot_mapping.
+//    2) or neighbours (2i, 2i + 1)), a blend with rows given apart ((1 - w) x + w y), then to
+//    plain rows or into the pools at slot_mapping.
 //  * masked_attention: any sizes, both dtypes, all arithmetic 32-bit; one workgroup a (token,
 //    kv head), one wave a query head.  A token's chunks of keys start at the first key it sees,
 //    so its result never depends on how the batch was cut.
@@ -56,6 +60,9 @@ struct RowSegment {
   int dst_off;               // first column in the destination row (pool: in the key row)
   int dst_hd;                // width a head takes in the destination (pool: of a pool row)
   int pool_heads;            // pool: kv heads
+  const void* blend;         // rows [T, width] in the source's type; null: none
+  long long blend_stride;
+  float blend_w;             // what leaves is (1 - blend_w) x + blend_w y
 };
 struct RowSegments {
   RowSegment s[PR_MAX_SEGMENTS];
@@ -149,6 +156,9 @@ __global__ __launch_bounds__(256) void project_rows_kernel(
         const float cs = cs_t[j], sn = sn_t[j];
         a = first ? a * cs - b * sn : a * cs + b * sn;
       }
+      if (g.blend != nullptr)
+        a = (1.0f - g.blend_w) * a
+            + g.blend_w * load_as_float<T>((const T*)g.blend + (size_t)t * g.blend_stride + i);
       if (g.to_pool) {
         T* o = (T*)g.dst + (pool_base + head) * page_size * (size_t)g.dst_hd
                + pool_at(pool_row, g.dst_off + (d - g.skip), page_size, g.dst_hd);
@@ -297,6 +307,12 @@ __global__ __launch_bounds__(256) void project_rows_vec8_kernel(
           a[e] = first ? a[e] * cs - b[e] * sn : a[e] * cs + b[e] * sn;
         }
       }
+      if (g.blend != nullptr) {
+        float b[8];
+        pr_unpack8(*(const uint4*)((const bf16_t*)g.blend + (size_t)t * g.blend_stride + i), b);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) a[e] = (1.0f - g.blend_w) * a[e] + g.blend_w * b[e];
+      }
       bf16_t* o;
       if (g.to_pool)
         o = (bf16_t*)g.dst + (pool_base + head) * page_size * (size_t)g.dst_hd
@@ -311,8 +327,9 @@ __global__ __launch_bounds__(256) void project_rows_vec8_kernel(
 }
 
 // ints: 11 a segment (src_off, width, hd, rot_off, rot_dims, skip, to_pool, dst_off, dst_hd,
-// pool_heads, flags: 1 = a norm a head, 2 = neighbouring pairs); floats: 2 a segment (eps, mag);
-// ptrs: 4 a segment (gain, freq, dst, bias); strides: 1 a segment
+// pool_heads, flags: 1 = a norm a head, 2 = neighbouring pairs); floats: 3 a segment (eps, mag,
+// blend weight); ptrs: 5 a segment (gain, freq, dst, bias, blend); strides: 2 a segment (dst,
+// blend)
 extern "C" int zf_project_rows(const void* src, int dtype, long long src_stride,
                                const int* positions, const int* slot_mapping, int T,
                                int page_size, int n_segs, const int* ints, const float* floats,
@@ -326,11 +343,11 @@ extern "C" int zf_project_rows(const void* src, int dtype, long long src_stride,
     const int* v = ints + 11 * i;
     g.src_off = v[0]; g.width = v[1]; g.hd = v[2]; g.rot_off = v[3]; g.rot_dims = v[4];
     g.skip = v[5]; g.to_pool = v[6]; g.dst_off = v[7]; g.dst_hd = v[8]; g.pool_heads = v[9];
-    g.eps = floats[2 * i]; g.mag = floats[2 * i + 1];
+    g.eps = floats[3 * i]; g.mag = floats[3 * i + 1]; g.blend_w = floats[3 * i + 2];
     g.per_head = v[10] & 1; g.interleaved = (v[10] >> 1) & 1;
-    g.gain = (const float*)ptrs[4 * i]; g.freq = (const float*)ptrs[4 * i + 1];
-    g.dst = ptrs[4 * i + 2]; g.bias = (const float*)ptrs[4 * i + 3];
-    g.dst_stride = strides[i];
+    g.gain = (const float*)ptrs[5 * i]; g.freq = (const float*)ptrs[5 * i + 1];
+    g.dst = ptrs[5 * i + 2]; g.bias = (const float*)ptrs[5 * i + 3]; g.blend = ptrs[5 * i + 4];
+    g.dst_stride = strides[2 * i]; g.blend_stride = strides[2 * i + 1];
     if (g.per_head && g.gain != nullptr && g.hd > 0 && g.width / g.hd > PR_MAX_HEADS) return -2;
     if (g.width <= 0 || g.hd <= 0 || g.width % g.hd != 0 || g.rot_dims < 0 || g.rot_dims % 2 != 0
         || g.rot_off < 0 || g.rot_off + g.rot_dims > g.hd || g.skip < 0 || g.skip >= g.hd
@@ -345,6 +362,7 @@ extern "C" int zf_project_rows(const void* src, int dtype, long long src_stride,
     vec8 = g.src_off % 8 == 0 && g.hd % 8 == 0 && g.rot_off % 8 == 0
         && g.rot_dims % (g.interleaved ? 8 : 16) == 0
         && (g.bias == nullptr || (uintptr_t)g.bias % 16 == 0)
+        && (g.blend == nullptr || ((uintptr_t)g.blend % 16 == 0 && g.blend_stride % 8 == 0))
         && g.skip % 8 == 0 && g.dst_off % 8 == 0 && g.dst_hd % 8 == 0 && (uintptr_t)g.dst % 16 == 0
         && (g.to_pool || g.dst_stride % 8 == 0) && (g.gain == nullptr || (uintptr_t)g.gain % 16 == 0);
   }
@@ -370,11 +388,17 @@ extern "C" int zf_project_rows(const void* src, int dtype, long long src_stride,
 #define MA_GATE_ELEMENT 1
 #define MA_GATE_HEAD 2
 
+// A table of biases by distance: a row a head of dist_n + 6 floats, the distance d at column
+// dist_n + 2 - d for 0 <= d < dist_n (distances run backwards, so that keys side by side read
+// numbers side by side), the last distance's number again in the three columns ahead of it and
+// zeros in the three columns behind distance 0.
 struct MaskedAttentionArgs {
-  long long q_stride, gate_stride;
+  long long q_stride, gate_stride, out_stride;
   float scale, cap;
   int window, chunk, gate_mode;
   int nH, nKV, KW, VW, page_size, max_pages, KC;
+  int keep, dist_n;
+  const float* dist_bias;    // null: none
 };
 
 template <typename T>
@@ -408,6 +432,12 @@ __global__ __launch_bounds__(MA_MAX_WAVES * ZF_WAVE) void masked_attention_kerne
   if (a.window > 0 && pos - a.window + 1 > lo) lo = pos - a.window + 1;
   if (a.chunk > 0 && pos / a.chunk * a.chunk > lo) lo = pos / a.chunk * a.chunk;
   const int* table = block_table + (size_t)s * a.max_pages;
+  // the token's keys in order: the kept ones ahead of lo, then lo .. pos
+  const int n_kept = min(a.keep, lo);
+  const int n_keys = n_kept + pos - lo + 1;
+  auto key_at = [&](int v) { return v < n_kept ? v : lo + v - n_kept; };
+  const float* brow = a.dist_bias != nullptr
+      ? a.dist_bias + (size_t)h * (a.dist_n + 6) + a.dist_n + 2 : nullptr;
 
   const T* qrow = q + (size_t)t * a.q_stride + (size_t)h * KW;
   float* qw = qs + wave * KW;
@@ -426,24 +456,24 @@ __global__ __launch_bounds__(MA_MAX_WAVES * ZF_WAVE) void masked_attention_kerne
   const float* vsrc = v_pool != nullptr ? vs : ks;
   const int ldvs = v_pool != nullptr ? ldv : ldk;
 
-  for (int base = lo; base <= pos; base += KC) {
-    const int nk = min(KC, pos - base + 1);
+  for (int base = 0; base < n_keys; base += KC) {
+    const int nk = min(KC, n_keys - base);
     __syncthreads();                               // the tiles of the chunk before are done with
     if ((int)threadIdx.x < KC) {
-      const int key = base + threadIdx.x;
-      rows[threadIdx.x] = key <= pos ? table[key / a.page_size] * a.nKV + kvh : -1;
+      const int v = base + threadIdx.x;
+      rows[threadIdx.x] = v < n_keys ? table[key_at(v) / a.page_size] * a.nKV + kvh : -1;
     }
     __syncthreads();
     for (int i = threadIdx.x; i < nk * KW; i += blockDim.x) {
       const int j = i / KW, d = i % KW;
       ks[j * ldk + d] = load_as_float<T>(k_pool + (size_t)rows[j] * a.page_size * KW
-                                         + pool_at((base + j) % a.page_size, d, a.page_size, KW));
+                                         + pool_at(key_at(base + j) % a.page_size, d, a.page_size, KW));
     }
     if (v_pool != nullptr)
       for (int i = threadIdx.x; i < nk * VW; i += blockDim.x) {
         const int j = i / VW, d = i % VW;
         vs[j * ldv + d] = load_as_float<T>(v_pool + (size_t)rows[j] * a.page_size * VW
-                                           + pool_at((base + j) % a.page_size, d, a.page_size, VW));
+                                           + pool_at(key_at(base + j) % a.page_size, d, a.page_size, VW));
       }
     __syncthreads();
     float sc = -INFINITY;
@@ -453,6 +483,7 @@ __global__ __launch_bounds__(MA_MAX_WAVES * ZF_WAVE) void masked_attention_kerne
       for (int d = 0; d < KW; ++d) dot = fmaf(qw[d], kr[d], dot);
       sc = dot * a.scale;
       if (a.cap > 0.f) sc = a.cap * tanhf(sc / a.cap);
+      if (brow != nullptr) sc += brow[-min(pos - key_at(base + lane), a.dist_n - 1)];
     }
     const float m_new = fmaxf(m, wave_max(sc));
     const float corr = expf(m - m_new);            // exp(-inf) = 0 on a first chunk without sink
@@ -475,7 +506,7 @@ __global__ __launch_bounds__(MA_MAX_WAVES * ZF_WAVE) void masked_attention_kerne
   }
   if (!live) return;
   const float inv = 1.0f / l;
-  T* orow = out + ((size_t)t * a.nH + h) * VW;
+  T* orow = out + (size_t)t * a.out_stride + (size_t)h * VW;
   float head_gate = 1.f;
   if (a.gate_mode == MA_GATE_HEAD)
     head_gate = 1.0f / (1.0f + expf(-load_as_float<T>(gate + (size_t)t * a.gate_stride + h)));
@@ -506,13 +537,15 @@ extern "C" int zf_masked_attention(const void* q, long long q_stride, const void
                                    const void* v_pool, int dtype, const float* sink,
                                    const int* block_table, const int* q_start,
                                    const int* ctx_len, const int* seq_index, void* out,
-                                   float scale, float cap, int window, int chunk, int T, int nH,
-                                   int nKV, int KW, int VW, int page_size, int max_pages,
+                                   long long out_stride, float scale, float cap, int window,
+                                   int chunk, int keep, const float* dist_bias, int dist_n, int T,
+                                   int nH, int nKV, int KW, int VW, int page_size, int max_pages,
                                    hipStream_t stream) {
   if (T <= 0) return 0;
   if (KW <= 0 || VW <= 0 || VW > 512 || nKV <= 0 || nH % nKV != 0 || page_size <= 0
       || (v_pool == nullptr && VW > KW) || (gate_mode != MA_GATE_NONE && gate == nullptr)
-      || gate_mode < 0 || gate_mode > 2 || window < 0 || chunk < 0 || cap < 0.f)
+      || gate_mode < 0 || gate_mode > 2 || window < 0 || chunk < 0 || cap < 0.f || keep < 0
+      || (dist_bias != nullptr && dist_n < 1))
     return -2;
   const int G = nH / nKV;
   // a wave a head, up to 16; fewer where wide rows would leave no room for a chunk of keys
@@ -524,6 +557,7 @@ extern "C" int zf_masked_attention(const void* q, long long q_stride, const void
   a.q_stride = q_stride; a.gate_stride = gate_stride; a.scale = scale; a.cap = cap;
   a.window = window; a.chunk = chunk; a.gate_mode = gate_mode; a.nH = nH; a.nKV = nKV;
   a.KW = KW; a.VW = VW; a.page_size = page_size; a.max_pages = max_pages; a.KC = KC;
+  a.out_stride = out_stride; a.keep = keep; a.dist_bias = dist_bias; a.dist_n = dist_n;
   dim3 grid(T, nKV, (G + n_waves - 1) / n_waves);
   const size_t smem = ((size_t)KC * (KW + 1) + (v_pool != nullptr ? (size_t)KC * (VW + 1) : 0)
                        + (size_t)n_waves * (KW + ZF_WAVE) + KC) * sizeof(float);
@@ -739,13 +773,17 @@ __device__ __forceinline__ float mw_tanh(float x) {
 }
 
 struct MaskedWaveArgs {
-  long long q_stride, gate_stride;
+  long long q_stride, gate_stride, out_stride;
   float scale, cap;
   int window, chunk, gate_mode;
   int n_seqs, nH, nKV, page_size, max_pages, QT, wave_keys;
+  int keep, dist_n;
+  const float* dist_bias;
 };
 
-template <int KD, int VD, bool TIED, bool DECODE>
+// EXT: the first `keep` positions seen from everywhere (a wave walks the chunks of 32 that hold
+// them ahead of its own first chunk, then its own), and a bias by distance behind the cap.
+template <int KD, int VD, bool TIED, bool DECODE, bool EXT>
 __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ gate,
     const bf16_t* __restrict__ k_pool, const bf16_t* __restrict__ v_pool,
@@ -844,6 +882,17 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
   }
 
   int k_begin = k_first / MW_KEYS * MW_KEYS;
+  // EXT: the wave walks keys v from v_begin to v_end of a row in which the n_far keys of the kept
+  // positions' chunks stand ahead of the keys from k_begin on (n_far a multiple of 32): key v of
+  // that row is v itself below n_far, v + v_shift from there on
+  int n_far = 0, v_shift = 0;
+  const int keep = EXT ? a.keep : 0;
+  if constexpr (EXT) {
+    n_far = min((keep + MW_KEYS - 1) / MW_KEYS * MW_KEYS, k_begin);
+    v_shift = k_begin - n_far;
+    k_begin = 0;
+    k_end -= v_shift;
+  }
   if constexpr (DECODE) {
     k_begin += split * a.wave_keys;
     k_end = min(k_end, k_begin + a.wave_keys);
@@ -852,6 +901,14 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
     k_begin += split * share;
     k_end = min(k_end, k_begin + share);
   }
+  // where a chunk of that row begins among the positions, and the end of its keys
+  auto at = [&](int v) { return EXT && v >= n_far ? v + v_shift : v; };
+  const int pos_end = EXT ? k_end + v_shift : k_end;
+  // this lane's row of the table of biases, the distance d at [-d]
+  const float* brow = nullptr;
+  if constexpr (EXT)
+    if (a.dist_bias != nullptr)
+      brow = a.dist_bias + (size_t)h * (a.dist_n + 6) + a.dist_n + 2;
 
   // this lane's key of a chunk: key base + c; of its key row the values 16 i + 8 hl .. + 8 for
   // every i, of its value row the same
@@ -860,7 +917,8 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
   // the block [page, kv head] of this lane's key, in rows: its row there is key % page_size
   auto row_of = [&](int base, bool& ok) {
     const int key = base + c;
-    ok = key >= k_first && key < k_end;          // (pages before k_first may have gone back)
+    // (pages before k_first may have gone back)
+    ok = (key >= k_first || (EXT && key < keep)) && key < pos_end;
     size_t prow = 0;
     if (ok) prow = ((size_t)table[key / page_size] * nKV + kvh) * page_size;
     return prow;
@@ -890,11 +948,12 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
     }
   };
   if (k_begin < k_end) {
-    fetch_k(k_begin);
-    fetch_v(k_begin);
+    fetch_k(at(k_begin));
+    fetch_v(at(k_begin));
   }
-  for (int base = k_begin; base < k_end; base += MW_KEYS) {
-    const bool more = base + MW_KEYS < k_end;
+  for (int vbase = k_begin; vbase < k_end; vbase += MW_KEYS) {
+    const int base = at(vbase);
+    const bool more = vbase + MW_KEYS < k_end;
     mw_f32x16_t sc;
 #pragma unroll
     for (int r = 0; r < 16; ++r) sc[r] = 0.f;
@@ -910,8 +969,8 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
         vt[(16 * i + 8 * hl + x) * LDT + mw_swz(c, 16 * i + 8 * hl)] = e[x];
     }
     if (more) {                                     // in flight while this chunk runs
-      fetch_k(base + MW_KEYS);
-      fetch_v(base + MW_KEYS);
+      fetch_k(at(vbase + MW_KEYS));
+      fetch_v(at(vbase + MW_KEYS));
     }
     float cmax = -INFINITY;
     if (capped) {
@@ -921,9 +980,29 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
 #pragma unroll
       for (int r = 0; r < 16; ++r) sc[r] *= scale_log2;
     }
+    if constexpr (EXT) {
+      if (brow != nullptr) {
+        // keys 8 (r / 4) + 4 hl + r % 4 of the chunk: four side by side read four numbers side
+        // by side; distances beyond the table read its last number, keys ahead of the row are
+        // masked below
+        const int far = a.dist_n - 1;
+        if (__all(!row_ok || pos_r - base - (MW_KEYS - 1) >= far)) {
+          const float b = brow[-far] * MW_LOG2E;
+#pragma unroll
+          for (int r = 0; r < 16; ++r) sc[r] += b;
+        } else {
+#pragma unroll
+          for (int r4 = 0; r4 < 4; ++r4) {
+            const int d = max(0, min(pos_r - base - 8 * r4 - 4 * hl, far + 3));
+#pragma unroll
+            for (int x = 0; x < 4; ++x) sc[4 * r4 + x] = fmaf(brow[x - d], MW_LOG2E, sc[4 * r4 + x]);
+          }
+        }
+      }
+    }
     // a chunk that every row of the wave sees whole needs no mask
-    const bool whole = row_ok && base >= lo_r && base + MW_KEYS - 1 <= pos_r &&
-                       base >= k_first && base + MW_KEYS <= k_end;
+    const bool whole = row_ok && base + MW_KEYS - 1 <= pos_r && base + MW_KEYS <= pos_end &&
+                       ((base >= lo_r && base >= k_first) || (EXT && base + MW_KEYS <= keep));
     if (__all(whole)) {
 #pragma unroll
       for (int r = 0; r < 16; ++r) cmax = fmaxf(cmax, sc[r]);
@@ -931,7 +1010,8 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int key = base + 8 * (r / 4) + 4 * hl + r % 4;
-        const bool seen = row_ok && key >= lo_r && key <= pos_r && key >= k_first && key < k_end;
+        const bool seen = row_ok && key <= pos_r && key < pos_end &&
+                          ((key >= lo_r && key >= k_first) || (EXT && key < keep));
         sc[r] = seen ? sc[r] : -INFINITY;
         cmax = fmaxf(cmax, sc[r]);
       }
@@ -1003,7 +1083,7 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
     float inv = 1.0f / l;
     if (a.gate_mode == MA_GATE_HEAD)
       inv *= 1.0f / (1.0f + expf(-bf16_to_float(gate[(size_t)tok * a.gate_stride + h])));
-    bf16_t* orow = out + ((size_t)tok * a.nH + h) * VD;
+    bf16_t* orow = out + (size_t)tok * a.out_stride + (size_t)h * VD;
     const bf16_t* grow = a.gate_mode == MA_GATE_ELEMENT
         ? gate + (size_t)tok * a.gate_stride + (size_t)h * VD : nullptr;
 #pragma unroll
@@ -1027,7 +1107,7 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
 __global__ __launch_bounds__(ZF_WAVE) void masked_attention_merge_kernel(
     const float* __restrict__ ws_o, const float* __restrict__ ws_ml,
     const bf16_t* __restrict__ gate, long long gate_stride, int gate_mode,
-    bf16_t* __restrict__ out, int nH, int vd, int n_splits) {
+    bf16_t* __restrict__ out, long long out_stride, int nH, int vd, int n_splits) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const size_t slot0 = ((size_t)t * nH + h) * n_splits;
   // lane z holds split z's maximum and sum (at most 64 splits); a split without keys has the
@@ -1053,12 +1133,12 @@ __global__ __launch_bounds__(ZF_WAVE) void masked_attention_merge_kernel(
     o *= inv;
     if (gate_mode == MA_GATE_ELEMENT)
       o *= 1.0f / (1.0f + expf(-bf16_to_float(gate[(size_t)t * gate_stride + (size_t)h * vd + d])));
-    out[((size_t)t * nH + h) * vd + d] = float_to_bf16(o);
+    out[(size_t)t * out_stride + (size_t)h * vd + d] = float_to_bf16(o);
   }
 }
 
-#define MW_LAUNCH(KD, VD, TIED, DEC)                                                             \
-  hipLaunchKernelGGL((masked_attention_wave_kernel<KD, VD, TIED, DEC>), grid, dim3(256), 0,      \
+#define MW_LAUNCH(KD, VD, TIED, DEC, EXT)                                                        \
+  hipLaunchKernelGGL((masked_attention_wave_kernel<KD, VD, TIED, DEC, EXT>), grid, dim3(256), 0, \
                      stream, (const bf16_t*)q, (const bf16_t*)gate, (const bf16_t*)k_pool,       \
                      (const bf16_t*)v_pool, sink, block_table, q_start, ctx_len, (bf16_t*)out,   \
                      ws_o, ws_ml, a)
@@ -1066,15 +1146,29 @@ __global__ __launch_bounds__(ZF_WAVE) void masked_attention_merge_kernel(
 // the shapes that are built: values of their own as wide as the keys; and the keys' leading
 // columns as values (a latent and a rotated part behind it, or the latent alone)
 #define MW_SHAPES(DEC)                                                                           \
-  if (!tied && KD == 64 && VD == 64) MW_LAUNCH(64, 64, false, DEC);                              \
-  else if (!tied && KD == 96 && VD == 96) MW_LAUNCH(96, 96, false, DEC);                         \
-  else if (!tied && KD == 128 && VD == 128) MW_LAUNCH(128, 128, false, DEC);                     \
-  else if (tied && KD == 64 && VD == 64) MW_LAUNCH(64, 64, true, DEC);                           \
-  else if (tied && KD == 96 && VD == 96) MW_LAUNCH(96, 96, true, DEC);                           \
-  else if (tied && KD == 128 && VD == 128) MW_LAUNCH(128, 128, true, DEC);                       \
-  else if (tied && KD == 96 && VD == 64) MW_LAUNCH(96, 64, true, DEC);                           \
-  else if (tied && KD == 160 && VD == 128) MW_LAUNCH(160, 128, true, DEC);                       \
-  else if (tied && KD == 192 && VD == 128) MW_LAUNCH(192, 128, true, DEC);                       \
+  if (!tied && KD == 64 && VD == 64) MW_LAUNCH(64, 64, false, DEC, false); \
+  else if (!tied && KD == 96 && VD == 96) MW_LAUNCH(96, 96, false, DEC, false); \
+  else if (!tied && KD == 128 && VD == 128) MW_LAUNCH(128, 128, false, DEC, false); \
+  else if (tied && KD == 64 && VD == 64) MW_LAUNCH(64, 64, true, DEC, false); \
+  else if (tied && KD == 96 && VD == 96) MW_LAUNCH(96, 96, true, DEC, false); \
+  else if (tied && KD == 128 && VD == 128) MW_LAUNCH(128, 128, true, DEC, false); \
+  else if (tied && KD == 96 && VD == 64) MW_LAUNCH(96, 64, true, DEC, false); \
+  else if (tied && KD == 160 && VD == 128) MW_LAUNCH(160, 128, true, DEC, false); \
+  else if (tied && KD == 192 && VD == 128) MW_LAUNCH(192, 128, true, DEC, false); \
+  else return -3
+// with kept positions or biases by distance: values of their own, every pair of these widths
+#define MW_EXT_WIDTHS(K, DEC)                                                                    \
+  if (VD == 32) MW_LAUNCH(K, 32, false, DEC, true);                                              \
+  else if (VD == 64) MW_LAUNCH(K, 64, false, DEC, true);                                         \
+  else if (VD == 96) MW_LAUNCH(K, 96, false, DEC, true);                                         \
+  else if (VD == 128) MW_LAUNCH(K, 128, false, DEC, true);                                       \
+  else return -3
+#define MW_EXT_SHAPES(DEC)                                                                       \
+  if (tied) return -3;                                                                           \
+  if (KD == 32) { MW_EXT_WIDTHS(32, DEC); }                                                      \
+  else if (KD == 64) { MW_EXT_WIDTHS(64, DEC); }                                                 \
+  else if (KD == 96) { MW_EXT_WIDTHS(96, DEC); }                                                 \
+  else if (KD == 128) { MW_EXT_WIDTHS(128, DEC); }                                               \
   else return -3
 
 // decode == 0: a step's tokens in tiles of 128 / G positions, n_tiles an upper bound of the
@@ -1087,9 +1181,10 @@ extern "C" int zf_masked_attention_mfma(const void* q, long long q_stride, const
                                         long long gate_stride, int gate_mode, const void* k_pool,
                                         const void* v_pool, const float* sink,
                                         const int* block_table, const int* q_start,
-                                        const int* ctx_len, void* out, float* ws_o, float* ws_ml,
-                                        float scale, float cap, int window, int chunk, int T,
-                                        int n_seqs, int n_tiles, int nH, int nKV, int KD, int VD,
+                                        const int* ctx_len, void* out, long long out_stride,
+                                        float* ws_o, float* ws_ml, float scale, float cap,
+                                        int window, int chunk, int keep, const float* dist_bias,
+                                        int dist_n, int T, int n_seqs, int n_tiles, int nH, int nKV, int KD, int VD,
                                         int page_size, int max_pages, int decode, int n_splits,
                                         int wave_keys, hipStream_t stream) {
   if (T <= 0) return 0;
@@ -1098,8 +1193,9 @@ extern "C" int zf_masked_attention_mfma(const void* q, long long q_stride, const
       splits > ZF_WAVE || ((decode || n_splits > 1) && (!ws_o || !ws_ml)) ||
       (decode && (wave_keys <= 0 || wave_keys % MW_KEYS != 0 || T != n_seqs)) ||
       gate_mode < 0 || gate_mode > 2 || (gate_mode != MA_GATE_NONE && gate == nullptr) ||
-      window < 0 || chunk < 0 || cap < 0.f)
+      window < 0 || chunk < 0 || cap < 0.f || keep < 0 || (dist_bias != nullptr && dist_n < 1))
     return -2;
+  const bool ext = keep > 0 || dist_bias != nullptr;
   const bool tied = v_pool == nullptr;
   MaskedWaveArgs a;
   a.q_stride = q_stride; a.gate_stride = gate_stride; a.scale = scale; a.cap = cap;
@@ -1107,17 +1203,21 @@ extern "C" int zf_masked_attention_mfma(const void* q, long long q_stride, const
   a.nKV = nKV; a.page_size = page_size; a.max_pages = max_pages;
   a.QT = decode ? 1 : MW_ROWS / (nH / nKV);
   a.wave_keys = wave_keys;
-  if (decode) {
-    dim3 grid(n_seqs, nKV, n_splits);
+  a.out_stride = out_stride; a.keep = keep; a.dist_bias = dist_bias; a.dist_n = dist_n;
+  if (!decode && n_tiles <= 0) return 0;
+  const dim3 grid(decode ? n_seqs : n_tiles, nKV, n_splits);
+  if (ext && decode) {
+    MW_EXT_SHAPES(true);
+  } else if (ext) {
+    MW_EXT_SHAPES(false);
+  } else if (decode) {
     MW_SHAPES(true);
   } else {
-    if (n_tiles <= 0) return 0;
-    dim3 grid(n_tiles, nKV, n_splits);
     MW_SHAPES(false);
   }
   if (decode || n_splits > 1)
     hipLaunchKernelGGL(masked_attention_merge_kernel, dim3(T, nH), dim3(ZF_WAVE), 0, stream, ws_o,
-                       ws_ml, (const bf16_t*)gate, gate_stride, gate_mode, (bf16_t*)out, nH, VD,
-                       splits);
+                       ws_ml, (const bf16_t*)gate, gate_stride, gate_mode, (bf16_t*)out,
+                       out_stride, nH, VD, splits);
   ZF_CHECK_LAUNCH();
 }

@@ -605,43 +605,82 @@ extern "C" int zf_decay_recurrence_spans(const void* q, long long q_stride, cons
 }
 
 // ---------------------------------------------------------------- norm a head, gain, gate
-// a wave a (token, head): out[t, h, :] = o / sqrt(mean(o^2) + eps) * gain * silu(g[t, h, :]);
-// gain [dv] (one for all heads) or [H dv].  o float32, g and out in the rows' type.
-template <typename T>
+// out[t, h, :] = o / sqrt(mean(o^2) + eps) * gain * gate(g[t, h, :]) with the gate silu (0) or the
+// sigmoid (1); gain [dv] (one for all heads), [H dv], or null.  o float32, g and out in the rows'
+// type, rows of g and out at strides of their own.  A wave a (token, head), or (WIDE) a workgroup
+// of four waves, whose sums are added in wave order.
+template <typename T, bool WIDE>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(
     const float* __restrict__ o, const float* __restrict__ gain, int gain_per_head,
-    const T* __restrict__ g, long long g_stride, T* __restrict__ out, int n_rows, int H, int dv,
-    float eps) {
+    const T* __restrict__ g, long long g_stride, int gate_kind, T* __restrict__ out,
+    long long out_stride, int n_rows, int H, int dv, float eps, int quads) {
+  __shared__ float red[16];
   const int wave = threadIdx.x / ZF_WAVE, lane = threadIdx.x % ZF_WAVE;
-  const int r = blockIdx.x * (blockDim.x / ZF_WAVE) + wave;       // (token, head)
-  if (r >= n_rows) return;
+  const int r = WIDE ? blockIdx.x : blockIdx.x * (blockDim.x / ZF_WAVE) + wave;   // (token, head)
+  if (r >= n_rows) return;                // (WIDE: the whole workgroup)
   const int t = r / H, hd = r % H;
+  const int at = WIDE ? threadIdx.x : lane, step = WIDE ? blockDim.x : ZF_WAVE;
   const float* row = o + (size_t)r * dv;
   float ss = 0.f;
-  for (int i = lane; i < dv; i += ZF_WAVE) ss = fmaf(row[i], row[i], ss);
-  ss = wave_sum(ss);
+  if (quads) {
+    for (int i = 4 * at; i < dv; i += 4 * step) {
+      const float4 x = *(const float4*)(row + i);
+      ss = fmaf(x.x, x.x, fmaf(x.y, x.y, fmaf(x.z, x.z, fmaf(x.w, x.w, ss))));
+    }
+  } else {
+    for (int i = at; i < dv; i += step) ss = fmaf(row[i], row[i], ss);
+  }
+  ss = WIDE ? block_sum(ss, red) : wave_sum(ss);
   const float inv = 1.0f / sqrtf(ss / (float)dv + eps);
-  const T* gr = g + (size_t)t * g_stride + hd * dv;
-  const float* gn = gain + (gain_per_head ? hd * dv : 0);
-  for (int i = lane; i < dv; i += ZF_WAVE) {
-    const float gv = load_as_float<T>(gr + i);
-    const float silu = gv / (1.0f + expf(-gv));
-    store_from_float<T>(out + (size_t)r * dv + i, row[i] * inv * gn[i] * silu);
+  const T* gr = g + (size_t)t * g_stride + (size_t)hd * dv;
+  T* orow = out + (size_t)t * out_stride + (size_t)hd * dv;
+  const float* gn = gain == nullptr ? nullptr : gain + (gain_per_head ? hd * dv : 0);
+  auto value = [&](float x, float gv, float gg) {
+    const float s = 1.0f / (1.0f + expf(-gv));
+    return x * inv * gg * (gate_kind == 0 ? gv * s : s);
+  };
+  if (quads) {
+    for (int i = 4 * at; i < dv; i += 4 * step) {
+      const float4 x = *(const float4*)(row + i);
+      float4 gg = float4{1.f, 1.f, 1.f, 1.f};
+      if (gn != nullptr) gg = *(const float4*)(gn + i);
+      if constexpr (sizeof(T) == 2) {
+        const uint2 w = *(const uint2*)(gr + i);
+        *(uint2*)(orow + i) = make_uint2(
+            pack_bf16x2(value(x.x, __uint_as_float(w.x << 16), gg.x),
+                        value(x.y, __uint_as_float(w.x & 0xffff0000u), gg.y)),
+            pack_bf16x2(value(x.z, __uint_as_float(w.y << 16), gg.z),
+                        value(x.w, __uint_as_float(w.y & 0xffff0000u), gg.w)));
+      } else {
+        const float4 w = *(const float4*)(gr + i);
+        *(float4*)(orow + i) = float4{value(x.x, w.x, gg.x), value(x.y, w.y, gg.y),
+                                      value(x.z, w.z, gg.z), value(x.w, w.w, gg.w)};
+      }
+    }
+  } else {
+    for (int i = at; i < dv; i += step)
+      store_from_float<T>(orow + i, value(row[i], load_as_float<T>(gr + i), gn != nullptr ? gn[i] : 1.f));
   }
 }
 
 extern "C" int zf_head_norm_gate(const float* o, const float* gain, int gain_per_head,
-                                 const void* g, long long g_stride, void* out, int dtype, int T,
-                                 int H, int dv, float eps, hipStream_t stream) {
+                                 const void* g, long long g_stride, int gate_kind, void* out,
+                                 long long out_stride, int dtype, int T, int H, int dv, float eps,
+                                 hipStream_t stream) {
   if (T <= 0) return 0;
-  if (H <= 0 || dv <= 0) return -2;
+  if (H <= 0 || dv <= 0 || gate_kind < 0 || gate_kind > 1) return -2;
   const int rows = T * H;
-  const dim3 grid((rows + 3) / 4), block(4 * ZF_WAVE);
-  if (dtype == ZF_F32)
-    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, block, 0, stream, o, gain,
-                       gain_per_head, (const float*)g, g_stride, (float*)out, rows, H, dv, eps);
-  else
-    hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, block, 0, stream, o, gain,
-                       gain_per_head, (const bf16_t*)g, g_stride, (bf16_t*)out, rows, H, dv, eps);
+  const int esz = dtype == ZF_F32 ? 4 : 2;
+  const int quads = dv % 4 == 0 && (uintptr_t)o % 16 == 0 && (uintptr_t)gain % 16 == 0 &&
+                    (uintptr_t)g % (4 * esz) == 0 && (uintptr_t)out % (4 * esz) == 0 &&
+                    g_stride % 4 == 0 && out_stride % 4 == 0;
+  const bool wide = dv > 512;
+  const dim3 grid(wide ? rows : (rows + 3) / 4), block(4 * ZF_WAVE);
+#define HNG(TT, W)                                                                               \
+  hipLaunchKernelGGL((head_norm_gate_kernel<TT, W>), grid, block, 0, stream, o, gain,            \
+                     gain_per_head, (const TT*)g, g_stride, gate_kind, (TT*)out, out_stride,     \
+                     rows, H, dv, eps, quads)
+  if (dtype == ZF_F32) { if (wide) HNG(float, true); else HNG(float, false); }
+  else { if (wide) HNG(bf16_t, true); else HNG(bf16_t, false); }
   ZF_CHECK_LAUNCH();
 }

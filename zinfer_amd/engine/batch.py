@@ -91,6 +91,9 @@ class StepContext:
     norm_after: object = None
     norm_after_block: object = None   # the norm that reads the stream first after this block
     norm_ready: object = None
+    # what a part leaves for later parts of the same pass over the step's tokens (the decoder
+    # empties it when a pass begins): a source layer's values, a rotation's table
+    shared: Dict[object, object] = field(default_factory=dict)
     _scratch: Scratch = None
 
     def scratch(self, name: str, shape, dtype) -> torch.Tensor:

@@ -134,6 +134,7 @@ class DecoderModel:
         ``caches[pos]`` is the cache view of schedule position ``pos`` (or None)."""
         s = self.spec
         T = step.n_tokens
+        step.shared.clear()
         copies = None
         if s.streams is not None:
             # the stream in several copies, all equal to the embedding's output at the start

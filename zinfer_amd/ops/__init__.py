@@ -2011,6 +2011,41 @@ def activation(x: torch.Tensor, out: torch.Tensor, kind: str) -> None:
 
 
 @_launches("norm_rope_write")
+def bias_act_rows(x: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor, kind: str,
+                  tail: int = 0, ones: int = 0) -> None:
+    """out[:, :n] = act(x + bias) for rows x [T, n] (a slice of columns of wider rows is fine, as
+    for ``out``) and ``bias`` float32 [n] or None, in 32-bit; ``kind`` as for ``activation``.
+    ``out`` is [T, n + tail]: its last ``tail`` columns become 1 (the first ``ones`` of them) or
+    0, which is what a product whose matrix carries biases as further columns reads there."""
+    for t in (x, bias, out):
+        if t is not None and not t.is_cuda:
+            raise KernelUnavailable("the HIP kernels run on GPU tensors only")
+    T, n = x.shape
+    xs, os_ = _columns(x, "bias_act_rows: x"), _columns(out, "bias_act_rows: out")
+    if kind not in ACTIVATIONS or out.shape != (T, n + tail) or out.dtype != x.dtype \
+            or not 0 <= ones <= tail or (bias is not None and (
+                bias.shape != (n,) or bias.dtype != torch.float32 or not bias.is_contiguous())):
+        raise KernelUnavailable(f"bias_act_rows: {tuple(x.shape)} {x.dtype} -> "
+                                f"{tuple(out.shape)} {out.dtype} with {tail} columns behind, kind "
+                                f"{kind!r} of {sorted(ACTIVATIONS)}")
+    lib = build.load("elementwise")
+    _check(lib.zf_bias_act_rows(_ptr(x), _dt(x), ctypes.c_longlong(xs), _ptr(bias), _ptr(out),
+                                ctypes.c_longlong(os_), T, n, ACTIVATIONS[kind], int(tail),
+                                int(ones), _stream()), "bias_act_rows")
+
+
+@_launches("norm_rope_write")
+def add_row(x: torch.Tensor, bias: torch.Tensor) -> None:
+    """x[t] += bias for every row of ``x`` [T, n], both float32."""
+    _need_gpu(x, bias)
+    T, n = x.shape
+    if x.dtype != torch.float32 or bias.dtype != torch.float32 or bias.shape != (n,):
+        raise KernelUnavailable(f"add_row: {tuple(x.shape)} {x.dtype} += {tuple(bias.shape)}")
+    lib = build.load("elementwise")
+    _check(lib.zf_add_row(_ptr(x), _ptr(bias), T, n, _stream()), "add_row")
+
+
+@_launches("norm_rope_write")
 def norm_add_store(y: torch.Tensor, gain: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
                    centred: bool, x: torch.Tensor, out: torch.Tensor) -> None:
     """x += norm(y); out = x rounded to ``out``'s type, row by row in 32-bit (``norm_rows`` with
@@ -2044,13 +2079,15 @@ class RowSegment:
     ``masked_pool_from_rows`` says) at the token's slot, from column dst_off of the row on.
     ``bias`` [width] float32 is added to the source's values before anything else.  ``per_head``:
     the norm runs over every head on its own and ``gain`` is [hd], one for all heads.
-    ``interleaved``: the rotated pairs are the neighbours (2i, 2i + 1), pair i by freq[i]."""
+    ``interleaved``: the rotated pairs are the neighbours (2i, 2i + 1), pair i by freq[i].
+    ``blend`` = (rows [T, width] in the source's type, w): what leaves is (1 - w) x + w y, x the
+    segment's value and y the given row's."""
 
     def __init__(self, src_off: int, width: int, dst: torch.Tensor, *, gain=None, eps: float = 0.0,
                  hd: Optional[int] = None, rot_off: int = 0, rot_dims: int = 0, freq=None,
                  mag: float = 1.0, skip: int = 0, dst_off: int = 0, dst_hd: Optional[int] = None,
                  pool_heads: Optional[int] = None, bias=None, per_head: bool = False,
-                 interleaved: bool = False):
+                 interleaved: bool = False, blend=None):
         self.src_off, self.width, self.dst = int(src_off), int(width), dst
         self.gain, self.eps = gain, float(eps)
         self.hd = int(hd) if hd is not None else int(width)
@@ -2059,6 +2096,7 @@ class RowSegment:
         self.dst_hd = int(dst_hd) if dst_hd is not None else self.hd - self.skip
         self.pool_heads = pool_heads
         self.bias, self.per_head, self.interleaved = bias, bool(per_head), bool(interleaved)
+        self.blend, self.blend_w = (None, 0.0) if blend is None else (blend[0], float(blend[1]))
 
 
 PROJECT_ROWS_MAX_SEGMENTS = 4
@@ -2094,7 +2132,10 @@ def project_rows(src: torch.Tensor, positions: torch.Tensor, slot_mapping: Optio
                                     and g.bias.shape == (g.width,) and g.bias.is_contiguous())) \
             and (g.rot_dims == 0 or (g.freq is not None and g.freq.is_cuda
                                      and g.freq.dtype == torch.float32
-                                     and g.freq.shape == (g.rot_dims // 2,)))
+                                     and g.freq.shape == (g.rot_dims // 2,))) \
+            and (g.blend is None or (g.blend.is_cuda and g.blend.dtype == src.dtype
+                                     and g.blend.shape == (T, g.width)
+                                     and g.blend.stride(1) == 1))
         heads = g.width // max(g.hd, 1)
         if ok and pool:
             _i32(slot_mapping, "slot_mapping")
@@ -2114,10 +2155,12 @@ def project_rows(src: torch.Tensor, positions: torch.Tensor, slot_mapping: Optio
         ints += [g.src_off, g.width, g.hd, g.rot_off, g.rot_dims, g.skip, 1 if pool else 0,
                  g.dst_off, g.dst_hd, g.pool_heads or 0,
                  (1 if g.per_head else 0) | (2 if g.interleaved else 0)]
-        floats += [g.eps, g.mag]
+        floats += [g.eps, g.mag, g.blend_w]
+        strides.append(g.blend.stride(0) if g.blend is not None else 0)
         ptrs += [g.gain.data_ptr() if g.gain is not None else None,
                  g.freq.data_ptr() if g.rot_dims else None, g.dst.data_ptr(),
-                 g.bias.data_ptr() if g.bias is not None else None]
+                 g.bias.data_ptr() if g.bias is not None else None,
+                 g.blend.data_ptr() if g.blend is not None else None]
     lib = build.load("masked_attention")
     _check(lib.zf_project_rows(
         _ptr(src), _dt(src), ctypes.c_longlong(stride), _ptr(positions), _ptr(slot_mapping), T,
@@ -2148,11 +2191,28 @@ def masked_pool_rows(pool: torch.Tensor, n_heads: int, page_size: int, width: in
 
 
 GATE_MODES = {None: 0, "element": 1, "head": 2}
+DISTANCE_PADS = 6            # three columns ahead of the last distance, three behind distance 0
+
+
+def distance_table(bias: torch.Tensor) -> torch.Tensor:
+    """The kernels' form of biases by distance, from ``bias`` [nH, N] (float32; entry n: the bias
+    of a key n positions back, the last one for every distance from N - 1 on): [nH, N + 6], the
+    distances running backwards so that keys side by side read numbers side by side, the last
+    one's number three times more ahead of it and three zeros behind distance 0."""
+    H, N = bias.shape
+    back = bias.to(torch.float32).flip(1)
+    return torch.cat([back[:, :1].expand(H, 3), back,
+                      torch.zeros((H, 3), dtype=torch.float32, device=bias.device)],
+                     dim=1).contiguous()
+
+
+def _distances(dist_bias) -> int:
+    return 0 if dist_bias is None else dist_bias.shape[1] - DISTANCE_PADS
 
 
 def _masked_attention_checks(what, q, gate, gate_mode, k_pool, v_pool, sink, block_table, q_start,
                              ctx_len, seq_index, out, n_heads, n_kv_heads, key_width,
-                             value_width, page_size, max_ctx_len):
+                             value_width, page_size, max_ctx_len, keep=0, dist_bias=None):
     for t in (q, gate, k_pool, v_pool, sink, block_table, q_start, ctx_len, seq_index, out):
         if t is not None and not t.is_cuda:
             raise KernelUnavailable("the HIP kernels run on GPU tensors only")
@@ -2161,8 +2221,14 @@ def _masked_attention_checks(what, q, gate, gate_mode, k_pool, v_pool, sink, blo
         raise KernelUnavailable(f"{what}: gate mode {gate_mode!r} of {list(GATE_MODES)}, with a "
                                 "gate exactly when there is a mode")
     gate_cols = {None: 0, "element": n_heads * value_width, "head": n_heads}[gate_mode]
+    if keep < 0 or (dist_bias is not None and (
+            not dist_bias.is_cuda or dist_bias.dtype != torch.float32 or dist_bias.dim() != 2
+            or dist_bias.shape[0] != n_heads or dist_bias.shape[1] < DISTANCE_PADS + 1
+            or not dist_bias.is_contiguous())):
+        raise KernelUnavailable(f"{what}: the table of biases by distance is float32 [nH, "
+                                "distances] as ``distance_table`` lays it out")
     if q.shape[1] != n_heads * key_width or out.shape != (T, n_heads * value_width) \
-            or not out.is_contiguous() or out.dtype != q.dtype or k_pool.dtype != q.dtype \
+            or out.stride(1) != 1 or out.dtype != q.dtype or k_pool.dtype != q.dtype \
             or (v_pool is not None and v_pool.dtype != q.dtype) \
             or (gate is not None and (gate.shape != (T, gate_cols) or gate.dtype != q.dtype)) \
             or (sink is not None and (sink.dtype != torch.float32 or sink.shape != (n_heads,))):
@@ -2195,7 +2261,8 @@ def masked_attention(q: torch.Tensor, gate: Optional[torch.Tensor], gate_mode: O
                      sink: Optional[torch.Tensor], block_table, q_start, ctx_len, seq_index,
                      out: torch.Tensor, scale: float, cap: float, window: int, chunk: int,
                      n_heads: int, n_kv_heads: int, key_width: int, value_width: int,
-                     page_size: int, max_ctx_len: int) -> None:
+                     page_size: int, max_ctx_len: int, keep: int = 0,
+                     dist_bias: Optional[torch.Tensor] = None) -> None:
     """Causal grouped-query attention over paged pools of blocks [page, kv head] of rows (laid
     out as ``masked_pool_from_rows`` says): keys of ``key_width``, values of ``value_width``
     elements, or with ``v_pool`` None the first ``value_width`` columns of the key rows.  Token t of sequence s = seq_index[t] has position p = ctx_len[s] -
@@ -2203,19 +2270,22 @@ def masked_attention(q: torch.Tensor, gate: Optional[torch.Tensor], gate_mode: O
     floor(j / chunk) == floor(p / chunk) (chunk > 0).  Scores are scale * q . k, then with
     cap > 0 cap * tanh(score / cap).  ``sink`` [nH] float32: the soft-max's denominator holds
     exp(sink_h) once more.  ``gate`` with mode "element" [T, nH * value width] or "head" [T, nH]:
-    the output is multiplied by sigmoid(gate).  ``q`` and ``gate`` may be column slices of a
-    wider product.  All arithmetic is 32-bit in both dtypes."""
+    the output is multiplied by sigmoid(gate).  The keys j < ``keep`` (and
+    j <= p) are read from everywhere, whatever window and chunk say.  ``dist_bias``
+    (``distance_table``): a number a head and distance p - j is added to the capped score.  ``q``,
+    ``gate`` and ``out`` may be column slices of wider rows.  All arithmetic is 32-bit in both dtypes."""
     _masked_attention_checks("masked_attention", q, gate, gate_mode, k_pool, v_pool, sink,
                              block_table, q_start, ctx_len, seq_index, out, n_heads, n_kv_heads,
-                             key_width, value_width, page_size, max_ctx_len)
+                             key_width, value_width, page_size, max_ctx_len, keep, dist_bias)
     qs = _columns(q, "masked_attention: q")
     gs = _columns(gate, "masked_attention: gate") if gate is not None else 0
     lib = build.load("masked_attention")
     code = lib.zf_masked_attention(
         _ptr(q), ctypes.c_longlong(qs), _ptr(gate), ctypes.c_longlong(gs), GATE_MODES[gate_mode],
         _ptr(k_pool), _ptr(v_pool), _dt(q), _ptr(sink), _ptr(block_table), _ptr(q_start),
-        _ptr(ctx_len), _ptr(seq_index), _ptr(out), ctypes.c_float(scale), ctypes.c_float(cap),
-        int(window), int(chunk), q.shape[0], n_heads, n_kv_heads, key_width, value_width,
+        _ptr(ctx_len), _ptr(seq_index), _ptr(out), ctypes.c_longlong(out.stride(0)),
+        ctypes.c_float(scale), ctypes.c_float(cap), int(window), int(chunk), int(keep),
+        _ptr(dist_bias), _distances(dist_bias), q.shape[0], n_heads, n_kv_heads, key_width, value_width,
         page_size, block_table.shape[1], _stream())
     if code == -3:
         raise KernelUnavailable(f"masked_attention: key rows of {key_width} are wider than the "
@@ -2258,6 +2328,8 @@ def head_products(a: torch.Tensor, a_off: int, a_hd: int, w: torch.Tensor,
 # leading columns as values
 MASKED_MFMA_SHAPES = {False: ((64, 64), (96, 96), (128, 128)),
                       True: ((64, 64), (96, 96), (128, 128), (96, 64), (160, 128), (192, 128))}
+# with kept first positions or biases by distance: values of their own, any pair of these
+MASKED_MFMA_EXT_WIDTHS = (32, 64, 96, 128)
 MASKED_MFMA_ROWS = 128           # (position, head) pairs a workgroup takes
 MASKED_ROWS_WAVES = 2048         # a prompt portion's keys are cut in parts until this many waves run
 MASKED_ROWS_MAX_PARTS = 4
@@ -2265,36 +2337,43 @@ MASKED_DECODE_WORKGROUPS = 1024  # a decode step's contexts are split until abou
 
 
 def masked_attention_mfma_covers(dtype, n_heads: int, n_kv_heads: int, key_width: int,
-                                 value_width: int, tied: bool) -> bool:
+                                 value_width: int, tied: bool, extended: bool = False) -> bool:
     """Whether the bfloat16 MFMA kernels take the shape; otherwise (and in 32-bit) the kernel
-    for every size runs."""
+    for every size runs.  ``extended``: with kept first positions or biases by distance."""
+    if extended:
+        return dtype == torch.bfloat16 and not tied and n_heads // n_kv_heads <= 32 \
+            and key_width in MASKED_MFMA_EXT_WIDTHS and value_width in MASKED_MFMA_EXT_WIDTHS
     return dtype == torch.bfloat16 and (key_width, value_width) in MASKED_MFMA_SHAPES[bool(tied)] \
         and n_heads // n_kv_heads <= 32
 
 
 def attend_masked(q, gate, gate_mode, k_pool, v_pool, sink, block_table, q_start, ctx_len,
                   seq_index, out, scale, cap, window, chunk, n_heads, n_kv_heads, key_width,
-                  value_width, page_size, max_q_len, max_ctx_len) -> None:
+                  value_width, page_size, max_q_len, max_ctx_len, keep: int = 0,
+                  dist_bias: Optional[torch.Tensor] = None) -> None:
     """``masked_attention`` through the fastest kernel that takes the shape: in bfloat16, for
     the widths of ``MASKED_MFMA_SHAPES``, the MFMA kernels (``masked_attention_mfma``); else
     the 32-bit kernel.  Same arguments, same result up to rounding."""
     if masked_attention_mfma_covers(q.dtype, n_heads, n_kv_heads, key_width, value_width,
-                                    v_pool is None) \
-            and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0:
+                                    v_pool is None, keep > 0 or dist_bias is not None) \
+            and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0 \
+            and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0:
         masked_attention_mfma(q, gate, gate_mode, k_pool, v_pool, sink, block_table, q_start,
                               ctx_len, out, scale, cap, window, chunk, n_heads, n_kv_heads,
-                              key_width, value_width, page_size, max_q_len, max_ctx_len)
+                              key_width, value_width, page_size, max_q_len, max_ctx_len,
+                              keep=keep, dist_bias=dist_bias)
     else:
         masked_attention(q, gate, gate_mode, k_pool, v_pool, sink, block_table, q_start, ctx_len,
                          seq_index, out, scale, cap, window, chunk, n_heads, n_kv_heads,
-                         key_width, value_width, page_size, max_ctx_len)
+                         key_width, value_width, page_size, max_ctx_len, keep, dist_bias)
 
 
 @_launches("attention")
 def masked_attention_mfma(q, gate, gate_mode, k_pool, v_pool, sink, block_table, q_start, ctx_len,
                           out, scale, cap, window, chunk, n_heads, n_kv_heads, key_width,
                           value_width, page_size, max_q_len, max_ctx_len,
-                          n_splits: Optional[int] = None) -> None:
+                          n_splits: Optional[int] = None, keep: int = 0,
+                          dist_bias: Optional[torch.Tensor] = None) -> None:
     """The bfloat16 MFMA form of ``masked_attention`` (see there for the arguments).  Scores, cap
     and soft-max are 32-bit; a weight enters the second product as the sum of two bfloat16
     numbers.  Every wave takes 32 (position, head) rows and walks their keys on its own.  A step
@@ -2305,21 +2384,26 @@ def masked_attention_mfma(q, gate, gate_mode, k_pool, v_pool, sink, block_table,
     waves take their keys in ``n_splits`` parts where few waves stand behind long contexts."""
     _masked_attention_checks("masked_attention_mfma", q, gate, gate_mode, k_pool, v_pool, sink,
                              block_table, q_start, ctx_len, None, out, n_heads, n_kv_heads,
-                             key_width, value_width, page_size, max_ctx_len)
+                             key_width, value_width, page_size, max_ctx_len, keep, dist_bias)
     T = q.shape[0]
     qs = _columns(q, "masked_attention_mfma: q")
     gs = _columns(gate, "masked_attention_mfma: gate") if gate is not None else 0
     if not masked_attention_mfma_covers(q.dtype, n_heads, n_kv_heads, key_width, value_width,
-                                        v_pool is None) or qs % 8 != 0 or q.data_ptr() % 16 != 0:
+                                        v_pool is None, keep > 0 or dist_bias is not None) \
+            or qs % 8 != 0 or q.data_ptr() % 16 != 0 or out.stride(0) % 4 != 0 \
+            or out.data_ptr() % 8 != 0:
         raise KernelUnavailable(f"masked_attention_mfma: bfloat16, (key, value) widths of "
-                                f"{MASKED_MFMA_SHAPES}, at most 32 heads a kv head, query rows "
-                                "aligned to 16 bytes")
+                                f"{MASKED_MFMA_SHAPES} (with kept positions or biases by distance "
+                                f"of {MASKED_MFMA_EXT_WIDTHS} each), at most 32 heads a kv head, "
+                                "query rows aligned to 16 bytes, output rows to 8")
     n_seqs = ctx_len.shape[0]
     max_pages = block_table.shape[1]
     keys = max_pages * page_size
     for bound in (window, chunk):
         if bound > 0:
             keys = min(keys, bound)
+    if keep > 0:                               # the kept positions' chunks, walked ahead
+        keys = min(keys + (keep + 31) // 32 * 32, max_pages * page_size)
     G = n_heads // n_kv_heads
     lib = build.load("masked_attention")
     decode = max_q_len == 1 and T == n_seqs
@@ -2350,8 +2434,9 @@ def masked_attention_mfma(q, gate, gate_mode, k_pool, v_pool, sink, block_table,
     code = lib.zf_masked_attention_mfma(
         _ptr(q), ctypes.c_longlong(qs), _ptr(gate), ctypes.c_longlong(gs), GATE_MODES[gate_mode],
         _ptr(k_pool), _ptr(v_pool), _ptr(sink), _ptr(block_table), _ptr(q_start), _ptr(ctx_len),
-        _ptr(out), _ptr(ws_o), _ptr(ws_ml), ctypes.c_float(scale), ctypes.c_float(cap),
-        int(window), int(chunk), T, n_seqs, n_tiles, n_heads, n_kv_heads, key_width, value_width,
+        _ptr(out), ctypes.c_longlong(out.stride(0)), _ptr(ws_o), _ptr(ws_ml),
+        ctypes.c_float(scale), ctypes.c_float(cap), int(window), int(chunk), int(keep),
+        _ptr(dist_bias), _distances(dist_bias), T, n_seqs, n_tiles, n_heads, n_kv_heads, key_width, value_width,
         page_size, max_pages, 1 if decode else 0, parts, wave_keys, _stream())
     _check(code, "masked_attention_mfma")
 
@@ -2534,30 +2619,166 @@ def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, z: torch
     _check(code, "decay_recurrence")
 
 
+GATE_KINDS = {"silu": 0, "sigmoid": 1}
+
+
 @_launches("norm_rope_write")
-def head_norm_gate(o: torch.Tensor, gain: torch.Tensor, gate: torch.Tensor, out: torch.Tensor,
-                   n_heads: int, eps: float) -> None:
-    """out[t, h, :] = o[t, h, :] / sqrt(mean(o[t, h, :]^2) + eps) * gain * silu(gate[t, h, :]):
-    ``o`` float32 [T, H * dv]; ``gain`` float32 [dv] (one for all heads) or [H * dv]; ``gate``
-    (contiguous rows, any row stride) and ``out`` [T, H * dv] in the products' type."""
-    _need_gpu(o, gain, out)
-    if not gate.is_cuda:
+def head_norm_gate(o: torch.Tensor, gain: Optional[torch.Tensor], gate: torch.Tensor,
+                   out: torch.Tensor, n_heads: int, eps: float, gate_kind: str = "silu") -> None:
+    """out[t, h, :] = o[t, h, :] / sqrt(mean(o[t, h, :]^2) + eps) * gain * act(gate[t, h, :]) with
+    ``gate_kind`` "silu" or "sigmoid": ``o`` float32 [T, H * dv]; ``gain`` float32 [dv] (one for
+    all heads), [H * dv] or None; ``gate`` and ``out`` [T, H * dv] (contiguous rows, any row
+    stride) in the products' type.  ``n_heads`` 1: the norm runs over the whole row."""
+    _need_gpu(o, gain)
+    if not gate.is_cuda or not out.is_cuda:
         raise KernelUnavailable("the HIP kernels run on GPU tensors only")
     T, width = o.shape
     H = int(n_heads)
     dv = width // H if H > 0 else 0
-    if H < 1 or dv * H != width or o.dtype != torch.float32 or gain.dtype != torch.float32 \
-            or gain.shape not in ((dv,), (width,)) or gate.shape != (T, width) \
-            or out.shape != (T, width) or gate.dtype != out.dtype:
+    if H < 1 or dv * H != width or o.dtype != torch.float32 or gate_kind not in GATE_KINDS \
+            or (gain is not None and (gain.dtype != torch.float32
+                                      or gain.shape not in ((dv,), (width,)))) \
+            or gate.shape != (T, width) or out.shape != (T, width) or gate.dtype != out.dtype:
         raise KernelUnavailable(f"head_norm_gate: o {tuple(o.shape)} {o.dtype}, gain "
-                                f"{tuple(gain.shape)}, gate {tuple(gate.shape)} {gate.dtype}, out "
-                                f"{tuple(out.shape)} {out.dtype}, {H} heads")
+                                f"{None if gain is None else tuple(gain.shape)}, gate "
+                                f"{tuple(gate.shape)} {gate.dtype}, out {tuple(out.shape)} "
+                                f"{out.dtype}, {H} heads, gate {gate_kind!r}")
     lib = build.load("recurrent")
-    per_head = 1 if gain.shape == (width,) and H > 1 else 0
+    per_head = 1 if gain is not None and gain.shape == (width,) and H > 1 else 0
     _check(lib.zf_head_norm_gate(_ptr(o), _ptr(gain), per_head, _ptr(gate),
                                  ctypes.c_longlong(_columns(gate, "head_norm_gate: gate")),
-                                 _ptr(out), _dt(out), T, H, dv, ctypes.c_float(eps), _stream()),
-           "head_norm_gate")
+                                 GATE_KINDS[gate_kind], _ptr(out),
+                                 ctypes.c_longlong(_columns(out, "head_norm_gate: out")), _dt(out),
+                                 T, H, dv, ctypes.c_float(eps), _stream()), "head_norm_gate")
+
+
+# ------------------------------------------------------------------------- linear attention with a fixed decay a head
+FIXED_DECAY_MAX_KEY_DIM = 256
+FIXED_DECAY_CHUNK = 128          # FC_C in fixed_decay.hip
+FIXED_DECAY_WALK_TOKENS = 32     # portions up to here run token by token in bfloat16, too
+
+
+def fixed_decay_state_size(n_heads: int, key_dim: int, value_dim: int) -> int:
+    """32-bit numbers a request's state takes: [head][value column][channels padded to 4]."""
+    return n_heads * value_dim * ((key_dim + 3) // 4 * 4)
+
+
+def fixed_decay_state_matrix(state: torch.Tensor, n_heads: int, key_dim: int,
+                             value_dim: int) -> torch.Tensor:
+    """The matrices S [.., head, key channel, value column] of states as the kernels keep them
+    (tests and inspection)."""
+    padded = (key_dim + 3) // 4 * 4
+    s = state[..., :n_heads * value_dim * padded]
+    s = s.reshape(s.shape[:-1] + (n_heads, value_dim, padded))
+    return s[..., :key_dim].transpose(-1, -2)
+
+
+@_launches("norm_rope_write")
+def rotation_table(positions: torch.Tensor, freq: torch.Tensor, mag: float,
+                   out: torch.Tensor) -> None:
+    """out[t, j] = (cos, sin) of positions[t] * freq[j] (the angle formed in 32-bit), times
+    ``mag``: float32 [T, len(freq), 2]."""
+    _need_gpu(positions, freq, out)
+    _i32(positions, "positions")
+    T, half = positions.shape[0], freq.shape[0]
+    if freq.dtype != torch.float32 or out.dtype != torch.float32 or out.shape != (T, half, 2):
+        raise KernelUnavailable(f"rotation_table: {T} positions, {tuple(freq.shape)} frequencies "
+                                f"-> {tuple(out.shape)} {out.dtype}")
+    lib = build.load("fixed_decay")
+    _check(lib.zf_rotation_table(_ptr(positions), _ptr(freq), ctypes.c_float(mag), _ptr(out), T,
+                                 half, _stream()), "rotation_table")
+
+
+def fixed_decay_chunk_lists(q_lens, longer_than: int = FIXED_DECAY_WALK_TOKENS):
+    """How a step's sequences are dealt to ``fixed_decay``'s two ways: (chunks [n, 4], firsts
+    [m, 3], shorts [s]) as int32 arrays, or None where no sequence brings more than
+    ``longer_than`` tokens.  chunks: sequence, first token (of the step), tokens, 0; firsts: a
+    long sequence, its first chunk, how many it has; shorts: the other sequences."""
+    import numpy as np
+    if max(q_lens) <= longer_than:
+        return None
+    chunks, firsts, shorts = [], [], []
+    t = 0
+    for s, n in enumerate(q_lens):
+        if n <= longer_than:
+            shorts.append(s)
+        else:
+            firsts.append((s, len(chunks), (n + FIXED_DECAY_CHUNK - 1) // FIXED_DECAY_CHUNK))
+            for c in range(0, n, FIXED_DECAY_CHUNK):
+                chunks.append((s, t + c, min(FIXED_DECAY_CHUNK, n - c), 0))
+        t += n
+    return (np.asarray(chunks, dtype=np.int32), np.asarray(firsts, dtype=np.int32),
+            np.asarray(shorts, dtype=np.int32))
+
+
+@_launches("attention")
+def fixed_decay(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor,
+                state: torch.Tensor, state_slots: torch.Tensor, q_start: torch.Tensor,
+                out: torch.Tensor, n_heads: int, key_dim: int, value_dim: int, *,
+                silu: bool = False, table: Optional[torch.Tensor] = None, k_scale: float = 1.0,
+                lists=None) -> None:
+    """S_t = g S_(t-1) + k_t v_t^T, o_t = S_t^T q_t a head, in 32-bit, over the rows of a step:
+    ``q``, ``k`` [T, >= H * d], ``v`` [T, >= H * dv] (contiguous rows, any row stride), with
+    ``decay`` float32 [2, H]: g and its base-2 logarithm.  On the way in q, k and v pass silu
+    (``silu``), then the pairs (i, i + half) of q's and k's heads turn by ``table`` float32 [T,
+    half, 2] (``rotation_table``), and k is multiplied by ``k_scale``.  ``out`` float32 [T, H *
+    dv].  Sequence s owns the rows q_start[s] .. q_start[s + 1] - 1; its state (row
+    state_slots[s] of ``state``, float32 [slots, >= ``fixed_decay_state_size``]) is read before
+    its first row and written behind its last.
+
+    ``lists`` (bfloat16 only): the int32 tensors of ``fixed_decay_chunk_lists``; long sequences
+    then run in chunks side by side through MFMAs, where an operand that is a 32-bit number
+    enters as two bfloat16 terms.  None: token by token, all 32-bit, every size and both types
+    (the same bits however a sequence is cut into steps)."""
+    _need_gpu(decay, state, state_slots, q_start, out, table)
+    for t in (q, k, v):
+        if not t.is_cuda:
+            raise KernelUnavailable("the HIP kernels run on GPU tensors only")
+    _i32(state_slots, "state_slots")
+    _i32(q_start, "q_start")
+    T = q.shape[0]
+    H, d, dv = int(n_heads), int(key_dim), int(value_dim)
+    n_seqs = state_slots.shape[0]
+    need = fixed_decay_state_size(H, d, dv)
+    half = 0 if table is None else table.shape[1]
+    if not 0 < d <= FIXED_DECAY_MAX_KEY_DIM or dv < 1 or H < 1 \
+            or q.shape[1] < H * d or k.shape[1] < H * d or v.shape[1] < H * dv \
+            or k.shape[0] != T or v.shape[0] != T or k.dtype != q.dtype or v.dtype != q.dtype \
+            or decay.shape != (2, H) or decay.dtype != torch.float32 \
+            or out.shape != (T, H * dv) or out.dtype != torch.float32 \
+            or state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] < need \
+            or state.shape[1] % 4 != 0 or q_start.shape[0] != n_seqs + 1 \
+            or (table is not None and (table.dtype != torch.float32 or half < 1 or 2 * half > d
+                                       or table.shape != (T, half, 2))) \
+            or (lists is not None and q.dtype != torch.bfloat16):
+        raise KernelUnavailable(f"fixed_decay: q {tuple(q.shape)}, k {tuple(k.shape)}, v "
+                                f"{tuple(v.shape)} {q.dtype}, out {tuple(out.shape)} {out.dtype}, "
+                                f"state {tuple(state.shape)} {state.dtype}, decay "
+                                f"{tuple(decay.shape)} for {H} heads of {d} x {dv} (key size up "
+                                f"to {FIXED_DECAY_MAX_KEY_DIM})")
+    lib = build.load("fixed_decay")
+    rows = (_ptr(q), ctypes.c_longlong(_columns(q, "fixed_decay: q")), _ptr(k),
+            ctypes.c_longlong(_columns(k, "fixed_decay: k")), _ptr(v),
+            ctypes.c_longlong(_columns(v, "fixed_decay: v")))
+    way = (_ptr(table), half, 1 if silu else 0, ctypes.c_float(k_scale))
+    shorts, n_short = None, n_seqs
+    if lists is not None:
+        chunks, firsts, shorts = lists
+        for t in (chunks, firsts, shorts):
+            if t is not None:
+                _i32(t, "fixed_decay: lists")
+        n_chunks, n_long = chunks.shape[0], firsts.shape[0]
+        n_short = 0 if shorts is None else shorts.shape[0]
+        states = _workspace("fixed_decay_states", n_chunks * need, torch.float32, q.device)
+        _check(lib.zf_fixed_decay_chunks(
+            *rows, *way, _ptr(decay[1]), _ptr(state), ctypes.c_longlong(state.shape[1]),
+            _ptr(state_slots), _ptr(chunks), n_chunks, _ptr(firsts), n_long, _ptr(states),
+            _ptr(out), H, d, dv, _stream()), "fixed_decay (chunks)")
+    if n_short:
+        _check(lib.zf_fixed_decay_walk(
+            *rows, _dt(q), *way, _ptr(decay[0]), _ptr(state), ctypes.c_longlong(state.shape[1]),
+            _ptr(state_slots), _ptr(q_start), _ptr(shorts), _ptr(out), n_short, H, d, dv,
+            _stream()), "fixed_decay (token by token)")
 
 
 # ------------------------------------------------------------------------- the residual stream in several copies

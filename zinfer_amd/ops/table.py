@@ -11,6 +11,7 @@ from typing import Callable, Dict
 
 from . import (gated_act, moe_grouped, norm_add_norm, tied_attention_mfma)
 from . import delta_recurrence, short_conv, streams_step
+from . import add_row, bias_act_rows, fixed_decay, rotation_table
 from . import (concat_rows, decay_recurrence, embed_sinusoid, head_norm_gate, token_shift_mix)
 from . import (activation, head_products, masked_attention, masked_attention_mfma,
                norm_add_store, project_rows)
@@ -118,6 +119,12 @@ KERNELS: Dict[str, KernelEntry] = {
                               "with silu and unit heads, the last rows kept as state"),
     "delta_recurrence": KernelEntry(delta_recurrence, "delta", "own: a matrix a head, decayed "
                                     "and corrected towards every token's value"),
+    "rotation_table": KernelEntry(rotation_table, "fixed_decay", "own: cosines and sines a token"),
+    "fixed_decay": KernelEntry(fixed_decay, "fixed_decay", "own: a matrix a head with one fixed "
+                               "decay a head, token by token or in chunks side by side"),
+    "bias_act_rows": KernelEntry(bias_act_rows, "elementwise", "own: an activation behind a bias "
+                                 "a column, over slices of wider rows"),
+    "add_row": KernelEntry(add_row, "elementwise", "own: one row added to every row"),
     "mfma_loop": KernelEntry(mfma_loop, "gemm",
                              "own: MFMAs alone, the rate the tiled products are measured against"),
 }

@@ -65,13 +65,15 @@ class KVNeed:
     values are narrower or wider than its keys (or that keeps one shared latent row:
     ``n_kv_heads`` 1) gets pools of its own widths; ``value_dim`` 0: the values are the keys,
     there is no value pool.  ``dtype``: what the pools hold (None: the engine's cache
-    dtype)."""
+    dtype).  ``keep_first``: the first so many positions are read by every query, however far
+    behind the window or chunk they lie: their pages stay."""
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     value_dim: Optional[int] = None
     dtype: Optional[torch.dtype] = None
     chunk: Optional[int] = None
+    keep_first: int = 0
 
     @property
     def key_width(self) -> int:
@@ -155,6 +157,14 @@ class Part:
         """The block-table width (>= ``pages``) a captured decode step should be made for, if
         the part's kernels care (their grids follow it); None: the engine's own bucket."""
         return None
+
+    # A sublayer that reads its input through one stacked matrix and writes its output through
+    # another may let a block that runs two of them on the same input join their products: it
+    # says ``joins`` and has ``input_matrices(tensors)`` (the rows of its input matrix, in order),
+    # ``output_matrix(tensors)`` ([hidden, k] and its bias [hidden] or None), ``bind_joined``
+    # (everything but those two) and ``inner(rows, out, step, *args)``, which takes its columns
+    # of the joined input product and leaves what the output matrix reads in ``out``.
+    joins = False
 
     def hint_providers(self) -> List["Part"]:
         """The parts below this one (itself included) that have hints to give."""

@@ -8,7 +8,7 @@ from ..config.specs import (ParallelBlockSpec, PostNormBlockSpec, PreNormBlockSp
                             SandwichNormBlockSpec, StreamBlockSpec)
 from ..errors import ConfigError
 from .base import Block, TensorDecl, build_part, register_part
-from .linear import place_gain
+from .linear import Linear, place_gain, place_matrix
 
 
 class PreNormBlock(Block):
@@ -276,7 +276,14 @@ class PostNormBlock(Block):
 class ParallelBlock(Block):
     """x += mixer(norm1(x)) + feed_forward(norm2(x)): both norms read the stream before either
     sublayer has added to it; the sublayers then add their outputs into the stream one after
-    the other, in 32-bit.  Without a feed-forward the block is its mixer's line."""
+    the other, in 32-bit.  Without a feed-forward the block is its mixer's line.
+
+    With one norm for both (``ff_norm`` None) the sublayers read the same rows: where both say
+    ``joins`` their input matrices lie one below the other and their output matrices side by
+    side, so that the layer is two products with what stands between them in each sublayer, and
+    the two outputs' sum is the second product's own.  Its biases are further columns of the
+    output matrix, which meet columns of ones.  The norm may then be taken apart by the products
+    around it, as in ``PreNormBlock``."""
 
     def __init__(self, spec: ParallelBlockSpec, ctx, prefix):
         super().__init__(spec, ctx, prefix)
@@ -285,11 +292,18 @@ class ParallelBlock(Block):
         self.parts = [self.mixer_norm, self.mixer]
         self.ff_norm = self.feed_forward = None
         if spec.feed_forward is not None:
-            self.ff_norm = build_part("norm", spec.ff_norm, ctx, prefix + spec.ff_norm_prefix)
+            if spec.ff_norm is not None:
+                self.ff_norm = build_part("norm", spec.ff_norm, ctx, prefix + spec.ff_norm_prefix)
+                self.parts.append(self.ff_norm)
             self.feed_forward = build_part("feed_forward", spec.feed_forward, ctx,
                                            prefix + spec.ff_prefix)
-            self.parts += [self.ff_norm, self.feed_forward]
+            self.parts.append(self.feed_forward)
         self.parts = tuple(self.parts)
+        self.joinable = self.feed_forward is not None and self.ff_norm is None \
+            and self.mixer.joins and self.feed_forward.joins
+        self.joined = None
+        # the norm that reads the stream first, if what a sum leaves for it is of use
+        self.entry_norm = self.mixer_norm if self.joinable and self.mixer_norm.defers else None
         self.graph_safe = all(p.graph_safe for p in self.parts)
         self.kernel_modules = tuple(sorted({m for p in self.parts for m in p.kernel_modules}))
 
@@ -300,8 +314,16 @@ class ParallelBlock(Block):
         return d
 
     def bind(self, tensors) -> None:
+        joined = self.joinable and JoinedProducts.fits(self.mixer, self.feed_forward, tensors)
+        self.joined = JoinedProducts(self.mixer, self.feed_forward, tensors, self.ctx) \
+            if joined else None
         for part in self.parts:
-            part.bind(tensors)
+            if joined and part is not self.mixer_norm:
+                part.bind_joined(tensors)
+            else:
+                part.bind(tensors)
+        if not joined:
+            self.entry_norm = None
 
     def cache_need(self):
         return self.mixer.cache_need()
@@ -312,17 +334,75 @@ class ParallelBlock(Block):
     def hint_providers(self):
         return [q for p in self.parts for q in p.hint_providers()]
 
+    def _forward_joined(self, x, step, cache) -> None:
+        j, act, T = self.joined, self.ctx.act_dtype, x.shape[0]
+        after = step.norm_after_block
+        left, step.norm_ready, step.norm_after = step.norm_ready, None, None
+        make = lambda: step.scratch("normed", x.shape, act)
+        h = self.mixer_norm.deferred(x, make, left if self.entry_norm is not None else None)
+        if h is None:
+            h = self.mixer_norm.forward(x, make())
+        rows = step.scratch("joined_in", (T, j.into.out_features), act)
+        j.into.forward(h, rows)
+        out = step.scratch("joined_out", (T, j.out.in_features), act)
+        self.mixer.inner(rows[:, :j.mixer_in], out[:, :j.mixer_out], step, cache)
+        self.feed_forward.inner(rows[:, j.mixer_in:j.mixer_in + j.ff_in], out[:, j.mixer_out:],
+                                step, tail=j.tail, ones=j.ones)
+        step.norm_after = after if getattr(after, "defers", False) else None
+        j.out.forward(out, x, accumulate=True, step=step)
+        step.norm_after = None
+
     def forward(self, x, step, cache) -> None:
+        if self.joined is not None:
+            self._forward_joined(x, step, cache)
+            return
         step.norm_ready = step.norm_after = None
         h1 = self.mixer_norm.forward(x, step.scratch("normed", x.shape, self.ctx.act_dtype))
-        h2 = None
-        if self.feed_forward is not None:
+        h2 = h1
+        if self.ff_norm is not None:
             # (before the mixer adds into the stream: both sublayers read the same rows)
             h2 = self.ff_norm.forward(x, step.scratch("normed_ff", x.shape, self.ctx.act_dtype))
         self.mixer.forward(h1, x, step, cache)
         if self.feed_forward is not None:
             self.feed_forward.forward(h2, x, step)
         step.norm_ready = step.norm_after = None
+
+
+class JoinedProducts:
+    """The two products of a ``ParallelBlock`` whose sublayers join: ``into`` [mixer's rows; feed-
+    forward's rows] and ``out`` [mixer's columns | feed-forward's | a column a bias | zeros], each
+    filled up with zeros to the multiple of 64 that the MFMA kernels' own order takes."""
+    ALIGN = 64
+
+    def __init__(self, mixer, feed_forward, tensors, ctx):
+        rows = [mixer.input_matrices(tensors), feed_forward.input_matrices(tensors)]
+        outs = [mixer.output_matrix(tensors), feed_forward.output_matrix(tensors)]
+        self.mixer_in, self.ff_in = (sum(m.shape[0] for m in r) for r in rows)
+        self.mixer_out = outs[0][0].shape[1]
+        self.ones = sum(b is not None for _, b in outs)
+        n, k = self.mixer_in + self.ff_in, self.mixer_out + outs[1][0].shape[1]
+        self.tail = -(-(k + self.ones) // self.ALIGN) * self.ALIGN - k
+        into = rows[0] + rows[1]
+        pad = -n % self.ALIGN
+        if pad:
+            into.append(into[0].new_zeros((pad, into[0].shape[1])))
+        self.into = Linear(place_matrix(torch.cat(into, dim=0), ctx))
+        columns = [m for m, _ in outs] + [b.to(outs[0][0].dtype)[:, None]
+                                          for _, b in outs if b is not None]
+        if self.tail > self.ones:
+            columns.append(outs[0][0].new_zeros((outs[0][0].shape[0], self.tail - self.ones)))
+        self.out = Linear(place_matrix(torch.cat(columns, dim=1).contiguous(), ctx))
+
+    @staticmethod
+    def fits(mixer, feed_forward, tensors) -> bool:
+        """Whether the matrices are stored in one type, and the biases are exact in it."""
+        outs = [mixer.output_matrix(tensors), feed_forward.output_matrix(tensors)]
+        matrices = mixer.input_matrices(tensors) + feed_forward.input_matrices(tensors) \
+            + [m for m, _ in outs]
+        if len({m.dtype for m in matrices}) > 1:
+            return False
+        kind = torch.bfloat16 if matrices[0].dtype == torch.float16 else matrices[0].dtype
+        return all(b is None or torch.equal(b.to(kind).double(), b.double()) for _, b in outs)
 
 
 class StreamRead:

@@ -5,8 +5,9 @@ from typing import Dict
 import torch
 
 from .. import ops
+from ..config.distance import bucket_of_distances
 from ..config.specs import LatentAttentionSpec, MaskedGqaAttentionSpec
-from ..errors import ConfigError
+from ..errors import ConfigError, StepError
 from .base import KVNeed, Mixer, TensorDecl, register_part
 from .linear import Linear, place_gain, place_matrix
 
@@ -16,6 +17,15 @@ def _frequencies(rotary, ctx):
     if rotary is None:
         return None
     return torch.tensor(rotary.frequencies, dtype=torch.float64).to(torch.float32).to(ctx.device)
+
+
+def finish(linear, bias, rows, residual, accumulate: bool, step) -> None:
+    """A sublayer's output product into the residual stream or branch, its bias behind it (the
+    norm that reads the stream next can only take what a sum leaves when nothing follows it)."""
+    linear.forward(rows, residual, accumulate=accumulate,
+                   step=step if accumulate and bias is None else None)
+    if bias is not None:
+        ops.add_row(residual, bias)
 
 
 def _check_mask(spec) -> None:
@@ -31,11 +41,14 @@ class MaskedGqaAttention(Mixer):
     its own dot product); one kernel norms q and k over their whole projections, rotates the
     leading elements of every head by the token's position, and stores the token's key and
     value rows in the cache; the attention kernel caps the scores, keeps to the query's chunk
-    or window, counts the head's sink in the denominator and multiplies by the head's gate.
+    or window, adds the distance's bias, counts the head's sink in the denominator and multiplies
+    by the head's gate.  Values that are mixed with an earlier layer's are mixed on their way
+    into the cache (``step.shared["values"]`` holds the source's rows).
     Norms, angles, scores, weights and their sums are 32-bit in both dtypes."""
     graph_safe = True
     stores_output = True
-    kernel_modules = ("gemm", "masked_attention")
+    joins = True
+    kernel_modules = ("elementwise", "gemm", "masked_attention")
 
     def __init__(self, spec: MaskedGqaAttentionSpec, ctx, prefix):
         super().__init__(spec, ctx, prefix)
@@ -51,6 +64,12 @@ class MaskedGqaAttention(Mixer):
                                          and len(s.rotary.frequencies) == s.rotary.dims // 2):
             raise ConfigError(f"a rotation of {s.rotary.dims} elements does not fit heads of "
                               f"{s.head_dim}")
+        if s.qk_norm_eps is not None and s.qk_unit_eps is not None:
+            raise ConfigError("q and k are normed with a gain or without one, not both")
+        if s.keep_first < 0:
+            raise ConfigError(f"keep_first={s.keep_first} must not be negative")
+        if s.value_mix not in (None, "idle", "source", "blend"):
+            raise ConfigError(f"value_mix={s.value_mix!r}: 'idle', 'source', 'blend' or None")
         _check_mask(s)
         self.q_width = s.n_heads * s.head_dim
         self.k_width = s.n_kv_heads * s.head_dim
@@ -75,17 +94,36 @@ class MaskedGqaAttention(Mixer):
             d[p + s.sink_name] = TensorDecl((s.n_heads,))
         if s.head_gate:
             d[p + s.gate_name] = TensorDecl((s.n_heads, s.hidden_size))
+        if s.distance_bias is not None:
+            d[p + s.distance_bias.name] = TensorDecl((s.distance_bias.buckets, s.n_heads), free=32)
+        if s.output_bias:
+            d[p + s.o_name + s.bias_suffix] = TensorDecl((s.hidden_size,))
+        if s.value_mix is not None:
+            d[p + s.value_mix_name] = TensorDecl((), optional=s.value_mix != "blend")
         return d
 
-    def bind(self, tensors) -> None:
+    def input_matrices(self, tensors):
         s, p = self.spec, self.prefix
-        rows = [tensors[p + s.q_name], tensors[p + s.k_name], tensors[p + s.v_name]]
-        if s.head_gate:
-            rows.append(tensors[p + s.gate_name])
+        names = [s.q_name, s.k_name, s.v_name] + ([s.gate_name] if s.head_gate else [])
+        return [tensors[p + n] for n in names]
+
+    def output_matrix(self, tensors):
+        s, p = self.spec, self.prefix
+        return tensors[p + s.o_name], \
+            tensors[p + s.o_name + s.bias_suffix] if s.output_bias else None
+
+    def bind(self, tensors) -> None:
+        rows = self.input_matrices(tensors)
         if len({t.dtype for t in rows}) > 1:
             rows = [t.float() for t in rows]
         self.proj = Linear(place_matrix(torch.cat(rows, dim=0), self.ctx))
-        self.o = Linear(place_matrix(tensors[p + s.o_name], self.ctx))
+        o, bias = self.output_matrix(tensors)
+        self.o = Linear(place_matrix(o, self.ctx))
+        self.o_bias = place_gain(bias, self.ctx) if bias is not None else None
+        self.bind_joined(tensors)
+
+    def bind_joined(self, tensors) -> None:
+        s, p = self.spec, self.prefix
         self.q_gain = self.k_gain = self.sink = None
         self.q_bias = self.k_bias = self.v_bias = None
         if s.bias:
@@ -95,12 +133,24 @@ class MaskedGqaAttention(Mixer):
         if s.qk_norm_eps is not None:
             self.q_gain = place_gain(tensors[p + s.q_norm_name], self.ctx)
             self.k_gain = place_gain(tensors[p + s.k_norm_name], self.ctx)
+        elif s.qk_unit_eps is not None:
+            # a norm a head whose gain is 1
+            self.q_gain = self.k_gain = place_gain(torch.ones(s.head_dim), self.ctx)
         if s.sink:
             self.sink = place_gain(tensors[p + s.sink_name], self.ctx)
+        self.dist_bias = None
+        if s.distance_bias is not None:
+            table = tensors[p + s.distance_bias.name].to(torch.float32)
+            rows = bucket_of_distances(table.shape[0], s.distance_bias.far)
+            by_distance = table[torch.tensor(rows, dtype=torch.long, device=table.device)]
+            self.dist_bias = ops.distance_table(by_distance.T.contiguous()).to(self.ctx.device)
+        self.mix_share = float(tensors[p + s.value_mix_name]) if s.value_mix == "blend" else 0.0
 
     def cache_need(self):
         s = self.spec
-        return KVNeed(s.n_kv_heads, s.head_dim, s.window, value_dim=s.value_dim, chunk=s.chunk)
+        bounded = s.window is not None or s.chunk is not None
+        return KVNeed(s.n_kv_heads, s.head_dim, s.window, value_dim=s.value_dim, chunk=s.chunk,
+                      keep_first=s.keep_first if bounded else 0)
 
     def accept_cache(self, cache) -> None:
         for pool in (cache.k_pool, cache.v_pool):
@@ -114,14 +164,31 @@ class MaskedGqaAttention(Mixer):
         act = self.ctx.act_dtype
         if hasattr(h, "materialize"):
             h = h.materialize()
-        kv = step.kv_tables(cache.group)
         proj = step.scratch("qkvg", (T, self.proj.out_features), act)
         self.proj.forward(h, proj)
+        attn = step.scratch("attn", (T, s.n_heads * s.value_dim), act)
+        self.inner(proj, attn, step, cache)
+        finish(self.o, self.o_bias, attn, residual, accumulate, step)
+
+    def inner(self, proj, attn, step, cache) -> None:
+        """From the rows [q | k | v | head gates] of the input product to the heads' outputs."""
+        s = self.spec
+        T = proj.shape[0]
+        act = self.ctx.act_dtype
+        kv = step.kv_tables(cache.group)
         q = step.scratch("q", (T, self.q_width), act)
-        eps = float(s.qk_norm_eps) if s.qk_norm_eps is not None else 0.0
+        eps = s.qk_norm_eps if s.qk_norm_eps is not None else s.qk_unit_eps
+        eps = float(eps) if eps is not None else 0.0
         rot = dict(rot_dims=s.rotary.dims, freq=self.freq, mag=s.rotary.magnitude,
                    interleaved=s.rotary.interleaved) if s.rotary is not None else {}
-        per = dict(per_head=s.qk_norm_per_head)
+        per = dict(per_head=s.qk_norm_per_head or s.qk_unit_eps is not None)
+        blend = None
+        if s.value_mix == "blend":
+            source = step.shared.get("values")
+            if source is None or source.shape != (T, self.v_width):
+                raise StepError(f"{self.prefix}: this layer mixes its values with an earlier "
+                                "layer's, which has not run on these tokens")
+            blend = (source, self.mix_share)
         segments = [ops.RowSegment(0, self.q_width, q, gain=self.q_gain, eps=eps, hd=s.head_dim,
                                    bias=self.q_bias, **per, **rot)]
         if cache.writes:
@@ -131,17 +198,24 @@ class MaskedGqaAttention(Mixer):
                                            **rot))
             segments.append(ops.RowSegment(self.q_width + self.k_width, self.v_width, cache.v_pool,
                                            hd=s.value_dim, pool_heads=s.n_kv_heads,
-                                           bias=self.v_bias))
+                                           bias=self.v_bias, blend=blend))
+        if s.value_mix == "source":
+            values = step.scratch("source_values", (T, self.v_width), act)
+            segments.append(ops.RowSegment(self.q_width + self.k_width, self.v_width, values,
+                                           hd=s.value_dim, bias=self.v_bias))
+            step.shared["values"] = values
         ops.project_rows(proj, step.positions, kv.slot_mapping if cache.writes else None,
                          cache.page_size, segments)
-        gate = proj[:, self.q_width + self.k_width + self.v_width:] if s.head_gate else None
-        attn = step.scratch("attn", (T, s.n_heads * s.value_dim), act)
+        gate = None
+        if s.head_gate:
+            at = self.q_width + self.k_width + self.v_width
+            gate = proj[:, at:at + s.n_heads]
         ops.attend_masked(q, gate, "head" if s.head_gate else None, cache.k_pool, cache.v_pool,
                           self.sink, kv.block_table, step.q_start, step.ctx_len, step.seq_index,
                           attn, float(s.scale), float(s.softcap or 0.0), int(s.window or 0),
                           int(s.chunk or 0), s.n_heads, s.n_kv_heads, s.head_dim, s.value_dim,
-                          cache.page_size, step.max_q_len, step.max_ctx_len)
-        self.o.forward(attn, residual, accumulate=accumulate, step=step if accumulate else None)
+                          cache.page_size, step.max_q_len, step.max_ctx_len,
+                          keep=s.keep_first, dist_bias=self.dist_bias)
 
 
 class LatentAttention(Mixer):

@@ -7,7 +7,7 @@ import torch
 from .. import ops
 from ..config.specs import DenseMlpSpec, SwiGluSpec
 from .base import FeedForward, TensorDecl, register_part
-from .linear import Linear, place_matrix
+from .linear import Linear, place_gain, place_matrix
 
 
 class SwiGluMlp(FeedForward):
@@ -69,32 +69,63 @@ class _probe:
 
 
 class DenseMlp(FeedForward):
-    """d = W_down act(W_up m), no gate; the activation (``ops.ACTIVATIONS``) runs in 32-bit on
-    the product's values."""
+    """d = W_down act(W_up m), no gate, with biases if the specification says so; bias and
+    activation (``ops.ACTIVATIONS``) run in 32-bit on the product's values."""
     graph_safe = True
     stores_output = True
+    joins = True
     kernel_modules = ("elementwise", "gemm")
 
     def declare(self) -> Dict[str, TensorDecl]:
         s, p = self.spec, self.prefix
-        return {p + s.up_name: TensorDecl((s.intermediate_size, s.hidden_size)),
-                p + s.down_name: TensorDecl((s.hidden_size, s.intermediate_size))}
+        d = {p + s.up_name: TensorDecl((s.intermediate_size, s.hidden_size)),
+             p + s.down_name: TensorDecl((s.hidden_size, s.intermediate_size))}
+        if s.bias:
+            d[p + s.up_name + s.bias_suffix] = TensorDecl((s.intermediate_size,))
+            d[p + s.down_name + s.bias_suffix] = TensorDecl((s.hidden_size,))
+        return d
 
-    def bind(self, tensors) -> None:
+    def input_matrices(self, tensors):
+        return [tensors[self.prefix + self.spec.up_name]]
+
+    def output_matrix(self, tensors):
+        s, p = self.spec, self.prefix
+        return tensors[p + s.down_name], \
+            tensors[p + s.down_name + s.bias_suffix] if s.bias else None
+
+    def bind_joined(self, tensors) -> None:
         s, p = self.spec, self.prefix
         if s.activation not in ops.ACTIVATIONS:
             from ..errors import ConfigError
             raise ConfigError(f"activation {s.activation!r}: known are {sorted(ops.ACTIVATIONS)}")
-        self.up = Linear(place_matrix(tensors[p + s.up_name], self.ctx))
-        self.down = Linear(place_matrix(tensors[p + s.down_name], self.ctx))
+        self.up_bias = place_gain(tensors[p + s.up_name + s.bias_suffix], self.ctx) \
+            if s.bias else None
+
+    def bind(self, tensors) -> None:
+        self.up = Linear(place_matrix(self.input_matrices(tensors)[0], self.ctx))
+        down, bias = self.output_matrix(tensors)
+        self.down = Linear(place_matrix(down, self.ctx))
+        self.down_bias = place_gain(bias, self.ctx) if bias is not None else None
+        self.bind_joined(tensors)
 
     def forward(self, h, residual, step, accumulate: bool = True) -> None:
         if hasattr(h, "materialize"):
             h = h.materialize()
         a = step.scratch("ff_act", (h.shape[0], self.spec.intermediate_size), self.ctx.act_dtype)
         self.up.forward(h, a)
-        ops.activation(a, a, self.spec.activation)
-        self.down.forward(a, residual, accumulate=accumulate, step=step if accumulate else None)
+        if self.up_bias is None:
+            ops.activation(a, a, self.spec.activation)
+        else:
+            ops.bias_act_rows(a, self.up_bias, a, self.spec.activation)
+        self.down.forward(a, residual, accumulate=accumulate,
+                          step=step if accumulate and self.down_bias is None else None)
+        if self.down_bias is not None:
+            ops.add_row(residual, self.down_bias)
+
+    def inner(self, rows, out, step, tail: int = 0, ones: int = 0) -> None:
+        """Bias and activation from the input product's columns to what the output product reads;
+        the last ``tail`` columns of ``out`` become ones and zeros (``ops.bias_act_rows``)."""
+        ops.bias_act_rows(rows, self.up_bias, out, self.spec.activation, tail=tail, ones=ones)
 
 
 register_part("feed_forward", SwiGluSpec, SwiGluMlp)

@@ -24,10 +24,10 @@ class RmsNorm(Norm):
 
 
     def declare(self) -> Dict[str, TensorDecl]:
-        return {self.prefix + "weight": TensorDecl((self.spec.width,), init="gain")}
+        return {self.prefix + self.spec.weight_name: TensorDecl((self.spec.width,), init="gain")}
 
     def bind(self, tensors) -> None:
-        self.gain = place_gain(tensors[self.prefix + "weight"], self.ctx)
+        self.gain = place_gain(tensors[self.prefix + self.spec.weight_name], self.ctx)
 
     def forward(self, x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
         ops.rmsnorm(x, self.gain, float(self.spec.eps), out)
