@@ -175,9 +175,11 @@ def retention_mixer(h, w, m: dict, eps: float) -> torch.Tensor:
     h = h.to(F64)
     T = h.shape[0]
     p = torch.arange(T)
-    dims, base = int(m["rot"]["dims"]), float(m["rot"]["base"])
-    q = rotate(linear(w["q"], h).view(T, H, d), p, dims, base)
-    k = rotate(linear(w["k"], h).view(T, H, d), p, dims, base) * d ** -0.5
+    q, k = linear(w["q"], h).view(T, H, d), linear(w["k"], h).view(T, H, d)
+    if m.get("rot") is not None:
+        dims, base = int(m["rot"]["dims"]), float(m["rot"]["base"])
+        q, k = rotate(q, p, dims, base), rotate(k, p, dims, base)
+    k = k * d ** -0.5
     o, _ = decayed_sums(q, k, linear(w["v"], h).view(T, H, dv), m["decay"])
     o = unit_rms(o, eps).reshape(T, H * dv)
     return linear(w["o"], o * silu(linear(w["g"], h)))

@@ -46,7 +46,7 @@ def draw_tensor(name: str, decl: TensorDecl, seed: int, dtype: torch.dtype,
         from .. import ops
         out = torch.empty((n,), dtype=dtype, device=device)
         ops.randinit(out, key, 0, decl.init, STD)
-        return out.view(*shape)
+        return out.view(shape)
     out = torch.empty((n,), dtype=dtype)
     for lo in range(0, n, _CHUNK):            # in pieces: a big matrix never exists in 64-bit
         m = min(_CHUNK, n - lo)
@@ -56,7 +56,7 @@ def draw_tensor(name: str, decl: TensorDecl, seed: int, dtype: torch.dtype,
             out[lo:lo + m] = torch.from_numpy(bits).view(torch.bfloat16)
         else:
             out[lo:lo + m] = torch.from_numpy(piece)
-    return out.view(*shape)
+    return out.view(shape)
 
 
 class DrawnTensors(Mapping):
