@@ -23,8 +23,8 @@ intermediate 25600; 65.5 GB of weights): a 2048-token prefill, then decode at ba
 64 with every request's context just below 8192 tokens; the cache pool is sized for
 64 x 8192 tokens (137 GB).
 
-``--workload fezupel``, ``--workload lodenex``, ``--workload nupovik`` and ``--workload kugisun``: shapes of those
-designs at layer sizes that resemble served models, each beside the dense Qwen3 decoder of equal
+``--workload fezupel``, ``--workload lodenex``, ``--workload nupovik``, ``--workload kugisun`` and
+``--workload fumanex``: shapes of those designs at layer sizes that resemble served models, each beside the dense Qwen3 decoder of equal
 size (prefill of 2048 tokens, decode at batch 8), and their kernels alone beside the like
 kernels of that decoder.
 
@@ -1598,11 +1598,284 @@ def main_kugisun(args) -> int:
     return 0
 
 
+# --------------------------------------------------------------------------- Fumanex beside Qwen3
+# Layer sizes that resemble served models of this kind: attention heads of 128 behind a window of
+# 1024 with kept first positions, retention and lightning heads of 128 x 128, feed-forwards four
+# times the width.  Every shape is run beside the dense Qwen3 decoder of the same width, depth,
+# vocabulary and attention heads whose gated feed-forward does the same matrix work a token; the
+# new kernels alone stand beside the like kernels of that decoder, of Lodenex (the closest
+# attention: a cap, a sink, a window) and of Nupovik (the closest recurrence: its gated linear
+# attention at the same heads).
+def _fx_attention(heads, kv, window):
+    return ("attention", dict(heads=heads, kv_heads=kv, dim=128, vdim=128, scale=128 ** -0.5,
+                              softcap=30.0, bias_max=256, v_mix=True,
+                              mask=None if window is None else dict(size=window, keep_first=4)))
+
+
+def _fx_recurrent(kind, heads, dim=128):
+    m = dict(heads=heads, dim=dim, vdim=dim,
+             decay=[1.0 - 2.0 ** (-4.0 - 5.0 * i / max(1, heads - 1)) for i in range(heads)])
+    if kind == "retention":
+        m["rot"] = dict(dims=dim, base=10000.0)
+    return (kind, m)
+
+
+FUMANEX_SHAPES = {
+    "medium": dict(width=2048, vocab=32768, heads=16, kv_heads=4, ff=8192, layers=[
+        _fx_attention(16, 4, 1024), _fx_recurrent("retention", 16),
+        _fx_recurrent("lightning", 32, 64), _fx_attention(16, 4, 1024)]),
+    "wide": dict(width=4096, vocab=32768, heads=32, kv_heads=8, ff=16384, layers=[
+        _fx_attention(32, 8, 1024), _fx_recurrent("retention", 32),
+        _fx_recurrent("lightning", 32), _fx_attention(32, 8, None)]),
+}
+
+
+def fumanex_config(sh: dict) -> dict:
+    return {"architecture": "Fumanex", "vocab": sh["vocab"], "width": sh["width"],
+            "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "logit_scale": 1.0,
+            "layers": [{"type": kind, "mixer": dict(m), "mlp": {"kind": "dense", "ff": sh["ff"]}}
+                       for kind, m in sh["layers"]]}
+
+
+def fumanex_twin(sh: dict, max_positions: int) -> dict:
+    return dict(architectures=["Qwen3ForCausalLM"], model_type="qwen3",
+                num_hidden_layers=len(sh["layers"]), hidden_size=sh["width"],
+                num_attention_heads=sh["heads"], num_key_value_heads=sh["kv_heads"], head_dim=128,
+                intermediate_size=sh["ff"] * 2 // 3 // 64 * 64, vocab_size=sh["vocab"],
+                rope_theta=1000000.0, rms_norm_eps=1e-6, tie_word_embeddings=False,
+                max_position_embeddings=max_positions, torch_dtype="bfloat16")
+
+
+def fumanex_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float) -> dict:
+    """The new design's kernels alone beside the like kernels of other designs, at ``T`` tokens of
+    one sequence that holds ``ctx`` tokens (T = ctx: a prompt; T = 1 x 8 sequences: a decode step).
+    Every figure has the fraction of its roofline it reaches: the larger of the matrix work at the
+    MFMA loop's rate and the bytes at the measured read stream, over the time.  (Nupovik's
+    recurrence has no matrix form; its work is counted against the 32-bit vector rate.)"""
+    import torch
+    import zinfer_amd.ops as ops
+    dev = "cuda:0"
+    W, nH, nKV, hd, ff = sh["width"], sh["heads"], sh["kv_heads"], 128, sh["ff"]
+    bf = torch.bfloat16
+    decode = T == 1
+    n_seqs = 8 if decode else 1
+    rows = n_seqs * T
+    g = torch.Generator(device=dev).manual_seed(1)
+    rnd = lambda *shape: (torch.randn(shape, generator=g, device=dev) * 0.05).to(bf)
+    i32 = lambda a: torch.tensor(a, dtype=torch.int32, device=dev)
+    pages = (ctx + PAGE - 1) // PAGE
+    table = torch.arange(n_seqs * pages, dtype=torch.int32, device=dev).view(n_seqs, pages)
+    q_start = i32([i * T for i in range(n_seqs + 1)])
+    ctx_len = i32([ctx] * n_seqs)
+    seq_index = i32([i for i in range(n_seqs) for _ in range(T)])
+    positions = i32([ctx - T + t for _ in range(n_seqs) for t in range(T)])
+    slots = i32([(s * pages) * PAGE + ctx - T + t for s in range(n_seqs) for t in range(T)])
+    state_slots = i32(list(range(n_seqs)))
+    out = {}
+
+    def roof(t, flops, nbytes, rate=mfma_rate):
+        return round(max(flops / rate, nbytes / read_bw) / t, 4)
+
+    def row(name, t_new, flops, nbytes, **like):
+        r = {"fumanex_us": round(t_new * 1e6, 1), "fumanex_frac": roof(t_new, flops, nbytes)}
+        for label, (t, fl, nb, *rate) in like.items():
+            r[label + "_us"] = round(t * 1e6, 1)
+            r[label + "_frac"] = roof(t, fl, nb, *rate)
+        out[name] = r
+
+    # ---- attention, with the shape's window and without one
+    q = rnd(rows, nH * hd)
+    k_pool, v_pool = rnd(n_seqs * pages, nKV * PAGE * hd), rnd(n_seqs * pages, nKV * PAGE * hd)
+    o = torch.empty((rows, nH * hd), dtype=bf, device=dev)
+    sink = torch.zeros((nH,), device=dev)
+    gate = rnd(rows, nH)
+    from zinfer_amd.config.distance import bucket_of_distances
+    n_dist = len(bucket_of_distances(32, 256))
+    bias = ops.distance_table(torch.randn((nH, n_dist), generator=g, device=dev))
+    for name, window in (("attention_window", 1024), ("attention_full", 0)):
+        if decode:
+            seen = n_seqs * (min(ctx, window) if window else ctx)
+            work = (0.0, seen * nKV * 2 * hd * 2)
+        else:
+            w = min(window or T, T)
+            seen = w * (w + 1) // 2 + (T - w) * w
+            work = (4.0 * seen * hd * nH, rows * (nH + nKV) * 2 * hd * 2)
+        t_new = _timed_graph(lambda: ops.attend_masked(
+            q, None, None, k_pool, v_pool, sink, table, q_start, ctx_len, seq_index, o, hd ** -0.5,
+            30.0, window, 0, nH, nKV, hd, hd, PAGE, T, ctx, keep=4 if window else 0, dist_bias=bias))
+        t_lx = _timed_graph(lambda: ops.attend_masked(
+            q, gate, "head", k_pool, v_pool, sink, table, q_start, ctx_len, seq_index, o, hd ** -0.5,
+            30.0, window, 0, nH, nKV, hd, hd, PAGE, T, ctx))
+        t_q3 = _timed_graph(lambda: ops.paged_attention(
+            q, k_pool, v_pool, table, q_start, ctx_len, seq_index, o, hd ** -0.5, window, nH, nKV,
+            hd, PAGE, T, ctx))
+        row(name, t_new, *work, lodenex=(t_lx, *work), qwen3=(t_q3, *work))
+    # ---- a projection's rows: biases, unit norms a head, blended values, into the cache
+    width = (nH + 2 * nKV) * hd
+    proj = rnd(rows, width)
+    b = torch.randn((width,), generator=g, device=dev)
+    bq, bk, bv = (t.contiguous() for t in b.split([nH * hd, nKV * hd, nKV * hd]))
+    ones = torch.ones((hd,), device=dev)
+    first = rnd(rows, nKV * hd)
+    unit = dict(gain=ones, eps=1e-6, hd=hd, per_head=True)
+    segs = [ops.RowSegment(0, nH * hd, q, bias=bq, **unit),
+            ops.RowSegment(nH * hd, nKV * hd, k_pool, bias=bk, pool_heads=nKV, **unit),
+            ops.RowSegment((nH + nKV) * hd, nKV * hd, v_pool, hd=hd, bias=bv, pool_heads=nKV,
+                           blend=(first, 0.5))]
+    t_new = _timed_graph(lambda: ops.project_rows(proj, positions, slots, PAGE, segs))
+    freq = torch.rand((hd // 4,), generator=g, device=dev)
+    gq, gk = torch.ones((nH * hd,), device=dev), torch.ones((nKV * hd,), device=dev)
+    lsegs = [ops.RowSegment(0, nH * hd, q, gain=gq, eps=1e-6, hd=hd, rot_dims=hd // 2, freq=freq),
+             ops.RowSegment(nH * hd, nKV * hd, k_pool, gain=gk, eps=1e-6, hd=hd, rot_dims=hd // 2,
+                            freq=freq, pool_heads=nKV),
+             ops.RowSegment((nH + nKV) * hd, nKV * hd, v_pool, hd=hd, pool_heads=nKV)]
+    t_lx = _timed_graph(lambda: ops.project_rows(proj, positions, slots, PAGE, lsegs))
+    cos = torch.rand((ctx + 1, hd // 2), generator=g, device=dev)
+    t_q3 = _timed_graph(lambda: ops.qk_norm_rope_kv_write(
+        proj, ones, ones, 1e-6, cos, cos, positions, slots, k_pool, v_pool, q, nH, nKV, hd, PAGE))
+    work = (0.0, rows * width * 4)
+    row("norm_blend_store", t_new, 0.0, rows * (width * 4 + nKV * hd * 2), lodenex=(t_lx, *work),
+        qwen3=(t_q3, *work))
+    # ---- the recurrences and what follows them
+    for kind, m in {k: m for k, m in sh["layers"] if k != "attention"}.items():
+        H, d, dv = m["heads"], m["dim"], m["vdim"]
+        wide = rnd(rows, 2 * H * d + 2 * H * dv)
+        qk = (wide[:, :H * d], wide[:, H * d:2 * H * d], wide[:, 2 * H * d:2 * H * d + H * dv])
+        size = ops.fixed_decay_state_size(H, d, dv)
+        state = torch.zeros((n_seqs, size), dtype=torch.float32, device=dev)
+        dec = torch.tensor(m["decay"], dtype=torch.float64)
+        decay = torch.stack([dec, dec.log2()]).float().to(dev)
+        rot = None
+        if kind == "retention":
+            rot = torch.empty((rows, d // 2, 2), device=dev)
+            ops.rotation_table(positions, torch.rand((d // 2,), generator=g, device=dev), 1.0, rot)
+        lists = ops.fixed_decay_chunk_lists([T] * n_seqs)
+        if lists is not None:
+            lists = tuple(torch.from_numpy(t).to(dev) if t.size else None for t in lists)
+        ro = torch.empty((rows, H * dv), dtype=torch.float32, device=dev)
+        t_new = _timed_graph(lambda: ops.fixed_decay(
+            *qk, decay, state, state_slots, q_start, ro, H, d, dv, silu=kind == "lightning",
+            table=rot, k_scale=d ** -0.5, lists=lists))
+        z = torch.randn((rows, H * d), generator=g, device=dev)
+        zb = torch.zeros((H * d,), device=dev)
+        old = torch.zeros((n_seqs, ops.recurrence_state_size(H, d, dv)), device=dev)
+        t_np = _timed_graph(lambda: ops.decay_recurrence(
+            *qk, z, zb, None, old, state_slots, q_start, ro, H, d, dv, "sigmoid_root", tau=16.0,
+            q_scale=d ** -0.5, max_q_len=T))
+        if decode:
+            work = (0.0, 2.0 * n_seqs * H * d * dv * 4)
+            row(kind + "_recurrence", t_new, *work, nupovik=(t_np, *work))
+        else:
+            # state read and grown (4 d dv a token and head), a chunk of 128's own pairs
+            flops = rows * H * (4.0 * d * dv + 128.0 * (d + dv))
+            nbytes = rows * H * ((2 * d + dv) * 2 + dv * 4)
+            row(kind + "_recurrence", t_new, flops, nbytes,
+                nupovik=(t_np, 5.0 * rows * H * d * dv, 0.0, PEAK_FLOPS["fp32"]))
+        mixed = torch.empty((rows, H * dv + 64), dtype=bf, device=dev)[:, :H * dv]
+        gt = wide[:, 2 * H * d + H * dv:]
+        gain = torch.ones((H * dv,), device=dev)
+        head = kind == "retention"
+        t_new = _timed_graph(lambda: ops.head_norm_gate(
+            ro, None if head else gain, gt, mixed, H if head else 1, 1e-6,
+            gate_kind="silu" if head else "sigmoid"))
+        dense = torch.empty((rows, H * dv), dtype=bf, device=dev)
+        t_np = _timed_graph(lambda: ops.head_norm_gate(ro, gain[:dv], gt, dense, H, 1e-6))
+        work = (0.0, rows * H * dv * (4 + 2 + 2))
+        row(kind + "_norm_gate", t_new, *work, nupovik=(t_np, *work))
+    # ---- the layer's two joined products with bias and activation between, beside the dense
+    # decoder's four products
+    n_in, k_out = width + ff, nH * hd + ff + 64
+    w_in, w_out = ops.pretile_weight(rnd(n_in, W)), ops.pretile_weight(rnd(W, k_out))
+    h, x = rnd(rows, W), torch.zeros((rows, W), dtype=torch.float32, device=dev)
+    y, a = torch.empty((rows, n_in), dtype=bf, device=dev), torch.empty((rows, k_out), dtype=bf, device=dev)
+    up_b = torch.randn((ff,), generator=g, device=dev)
+
+    def joined():
+        ops.gemm(h, w_in, y, w_tiled=True)
+        ops.bias_act_rows(y[:, width:], up_b, a[:, nH * hd:], "gelu_tanh", tail=64, ones=2)
+        ops.gemm(a, w_out, x, accumulate=True, w_tiled=True)
+    t_new = _timed_graph(joined)
+    t_act = _timed_graph(lambda: ops.bias_act_rows(y[:, width:], up_b, a[:, nH * hd:], "gelu_tanh",
+                                                   tail=64, ones=2))
+    inter = ff * 2 // 3 // 64 * 64
+    w_qkv, w_o = ops.pretile_weight(rnd(width, W)), ops.pretile_weight(rnd(W, nH * hd))
+    w_gu = ops.pretile_weight(ops.interleave_gate_up(rnd(inter, W), rnd(inter, W)))
+    w_d = ops.pretile_weight(rnd(W, inter))
+    qkv, a2 = torch.empty((rows, width), dtype=bf, device=dev), torch.empty((rows, inter), dtype=bf, device=dev)
+
+    def apart():
+        ops.gemm(h, w_qkv, qkv, w_tiled=True)
+        ops.gemm(q, w_o, x, accumulate=True, w_tiled=True)
+        ops.gemm_swiglu(h, w_gu, a2, w_tiled=True)
+        ops.gemm(a2, w_d, x, accumulate=True, w_tiled=True)
+    t_q3 = _timed_graph(apart)
+    new_n, old_n = W * (n_in + k_out - 64), W * (width + nH * hd + 3 * inter)
+    row("joined_products", t_new, 2.0 * rows * new_n, 2.0 * new_n,
+        qwen3=(t_q3, 2.0 * rows * old_n, 2.0 * old_n))
+    t_lx = _timed_graph(lambda: ops.activation(y, y, "gelu_tanh"))
+    row("bias_act", t_act, 0.0, rows * ff * 4, lodenex=(t_lx, 0.0, rows * n_in * 4))
+    return out
+
+
+def main_fumanex(args) -> int:
+    """Prefill and decode throughput of Fumanex shapes beside the dense Qwen3 decoder of equal
+    size, and the new kernels alone beside the like kernels of other designs."""
+    import torch
+    import zinfer_amd.ops as ops
+    from zinfer_amd.config import entry_for
+    T, batch, prompt = args.prefill_tokens, args.batch, args.prompt_len
+    max_positions = max(T, prompt + args.steps + args.warmup + 64) + 64
+    read_bw = ops.measure_read_bandwidth("cuda:0")
+    mfma_rate = ops.measure_mfma_rate("cuda:0")
+    names = [args.fumanex_shape] if args.fumanex_shape else list(FUMANEX_SHAPES)
+    shapes = {}
+    for name in names:
+        sh = FUMANEX_SHAPES[name]
+        row = {"sizes": {"width": sh["width"], "vocab": sh["vocab"], "ff": sh["ff"],
+                         "layers": [[k, {n: v for n, v in m.items() if n != "decay"}]
+                                    for k, m in sh["layers"]]}}
+        for label, raw in (("fumanex", fumanex_config(sh)), ("qwen3", fumanex_twin(sh, max_positions))):
+            cfg = entry_for(raw).config_type.from_dict(raw)
+            pool = batch * (prompt + args.steps + args.warmup + 64) + T + 256
+            llm = build_llm(raw, args.dtype, args.seed, pool, max(batch, 8),
+                            max_step_tokens=max(T, 2048), multi_step=args.multi_step)
+            t_pre = run_prefill(llm, cfg, T, args.seed + 1)
+            dt, mean_ctx = run_decode(llm, cfg, batch, prompt, args.steps, args.warmup, args.seed + 2)
+            row[label] = {"prefill_tokens_per_s": round(T / t_pre, 1), "prefill_ms": round(t_pre * 1e3, 3),
+                          "decode_tokens_per_s": round(batch * args.steps / dt, 1),
+                          "decode_ms_per_step": round(dt / args.steps * 1e3, 4),
+                          "decode_mean_context": round(mean_ctx, 1)}
+            drop(llm)
+        row["prefill_vs_qwen3"] = round(row["fumanex"]["prefill_tokens_per_s"]
+                                        / row["qwen3"]["prefill_tokens_per_s"], 3)
+        row["decode_vs_qwen3"] = round(row["fumanex"]["decode_tokens_per_s"]
+                                       / row["qwen3"]["decode_tokens_per_s"], 3)
+        if args.dtype == "bfloat16":
+            row["kernels_prefill"] = fumanex_kernels(sh, T, T, mfma_rate, read_bw)
+            row["kernels_decode"] = fumanex_kernels(sh, 1, prompt, mfma_rate, read_bw)
+        ops._workspaces.clear()
+        torch.cuda.empty_cache()
+        shapes[name] = row
+    first = shapes[names[0]]
+    print(json.dumps({
+        "metric": "fumanex_decode_tokens_per_s", "value": first["fumanex"]["decode_tokens_per_s"],
+        "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": first["fumanex"]["decode_ms_per_step"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+        "data": "synthetic", "config": {"model": f"Fumanex {names[0]} shape beside the dense Qwen3 "
+                                                 "decoder of equal size, random weights",
+                                        "batch": batch, "prompt_len": prompt, "prefill_tokens": T,
+                                        "parallelism": "single GPU"},
+        "measured_read_gbs": round(read_bw / 1e9, 1), "mfma_loop_tflops": round(mfma_rate / 1e12, 1),
+        "shapes": shapes}))
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "long-context", "fezupel", "lodenex", "nupovik",
-                             "kugisun"])
+                             "kugisun", "fumanex"])
     ap.add_argument("--shape", default=None, choices=sorted(SHAPES),
                     help="layer sizes (default: 8b for decode, 14b for continuous, 32b for "
                          "long-context)")
@@ -1644,6 +1917,8 @@ def main() -> int:
                     help="nupovik: only this shape (default: all of them)")
     ap.add_argument("--kugisun-shape", default=None, choices=sorted(KUGISUN_SHAPES),
                     help="kugisun: only this shape (default: all of them)")
+    ap.add_argument("--fumanex-shape", default=None, choices=sorted(FUMANEX_SHAPES),
+                    help="fumanex: only this shape (default: all of them)")
     ap.add_argument("--no-run-graphs", action="store_true",
                     help="decode steps in a row replay one graph per step instead of one for the run")
     args = ap.parse_args()
@@ -1654,7 +1929,7 @@ def main() -> int:
     return {"decode": main_decode, "continuous": main_continuous,
             "long-context": main_long_context, "fezupel": main_fezupel,
             "lodenex": main_lodenex, "nupovik": main_nupovik,
-            "kugisun": main_kugisun}[args.workload](args)
+            "kugisun": main_kugisun, "fumanex": main_fumanex}[args.workload](args)
 
 
 if __name__ == "__main__":

@@ -214,6 +214,11 @@ __global__ __launch_bounds__(256) void project_rows_vec8_kernel(
     const RowSegment& g = segs.s[si];
     const bf16_t* x = row + g.src_off;
     const int n8 = g.width / 8;
+    // a norm a head whose 8-element groups are a power of two: the lanes that hold a head lie side
+    // by side in a wave and add their squares among themselves, in the pass that writes
+    const int groups = g.hd / 8;
+    const int lph = g.gain != nullptr && g.per_head && groups <= ZF_WAVE
+        && (groups & (groups - 1)) == 0 ? groups : 0;
     float inv = 1.f;
     if (g.gain != nullptr && !g.per_head) {
       float ss = 0.f;
@@ -225,7 +230,7 @@ __global__ __launch_bounds__(256) void project_rows_vec8_kernel(
       }
       ss = block_sum(ss, red);
       inv = 1.0f / sqrtf(ss / (float)g.width + g.eps);
-    } else if (g.gain != nullptr) {
+    } else if (g.gain != nullptr && lph == 0) {
       __syncthreads();
       const int wave = threadIdx.x / ZF_WAVE, lane = threadIdx.x % ZF_WAVE;
       for (int head = wave; head < g.width / g.hd; head += blockDim.x / ZF_WAVE) {
@@ -268,7 +273,16 @@ __global__ __launch_bounds__(256) void project_rows_vec8_kernel(
       if (d < g.skip) continue;
       float a[8];
       pr_load8(x, g.bias, i, a);
-      const float inv_i = g.per_head ? inv_h[head] : inv;
+      float inv_i = inv;
+      if (lph > 0) {
+        float ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += a[e] * a[e];
+        for (int m = 1; m < lph; m <<= 1) ss += __shfl_xor(ss, m, ZF_WAVE);
+        inv_i = 1.0f / sqrtf(ss / (float)g.hd + g.eps);
+      } else if (g.per_head && g.gain != nullptr) {
+        inv_i = inv_h[head];
+      }
       if (g.gain != nullptr) {
         const int gi = g.per_head ? d : i;
         const float4 g0 = *(const float4*)(g.gain + gi), g1 = *(const float4*)(g.gain + gi + 4);
@@ -906,9 +920,12 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
   const int pos_end = EXT ? k_end + v_shift : k_end;
   // this lane's row of the table of biases, the distance d at [-d]
   const float* brow = nullptr;
+  float brow_last = 0.f;                             // its last number, times log2(e)
   if constexpr (EXT)
-    if (a.dist_bias != nullptr)
+    if (a.dist_bias != nullptr) {
       brow = a.dist_bias + (size_t)h * (a.dist_n + 6) + a.dist_n + 2;
+      brow_last = brow[1 - a.dist_n] * MW_LOG2E;
+    }
 
   // this lane's key of a chunk: key base + c; of its key row the values 16 i + 8 hl .. + 8 for
   // every i, of its value row the same
@@ -973,30 +990,40 @@ __global__ __launch_bounds__(256, 2) void masked_attention_wave_kernel(
       fetch_v(at(vbase + MW_KEYS));
     }
     float cmax = -INFINITY;
+    // (EXT) a chunk whose keys all lie at the table's last distance or beyond: one number a row
+    bool far_chunk = true;
+    float b_far = 0.f;
+    if constexpr (EXT)
+      if (brow != nullptr) {
+        far_chunk = __all(!row_ok || pos_r - base - (MW_KEYS - 1) >= a.dist_n - 1);
+        if (far_chunk) b_far = brow_last;
+      }
     if (capped) {
+      if constexpr (EXT) {
+        // cap tanh(s / cap) + b = (cap + b) - 2 cap / (e^(2 s / cap) + 1)
+        const float c0 = cap_log2 + b_far, c1 = -2.0f * cap_log2;
+        const float u = inv_cap * (2.0f * MW_LOG2E);
 #pragma unroll
-      for (int r = 0; r < 16; ++r) sc[r] = cap_log2 * mw_tanh(sc[r] * inv_cap);
+        for (int r = 0; r < 16; ++r)
+          sc[r] = fmaf(c1, __builtin_amdgcn_rcpf(mw_exp2(sc[r] * u) + 1.0f), c0);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 16; ++r) sc[r] = cap_log2 * mw_tanh(sc[r] * inv_cap);
+      }
     } else {
 #pragma unroll
-      for (int r = 0; r < 16; ++r) sc[r] *= scale_log2;
+      for (int r = 0; r < 16; ++r) sc[r] = EXT ? fmaf(sc[r], scale_log2, b_far) : sc[r] * scale_log2;
     }
     if constexpr (EXT) {
-      if (brow != nullptr) {
+      if (!far_chunk) {
         // keys 8 (r / 4) + 4 hl + r % 4 of the chunk: four side by side read four numbers side
         // by side; distances beyond the table read its last number, keys ahead of the row are
         // masked below
-        const int far = a.dist_n - 1;
-        if (__all(!row_ok || pos_r - base - (MW_KEYS - 1) >= far)) {
-          const float b = brow[-far] * MW_LOG2E;
 #pragma unroll
-          for (int r = 0; r < 16; ++r) sc[r] += b;
-        } else {
+        for (int r4 = 0; r4 < 4; ++r4) {
+          const int d = max(0, min(pos_r - base - 8 * r4 - 4 * hl, a.dist_n + 2));
 #pragma unroll
-          for (int r4 = 0; r4 < 4; ++r4) {
-            const int d = max(0, min(pos_r - base - 8 * r4 - 4 * hl, far + 3));
-#pragma unroll
-            for (int x = 0; x < 4; ++x) sc[4 * r4 + x] = fmaf(brow[x - d], MW_LOG2E, sc[4 * r4 + x]);
-          }
+          for (int x = 0; x < 4; ++x) sc[4 * r4 + x] = fmaf(brow[x - d], MW_LOG2E, sc[4 * r4 + x]);
         }
       }
     }

@@ -607,19 +607,19 @@ extern "C" int zf_decay_recurrence_spans(const void* q, long long q_stride, cons
 // ---------------------------------------------------------------- norm a head, gain, gate
 // out[t, h, :] = o / sqrt(mean(o^2) + eps) * gain * gate(g[t, h, :]) with the gate silu (0) or the
 // sigmoid (1); gain [dv] (one for all heads), [H dv], or null.  o float32, g and out in the rows'
-// type, rows of g and out at strides of their own.  A wave a (token, head), or (WIDE) a workgroup
-// of four waves, whose sums are added in wave order.
+// type, rows of g and out at strides of their own.  A wave a (token, head), or ``lph`` lanes of it
+// where that many lanes of four elements each hold a head (lph a power of two), or (WIDE) a
+// workgroup of four waves, whose sums are added in wave order.
 template <typename T, bool WIDE>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(
     const float* __restrict__ o, const float* __restrict__ gain, int gain_per_head,
     const T* __restrict__ g, long long g_stride, int gate_kind, T* __restrict__ out,
-    long long out_stride, int n_rows, int H, int dv, float eps, int quads) {
+    long long out_stride, int n_rows, int H, int dv, float eps, int quads, int lph) {
   __shared__ float red[16];
-  const int wave = threadIdx.x / ZF_WAVE, lane = threadIdx.x % ZF_WAVE;
-  const int r = WIDE ? blockIdx.x : blockIdx.x * (blockDim.x / ZF_WAVE) + wave;   // (token, head)
-  if (r >= n_rows) return;                // (WIDE: the whole workgroup)
+  const int r = WIDE ? blockIdx.x : (blockIdx.x * blockDim.x + threadIdx.x) / lph;  // (token, head)
+  if (r >= n_rows) return;                // (WIDE: the whole workgroup; else all lanes of a head)
   const int t = r / H, hd = r % H;
-  const int at = WIDE ? threadIdx.x : lane, step = WIDE ? blockDim.x : ZF_WAVE;
+  const int at = WIDE ? threadIdx.x : threadIdx.x % lph, step = WIDE ? blockDim.x : lph;
   const float* row = o + (size_t)r * dv;
   float ss = 0.f;
   if (quads) {
@@ -630,7 +630,11 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(
   } else {
     for (int i = at; i < dv; i += step) ss = fmaf(row[i], row[i], ss);
   }
-  ss = WIDE ? block_sum(ss, red) : wave_sum(ss);
+  if constexpr (WIDE) {
+    ss = block_sum(ss, red);
+  } else {
+    for (int m = lph / 2; m > 0; m >>= 1) ss += __shfl_xor(ss, m, ZF_WAVE);
+  }
   const float inv = 1.0f / sqrtf(ss / (float)dv + eps);
   const T* gr = g + (size_t)t * g_stride + (size_t)hd * dv;
   T* orow = out + (size_t)t * out_stride + (size_t)hd * dv;
@@ -675,11 +679,14 @@ extern "C" int zf_head_norm_gate(const float* o, const float* gain, int gain_per
                     (uintptr_t)g % (4 * esz) == 0 && (uintptr_t)out % (4 * esz) == 0 &&
                     g_stride % 4 == 0 && out_stride % 4 == 0;
   const bool wide = dv > 512;
-  const dim3 grid(wide ? rows : (rows + 3) / 4), block(4 * ZF_WAVE);
+  int lph = ZF_WAVE;
+  if (quads && dv / 4 < ZF_WAVE && (dv / 4 & (dv / 4 - 1)) == 0) lph = dv / 4;
+  const int per_group = 4 * ZF_WAVE / lph;
+  const dim3 grid(wide ? rows : (rows + per_group - 1) / per_group), block(4 * ZF_WAVE);
 #define HNG(TT, W)                                                                               \
   hipLaunchKernelGGL((head_norm_gate_kernel<TT, W>), grid, block, 0, stream, o, gain,            \
                      gain_per_head, (const TT*)g, g_stride, gate_kind, (TT*)out, out_stride,     \
-                     rows, H, dv, eps, quads)
+                     rows, H, dv, eps, quads, lph)
   if (dtype == ZF_F32) { if (wide) HNG(float, true); else HNG(float, false); }
   else { if (wide) HNG(bf16_t, true); else HNG(bf16_t, false); }
   ZF_CHECK_LAUNCH();
