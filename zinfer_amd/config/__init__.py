@@ -17,3 +17,5 @@ from .specs import GatedDeltaRuleSpec, ParallelMixerSpec, StreamBlockSpec
 from .kugisun import KugisunConfig
 from .specs import DistanceBiasSpec, FixedDecayAttentionSpec
 from .fumanex import FumanexConfig
+from .specs import GatedMlpSpec, StateSpaceSpec
+from .tigesun import TigesunConfig

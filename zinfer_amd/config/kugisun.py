@@ -62,6 +62,24 @@ def pair_frequencies(dims: int, base: float) -> Tuple[float, ...]:
     return tuple(float(base) ** (-2.0 * i / dims) for i in range(dims // 2))
 
 
+def weight_owners(layers) -> Tuple[int, ...]:
+    """For every layer the layer whose tensors it runs with: itself, or where its ``weights_of``
+    (and that layer's, and so on) leads."""
+    owners = []
+    for i, L in enumerate(layers):
+        if not isinstance(L, dict):
+            raise ConfigError(f"config.json: layers[{i}] must be an object")
+        j, seen = i, set()
+        while layers[j].get("weights_of") is not None:
+            seen.add(j)
+            j = _int(layers[j], "weights_of", f"layers[{j}].", 0)
+            if j >= len(layers) or j in seen or not isinstance(layers[j], dict):
+                raise ConfigError(f"config.json: layers[{i}].weights_of does not lead to a layer "
+                                  "with tensors of its own")
+        owners.append(j)
+    return tuple(owners)
+
+
 @dataclass(frozen=True)
 class KugisunConfig:
     vocab: int
@@ -87,20 +105,7 @@ class KugisunConfig:
         layers = raw.get("layers")
         if not isinstance(layers, list) or not layers:
             raise ConfigError("config.json: 'layers' must be a list with at least one layer")
-        # whose tensors every layer runs with
-        owner = []
-        for i, L in enumerate(layers):
-            if not isinstance(L, dict):
-                raise ConfigError(f"config.json: layers[{i}] must be an object")
-            j = i
-            seen = set()
-            while layers[j].get("weights_of") is not None:
-                seen.add(j)
-                j = _int(layers[j], "weights_of", f"layers[{j}].", 0)
-                if j >= len(layers) or j in seen or not isinstance(layers[j], dict):
-                    raise ConfigError(f"config.json: layers[{i}].weights_of does not lead to a "
-                                      "layer with tensors of its own")
-            owner.append(j)
+        owner = weight_owners(layers)
         numbers = tuple(sorted(set(owner)))
         norm = cls._norm(width, eps)
         blocks = tuple(cls._block(j, layers[j], width, eps, norm, streams) for j in numbers)

@@ -336,6 +336,36 @@ class GatedDeltaRuleSpec:
 
 
 @dataclass(frozen=True)
+class StateSpaceSpec:
+    """A mixer whose memory is one matrix a head, S [state_dim, value_dim], carried from token to
+    token in 32-bit with one decay a head and token.  W_in h = [z | x | B | C | s] with ``n_heads``
+    heads of ``value_dim`` in z and x, ``n_groups`` groups of ``state_dim`` in B and C (head h
+    reads group floor(h / (n_heads / n_groups))) and one number a head in s.  x, B and C each pass a
+    causal convolution over time a channel (``conv_taps`` taps, the last one the token's own,
+    zeros before a sequence's start; the taps - 1 rows before a step are part of the state), its
+    bias and silu.  dt = softplus(s + bias), S_t = exp(-exp(A) dt) S_(t-1) + dt B_t x_t^T, y_t =
+    S_t^T C_t + D x_t.  The heads side by side are multiplied by silu(z), then normed in
+    ``norm_groups`` equal parts with a gain [n_heads * value_dim], then W_o.  The ``*_name`` fields
+    are the tensor names below the mixer's prefix."""
+    hidden_size: int
+    n_heads: int
+    value_dim: int
+    state_dim: int
+    n_groups: int
+    conv_taps: int
+    norm_groups: int
+    norm_eps: float
+    in_name: str = "in"
+    conv_name: str = "conv"
+    conv_bias_name: str = "conv.b"
+    step_bias_name: str = "dt_bias"
+    decay_log_name: str = "A_log"
+    skip_name: str = "D"
+    norm_name: str = "norm"
+    o_name: str = "o"
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers side by side that read the same input: ``left_scale`` * left(h) +
     ``right_scale`` * right(h).  Each has its own tensors (below ``left_prefix`` and
@@ -415,6 +445,20 @@ class SwiGluSpec:
     part's prefix."""
     hidden_size: int
     intermediate_size: int
+    gate_name: str = "gate_proj.weight"
+    up_name: str = "up_proj.weight"
+    down_name: str = "down_proj.weight"
+
+
+@dataclass(frozen=True)
+class GatedMlpSpec:
+    """down(act(gate(x)) * up(x)), ``activation`` as in ``DenseMlpSpec``; ``bias``: all three
+    projections have one (``bias_suffix`` behind the matrix's name)."""
+    hidden_size: int
+    intermediate_size: int
+    activation: str = "gelu_tanh"
+    bias: bool = False
+    bias_suffix: str = ".b"
     gate_name: str = "gate_proj.weight"
     up_name: str = "up_proj.weight"
     down_name: str = "down_proj.weight"
@@ -547,6 +591,10 @@ class ModelSpec:
     embedding_multiplier: float = 1.0       # the embedding row times this enters the stream
     logit_scale: float = 1.0                # logits = head(x) * logit_scale ...
     logit_softcap: Optional[float] = None   # ... then cap * tanh(logits / cap) if given
+    # a norm the (multiplied) embedding row passes before it enters the stream; its gain is the
+    # tensor embedding_norm_prefix + the norm's own weight name
+    embedding_norm: Optional[object] = None
+    embedding_norm_prefix: str = "model.embed_norm."
     # a learned position table [max_positions, hidden]: its row at a token's position is added
     # to the embedding row (not scaled); None: positions enter through the mixers only
     position_table_name: Optional[str] = None

@@ -6,10 +6,10 @@
 // with one decay g_t = exp(-exp(A) softplus(z_a + dt)) and one step size beta_t = sigmoid(z_b) a
 // head and token, and the short convolutions that feed it.  All arithmetic is 32-bit.
 //
-//  * short_conv        rows of a projection -> silu(causal convolution over time a channel); the
-//                      leading channels are heads that are made unit vectors (and the first of
-//                      those multiplied by a scale).  The taps - 1 rows before a step come from the
-//                      request's state.
+//  * short_conv        rows of a projection -> silu(causal convolution over time a channel, plus a
+//                      bias); the leading channels are heads that are made unit vectors (and the
+//                      first of those multiplied by a scale).  The taps - 1 rows before a step come
+//                      from the request's state.
 //  * short_conv_state  the state takes the step's last taps - 1 rows.
 //  * delta_recurrence  the recurrence over the rows of a step, sequence by sequence.
 //
@@ -53,8 +53,8 @@ __device__ __forceinline__ float dl_lanes_sum(float v) {
 }
 
 // ------------------------------------------------------------------ short convolutions
-// src [T, >= C] (row stride given), taps [C, n] float32 (the last column is the token's own),
-// out float32 [T, C].  Channels [0, unit_heads * hd) are heads of hd that leave as unit vectors
+// src [T, >= C] (row stride given), taps [C, n] float32 (the last column is the token's own), bias
+// float32 [C] or null, out [T, C] in float32 or bfloat16.  Channels [0, unit_heads * hd) are heads of hd that leave as unit vectors
 // x / sqrt(sum x^2 + unit_eps), the first scaled_heads of them times `scale`.  State of a
 // request: [n - 1, C] floats at state + slot * state_stride + state_off, oldest row first.
 // Grid (token, block of channels): the first head_blocks blocks hold hpb whole heads each, a
@@ -67,12 +67,12 @@ __device__ __forceinline__ float dl_lanes_sum(float v) {
 #define DL_CONV_MAX_TAPS 8
 #define DL_CONV_PER_THREAD 4     // channels a thread takes of a head wider than the workgroup
 
-template <typename T>
+template <typename T, typename TO>
 __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_kernel(
     const T* __restrict__ src, long long src_stride, const float* __restrict__ taps, int n_taps,
-    float* __restrict__ state, long long state_stride, long long state_off,
-    const int* __restrict__ state_slots, const int* __restrict__ seq_index,
-    const int* __restrict__ q_start, float* __restrict__ out, int C, int unit_heads, int hd,
+    const float* __restrict__ bias, float* __restrict__ state, long long state_stride,
+    long long state_off, const int* __restrict__ state_slots, const int* __restrict__ seq_index,
+    const int* __restrict__ q_start, TO* __restrict__ out, int C, int unit_heads, int hd,
     int scaled_heads, float scale, float unit_eps, int update_state, int head_blocks, int hpb) {
 #pragma clang fp contract(off)
   __shared__ float sq[DL_CONV_THREADS / ZF_WAVE];
@@ -102,13 +102,13 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_kernel(
       for (int j = 1; j < DL_CONV_MAX_TAPS; ++j)
         if (j < n_taps) st[(size_t)(j - 1) * C + c] = x[j];
     }
-    return dl_silu(acc);
+    return dl_silu(bias != nullptr ? acc + bias[c] : acc);
   };
-  float* o = out + (size_t)t * C;
+  TO* o = out + (size_t)t * C;
   const int b = blockIdx.y;
   if (b >= head_blocks) {
     const int c = unit_heads * hd + (b - head_blocks) * DL_CONV_THREADS + threadIdx.x;
-    if (c < C) o[c] = conv(c);
+    if (c < C) store_from_float<TO>(o + c, conv(c));
     return;
   }
   // a head takes tph threads, whole waves of them (hpb heads a block), a thread `per` channels
@@ -141,7 +141,126 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_kernel(
 #pragma unroll
   for (int j = 0; j < DL_CONV_PER_THREAD; ++j) {
     const int dd = d0 + j * tph;
-    if (j < per && dd < hd) o[head * hd + dd] = v[j] * inv;
+    if (j < per && dd < hd) store_from_float<TO>(o + head * hd + dd, v[j] * inv);
+  }
+}
+
+// The same where no channel belongs to a head: a thread takes V neighbouring channels (16 bytes of a
+// row) of TT tokens one behind the other and keeps the rows before the token in registers, NT of
+// them with the token's own (n_taps <= NT; the rows further back meet taps of zero).  The same
+// products and sums in the same order as above.  Grid (blocks of TT tokens, blocks of channels).
+template <typename T, typename TO, int V, int NT>
+__global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_rows_kernel(
+    const T* __restrict__ src, long long src_stride, const float* __restrict__ taps, int n_taps,
+    const float* __restrict__ bias, float* __restrict__ state, long long state_stride,
+    long long state_off, const int* __restrict__ state_slots, const int* __restrict__ seq_index,
+    const int* __restrict__ q_start, TO* __restrict__ out, int n_tokens, int C, int TT,
+    int update_state) {
+#pragma clang fp contract(off)
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (c >= C) return;
+  const int hist = n_taps - 1;
+  float tp[NT][V], b[V], w[NT][V];
+  if (n_taps == NT) {
+    float flat[V * NT];
+#pragma unroll
+    for (int i = 0; i < V * NT; i += 4) {
+      const float4 f = *(const float4*)(taps + (size_t)c * NT + i);
+      flat[i] = f.x; flat[i + 1] = f.y; flat[i + 2] = f.z; flat[i + 3] = f.w;
+    }
+#pragma unroll
+    for (int k = 0; k < NT; ++k)
+#pragma unroll
+      for (int v = 0; v < V; ++v) tp[k][v] = flat[v * NT + k];
+  } else {
+#pragma unroll
+    for (int k = 0; k < NT; ++k)
+#pragma unroll
+      for (int v = 0; v < V; ++v) {
+        const int j = k - (NT - n_taps);
+        tp[k][v] = j >= 0 ? taps[(size_t)(c + v) * n_taps + j] : 0.f;
+      }
+  }
+#pragma unroll
+  for (int v = 0; v < V; v += 4) {
+    float4 f = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (bias != nullptr) f = *(const float4*)(bias + c + v);
+    b[v] = f.x; b[v + 1] = f.y; b[v + 2] = f.z; b[v + 3] = f.w;
+  }
+  auto load_row = [&](int t, float (&x)[V]) {
+    if constexpr (sizeof(T) == 2) {
+      const uint4 r = *(const uint4*)(src + (size_t)t * src_stride + c);
+      const uint32_t u[4] = {r.x, r.y, r.z, r.w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        x[2 * i] = __uint_as_float(u[i] << 16);
+        x[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u);
+      }
+    } else {
+      const float4 f = *(const float4*)(src + (size_t)t * src_stride + c);
+      x[0] = f.x; x[1] = f.y; x[2] = f.z; x[3] = f.w;
+    }
+  };
+  const int first = blockIdx.x * TT, last = min(n_tokens, first + TT);
+  int seq = -1;
+  for (int t = first; t < last; ++t) {
+    const int s = seq_index[t];
+    float* st = state + (size_t)state_slots[s] * state_stride + state_off;
+    if (s != seq) {
+      // the rows before this token: of its portion, or of the request's state
+      const int i0 = t - q_start[s];
+#pragma unroll
+      for (int k = 0; k < NT - 1; ++k) {
+        const int back = NT - 1 - k;
+#pragma unroll
+        for (int v = 0; v < V; ++v) w[k][v] = 0.f;
+        if (back <= hist) {
+          if (back <= i0) {
+            load_row(t - back, w[k]);
+          } else {
+#pragma unroll
+            for (int v = 0; v < V; v += 4) {
+              const float4 f = *(const float4*)(st + (size_t)(hist + i0 - back) * C + c + v);
+              w[k][v] = f.x; w[k][v + 1] = f.y; w[k][v + 2] = f.z; w[k][v + 3] = f.w;
+            }
+          }
+        }
+      }
+      seq = s;
+    }
+    load_row(t, w[NT - 1]);
+    float acc[V];
+#pragma unroll
+    for (int v = 0; v < V; ++v) {
+      acc[v] = 0.f;
+#pragma unroll
+      for (int k = 0; k < NT; ++k) acc[v] = acc[v] + tp[k][v] * w[k][v];
+      acc[v] = dl_silu(bias != nullptr ? acc[v] + b[v] : acc[v]);
+    }
+    TO* o = out + (size_t)t * C + c;
+    if constexpr (sizeof(TO) == 2) {
+      *(uint4*)o = make_uint4(pack_bf16x2(acc[0], acc[1]), pack_bf16x2(acc[2], acc[3]),
+                              pack_bf16x2(acc[4], acc[5]), pack_bf16x2(acc[6], acc[7]));
+    } else {
+#pragma unroll
+      for (int v = 0; v < V; v += 4)
+        *(float4*)(o + v) = make_float4(acc[v], acc[v + 1], acc[v + 2], acc[v + 3]);
+    }
+    if (update_state) {
+      // the kept rows move on by one: the last n_taps - 1 rows of the window
+#pragma unroll
+      for (int k = 1; k < NT; ++k)
+        if (k >= NT - hist) {
+#pragma unroll
+          for (int v = 0; v < V; v += 4)
+            *(float4*)(st + (size_t)(k - (NT - hist)) * C + c + v) =
+                make_float4(w[k][v], w[k][v + 1], w[k][v + 2], w[k][v + 3]);
+        }
+    }
+#pragma unroll
+    for (int k = 0; k + 1 < NT; ++k)
+#pragma unroll
+      for (int v = 0; v < V; ++v) w[k][v] = w[k + 1][v];
   }
 }
 
@@ -168,15 +287,16 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_state_kernel(
 }
 
 extern "C" int zf_short_conv(const void* src, int dtype, long long src_stride, const float* taps,
-                             int n_taps, float* state, long long state_stride,
+                             int n_taps, const float* bias, float* state, long long state_stride,
                              long long state_off, const int* state_slots, const int* seq_index,
-                             const int* q_start, float* out, int T, int n_seqs, int C,
+                             const int* q_start, void* out, int out_dtype, int T, int n_seqs, int C,
                              int unit_heads, int hd, int scaled_heads, float scale,
                              float unit_eps, int single_tokens, hipStream_t stream) {
   if (T <= 0) return 0;
   if (C <= 0 || n_taps < 1 || n_taps > DL_CONV_MAX_TAPS || unit_heads < 0 || hd < 1 ||
       (size_t)unit_heads * hd > (size_t)C || scaled_heads > unit_heads || n_seqs < 1 ||
-      (single_tokens && T != n_seqs) || hd > DL_CONV_THREADS * DL_CONV_PER_THREAD)
+      (single_tokens && T != n_seqs) || hd > DL_CONV_THREADS * DL_CONV_PER_THREAD ||
+      (dtype == ZF_F32 && out_dtype != ZF_F32))
     return -2;
   // a head takes whole waves (one, two or four): as many heads a block as fit
   const int hw = hd > 128 ? 4 : (hd > 64 ? 2 : 1);
@@ -185,16 +305,35 @@ extern "C" int zf_short_conv(const void* src, int dtype, long long src_stride, c
   const int plain = C - unit_heads * hd;
   const dim3 grid(T, head_blocks + (plain + DL_CONV_THREADS - 1) / DL_CONV_THREADS);
   const dim3 sgrid(n_seqs, (C + DL_CONV_THREADS - 1) / DL_CONV_THREADS);
-#define DL_CONV_LAUNCH(TT)                                                                        \
-  hipLaunchKernelGGL(short_conv_kernel<TT>, grid, dim3(DL_CONV_THREADS), 0, stream,              \
-                     (const TT*)src, src_stride, taps, n_taps, state, state_stride, state_off,   \
-                     state_slots, seq_index, q_start, out, C, unit_heads, hd, scaled_heads,      \
-                     scale, unit_eps, single_tokens, head_blocks, hpb);                          \
-  if (!single_tokens && n_taps > 1)                                                               \
-    hipLaunchKernelGGL(short_conv_state_kernel<TT>, sgrid, dim3(DL_CONV_THREADS), 0, stream,     \
-                       (const TT*)src, src_stride, n_taps, state, state_stride, state_off,       \
+  const int V = dtype == ZF_F32 ? 4 : 8;
+  const bool rows = unit_heads == 0 && C % V == 0 && src_stride % V == 0 && state_stride % 4 == 0 &&
+                    state_off % 4 == 0 && (uintptr_t)src % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+                    (uintptr_t)taps % 16 == 0 && (uintptr_t)bias % 16 == 0 &&
+                    (uintptr_t)state % 16 == 0;
+  const int threads = 64;
+  const int TT = single_tokens ? 1 : (T >= 1024 ? 8 : (T >= 256 ? 4 : 2));
+  const dim3 rgrid((T + TT - 1) / TT, (C / V + threads - 1) / threads);
+#define DL_CONV_ROWS(TT_, TO_, V_, N_)                                                            \
+  hipLaunchKernelGGL((short_conv_rows_kernel<TT_, TO_, V_, N_>), rgrid, dim3(threads), 0, stream,\
+                     (const TT_*)src, src_stride, taps, n_taps, bias, state, state_stride,       \
+                     state_off, state_slots, seq_index, q_start, (TO_*)out, T, C, TT, single_tokens)
+#define DL_CONV_LAUNCH(TT_, TO_, V_)                                                              \
+  if (rows) {                                                                                    \
+    if (n_taps <= 4) DL_CONV_ROWS(TT_, TO_, V_, 4);                                              \
+    else DL_CONV_ROWS(TT_, TO_, V_, 8);                                                          \
+  } else {                                                                                       \
+    hipLaunchKernelGGL((short_conv_kernel<TT_, TO_>), grid, dim3(DL_CONV_THREADS), 0, stream,    \
+                       (const TT_*)src, src_stride, taps, n_taps, bias, state, state_stride,     \
+                       state_off, state_slots, seq_index, q_start, (TO_*)out, C, unit_heads, hd, \
+                       scaled_heads, scale, unit_eps, single_tokens, head_blocks, hpb);          \
+  }                                                                                              \
+  if (!single_tokens && n_taps > 1)                                                              \
+    hipLaunchKernelGGL(short_conv_state_kernel<TT_>, sgrid, dim3(DL_CONV_THREADS), 0, stream,    \
+                       (const TT_*)src, src_stride, n_taps, state, state_stride, state_off,      \
                        state_slots, q_start, C)
-  if (dtype == ZF_F32) { DL_CONV_LAUNCH(float); } else { DL_CONV_LAUNCH(bf16_t); }
+  if (dtype == ZF_F32) { DL_CONV_LAUNCH(float, float, 4); }
+  else if (out_dtype == ZF_F32) { DL_CONV_LAUNCH(bf16_t, float, 8); }
+  else { DL_CONV_LAUNCH(bf16_t, bf16_t, 8); }
   ZF_CHECK_LAUNCH();
 }
 

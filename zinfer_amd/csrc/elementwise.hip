@@ -647,6 +647,63 @@ extern "C" int zf_bias_act_rows(const void* x, int dtype, long long x_stride, co
   ZF_CHECK_LAUNCH();
 }
 
+// out[t, i] = act(x[t, i] + bias[i]) * (x[t, n + i] + bias[n + i]) for i < n: rows of a product over
+// a gate's and an up projection's stacked rows, with their biases (or null); the activation as
+// above, 32-bit.  grid (blocks of columns, rows); V neighbouring columns a thread.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void gated_rows_kernel(
+    const T* __restrict__ x, long long x_stride, const float* __restrict__ bias,
+    T* __restrict__ out, int n, int kind) {
+  const T* g = x + (size_t)blockIdx.y * x_stride;
+  const T* u = g + n;
+  T* o = out + (size_t)blockIdx.y * n;
+  const int i = (blockIdx.x * blockDim.x + threadIdx.x) * V;
+  if (i >= n) return;
+  if (V == 8) {
+    const uint4 gv = *(const uint4*)(g + i), uv = *(const uint4*)(u + i);
+    const uint32_t gw[4] = {gv.x, gv.y, gv.z, gv.w}, uw[4] = {uv.x, uv.y, uv.z, uv.w};
+    float gb[8], ub[8];
+#pragma unroll
+    for (int e = 0; e < 8; e += 4) {
+      float4 a = make_float4(0.f, 0.f, 0.f, 0.f), b = a;
+      if (bias != nullptr) { a = *(const float4*)(bias + i + e); b = *(const float4*)(bias + n + i + e); }
+      gb[e] = a.x; gb[e + 1] = a.y; gb[e + 2] = a.z; gb[e + 3] = a.w;
+      ub[e] = b.x; ub[e + 1] = b.y; ub[e + 2] = b.z; ub[e + 3] = b.w;
+    }
+    uint32_t w[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      w[e] = pack_bf16x2(bias_act_value<T>(__uint_as_float(gw[e] << 16) + gb[2 * e], kind)
+                             * (__uint_as_float(uw[e] << 16) + ub[2 * e]),
+                         bias_act_value<T>(__uint_as_float(gw[e] & 0xffff0000u) + gb[2 * e + 1], kind)
+                             * (__uint_as_float(uw[e] & 0xffff0000u) + ub[2 * e + 1]));
+    *(uint4*)(o + i) = make_uint4(w[0], w[1], w[2], w[3]);
+  } else {
+    const float gb = bias != nullptr ? bias[i] : 0.f, ub = bias != nullptr ? bias[n + i] : 0.f;
+    store_from_float<T>(o + i, bias_act_value<T>(load_as_float<T>(g + i) + gb, kind)
+                                   * (load_as_float<T>(u + i) + ub));
+  }
+}
+
+extern "C" int zf_gated_rows(const void* x, int dtype, long long x_stride, const float* bias,
+                             void* out, int T, int n, int kind, hipStream_t stream) {
+  if (T <= 0 || n <= 0) return 0;
+  if (kind < 0 || kind > 4) return -2;
+  const bool vec = dtype == ZF_BF16 && n % 8 == 0 && x_stride % 8 == 0 && (uintptr_t)x % 16 == 0 &&
+                   (uintptr_t)out % 16 == 0 && (uintptr_t)bias % 16 == 0;
+  const dim3 grid((unsigned)((n / (vec ? 8 : 1) + 255) / 256), T);
+  if (vec)
+    hipLaunchKernelGGL((gated_rows_kernel<bf16_t, 8>), grid, dim3(256), 0, stream,
+                       (const bf16_t*)x, x_stride, bias, (bf16_t*)out, n, kind);
+  else if (dtype == ZF_BF16)
+    hipLaunchKernelGGL((gated_rows_kernel<bf16_t, 1>), grid, dim3(256), 0, stream,
+                       (const bf16_t*)x, x_stride, bias, (bf16_t*)out, n, kind);
+  else
+    hipLaunchKernelGGL((gated_rows_kernel<float, 1>), grid, dim3(256), 0, stream,
+                       (const float*)x, x_stride, bias, (float*)out, n, kind);
+  ZF_CHECK_LAUNCH();
+}
+
 // x[t, i] += bias[i] for float32 rows
 __global__ __launch_bounds__(256) void add_row_kernel(float* __restrict__ x,
                                                       const float* __restrict__ bias, int n) {

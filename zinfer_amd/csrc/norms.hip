@@ -18,9 +18,11 @@ __device__ __forceinline__ void norm_store(TO* o, float v) {
   }
 }
 
-// any width: the row is read three times
+// any width: the row is read three times.  x_bias (or null): a row added to x first, what a
+// sublayer's output product leaves out
 template <typename TO, bool ADD>
 __global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict__ x,
+                                                        const float* __restrict__ x_bias,
                                                         const float* __restrict__ gain,
                                                         const float* __restrict__ bias,
                                                         TO* __restrict__ out, int W, float eps,
@@ -28,21 +30,22 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict_
   __shared__ float red[16];
   const float* row = x + (size_t)blockIdx.x * W;
   TO* o = out + (size_t)blockIdx.x * W;
+  auto at = [&](int i) { return x_bias != nullptr ? row[i] + x_bias[i] : row[i]; };
   float mean = 0.f;
   if (centred) {
     float s = 0.f;
-    for (int i = threadIdx.x; i < W; i += blockDim.x) s += row[i];
+    for (int i = threadIdx.x; i < W; i += blockDim.x) s += at(i);
     mean = block_sum(s, red) / (float)W;
   }
   float ss = 0.f;
   for (int i = threadIdx.x; i < W; i += blockDim.x) {
-    const float d = row[i] - mean;
+    const float d = at(i) - mean;
     ss += d * d;
   }
   ss = block_sum(ss, red);
   const float inv = 1.0f / sqrtf(ss / (float)W + eps);
   for (int i = threadIdx.x; i < W; i += blockDim.x) {
-    float v = (row[i] - mean) * inv * gain[i];
+    float v = (at(i) - mean) * inv * gain[i];
     if (bias != nullptr) v += bias[i];
     norm_store<TO, ADD>(o + i, v);
   }
@@ -52,6 +55,7 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(const float* __restrict_
 // float4) in registers, so the row is read once
 template <typename TO, bool ADD>
 __global__ __launch_bounds__(256) void norm_rows_vec_kernel(const float* __restrict__ x,
+                                                            const float* __restrict__ x_bias,
                                                             const float* __restrict__ gain,
                                                             const float* __restrict__ bias,
                                                             TO* __restrict__ out, int W,
@@ -65,6 +69,10 @@ __global__ __launch_bounds__(256) void norm_rows_vec_kernel(const float* __restr
   for (int i = 0; i < 8; ++i) {
     const int c = threadIdx.x + i * 256;
     v[i] = c < n4 ? row[c] : make_float4(0.f, 0.f, 0.f, 0.f);
+    if (x_bias != nullptr && c < n4) {
+      const float4 b = ((const float4*)x_bias)[c];
+      v[i].x += b.x; v[i].y += b.y; v[i].z += b.z; v[i].w += b.w;
+    }
   }
   float mean = 0.f;
   if (centred) {
@@ -100,40 +108,42 @@ __global__ __launch_bounds__(256) void norm_rows_vec_kernel(const float* __restr
 }
 
 template <typename TO, bool ADD>
-static void launch_norm_rows(const float* x, const float* gain, const float* bias, void* out,
-                             int T, int W, float eps, int centred, hipStream_t stream) {
+static void launch_norm_rows(const float* x, const float* x_bias, const float* gain,
+                             const float* bias, void* out, int T, int W, float eps, int centred,
+                             hipStream_t stream) {
   if (W % 4 == 0 && W <= 8192)
-    hipLaunchKernelGGL((norm_rows_vec_kernel<TO, ADD>), dim3(T), dim3(256), 0, stream, x, gain,
-                       bias, (TO*)out, W, eps, centred);
+    hipLaunchKernelGGL((norm_rows_vec_kernel<TO, ADD>), dim3(T), dim3(256), 0, stream, x, x_bias,
+                       gain, bias, (TO*)out, W, eps, centred);
   else
-    hipLaunchKernelGGL((norm_rows_kernel<TO, ADD>), dim3(T), dim3(256), 0, stream, x, gain, bias,
-                       (TO*)out, W, eps, centred);
+    hipLaunchKernelGGL((norm_rows_kernel<TO, ADD>), dim3(T), dim3(256), 0, stream, x, x_bias, gain,
+                       bias, (TO*)out, W, eps, centred);
 }
 
-// out = norm(x) (add == 0) or out += norm(x) (add != 0, out float32); bias may be null
-extern "C" int zf_norm_rows(const float* x, const float* gain, const float* bias, void* out,
-                            int out_dtype, int T, int W, float eps, int centred, int add,
-                            hipStream_t stream) {
+// out = norm(x + x_bias) (add == 0) or out += norm(x + x_bias) (add != 0, out float32); x_bias and
+// bias may be null
+extern "C" int zf_norm_rows(const float* x, const float* x_bias, const float* gain,
+                            const float* bias, void* out, int out_dtype, int T, int W, float eps,
+                            int centred, int add, hipStream_t stream) {
   if (T <= 0) return 0;
   if (W <= 0 || (add && out_dtype != ZF_F32)) return -2;
   if (add)
-    launch_norm_rows<float, true>(x, gain, bias, out, T, W, eps, centred, stream);
+    launch_norm_rows<float, true>(x, x_bias, gain, bias, out, T, W, eps, centred, stream);
   else if (out_dtype == ZF_F32)
-    launch_norm_rows<float, false>(x, gain, bias, out, T, W, eps, centred, stream);
+    launch_norm_rows<float, false>(x, x_bias, gain, bias, out, T, W, eps, centred, stream);
   else
-    launch_norm_rows<bf16_t, false>(x, gain, bias, out, T, W, eps, centred, stream);
+    launch_norm_rows<bf16_t, false>(x, x_bias, gain, bias, out, T, W, eps, centred, stream);
   ZF_CHECK_LAUNCH();
 }
 
 // ---------------------------------------------------------------- a norm behind a sublayer and the one before the next
-// x += norm_a(y); out = norm_b(x): the norm that closes a sublayer adds its result into the
+// x += norm_a(y + y_bias); out = norm_b(x): the norm that closes a sublayer adds its result into the
 // residual stream, and the norm that opens the next sublayer reads the sum while the row is
 // still in registers (one kernel and one pass over the stream instead of two).  Widths that
 // are a multiple of 4 up to 8192.  Each norm as in norm_rows (32-bit, mean first, variance from
 // the deviations): the same numbers as the two kernels one after the other.
 template <typename TO>
 __global__ __launch_bounds__(256) void norm_add_norm_kernel(
-    const float* __restrict__ y, const float* __restrict__ gain_a, const float* __restrict__ bias_a,
+    const float* __restrict__ y, const float* __restrict__ y_bias, const float* __restrict__ gain_a, const float* __restrict__ bias_a,
     float eps_a, int centred_a, float* __restrict__ x, const float* __restrict__ gain_b,
     const float* __restrict__ bias_b, float eps_b, int centred_b, TO* __restrict__ out, int W) {
   __shared__ float red[16];
@@ -146,6 +156,10 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
   for (int i = 0; i < 8; ++i) {
     const int c = threadIdx.x + i * 256;
     v[i] = c < n4 ? yrow[c] : make_float4(0.f, 0.f, 0.f, 0.f);
+    if (y_bias != nullptr && c < n4) {
+      const float4 b = ((const float4*)y_bias)[c];
+      v[i].x += b.x; v[i].y += b.y; v[i].z += b.z; v[i].w += b.w;
+    }
   }
   // one norm over the row held in v: v = (v - mean) * inv * gain + bias, in place
   auto norm = [&](const float* gain, const float* bias, float eps, int centred) {
@@ -204,18 +218,18 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
   }
 }
 
-extern "C" int zf_norm_add_norm(const float* y, const float* gain_a, const float* bias_a,
+extern "C" int zf_norm_add_norm(const float* y, const float* y_bias, const float* gain_a, const float* bias_a,
                                 float eps_a, int centred_a, float* x, const float* gain_b,
                                 const float* bias_b, float eps_b, int centred_b, void* out,
                                 int out_dtype, int T, int W, hipStream_t stream) {
   if (T <= 0) return 0;
   if (W <= 0 || W % 4 != 0 || W > 8192) return -2;
   if (out_dtype == ZF_F32)
-    hipLaunchKernelGGL(norm_add_norm_kernel<float>, dim3(T), dim3(256), 0, stream, y, gain_a,
-                       bias_a, eps_a, centred_a, x, gain_b, bias_b, eps_b, centred_b, (float*)out, W);
+    hipLaunchKernelGGL(norm_add_norm_kernel<float>, dim3(T), dim3(256), 0, stream, y, y_bias,
+                       gain_a, bias_a, eps_a, centred_a, x, gain_b, bias_b, eps_b, centred_b, (float*)out, W);
   else
-    hipLaunchKernelGGL(norm_add_norm_kernel<bf16_t>, dim3(T), dim3(256), 0, stream, y, gain_a,
-                       bias_a, eps_a, centred_a, x, gain_b, bias_b, eps_b, centred_b,
+    hipLaunchKernelGGL(norm_add_norm_kernel<bf16_t>, dim3(T), dim3(256), 0, stream, y, y_bias,
+                       gain_a, bias_a, eps_a, centred_a, x, gain_b, bias_b, eps_b, centred_b,
                        (bf16_t*)out, W);
   ZF_CHECK_LAUNCH();
 }
@@ -453,6 +467,54 @@ extern "C" int zf_streams_step(float* x, long long copy_stride, int S, const flo
     if (vec) STREAMS_LAUNCH(float, 4); else STREAMS_LAUNCH(float, 1);
   } else {
     if (vec) STREAMS_LAUNCH(bf16_t, 4); else STREAMS_LAUNCH(bf16_t, 1);
+  }
+  ZF_CHECK_LAUNCH();
+}
+
+// ---------------------------------------------------------------- the embedding through a norm
+// x[t, :] = e / sqrt(mean(e^2) + eps) * gain with e = E[id[t], :] * scale, float32; and (gain_b not
+// null) the norm that reads x next: out[t, :] = x / sqrt(mean(x^2) + eps_b) * gain_b.  A workgroup a
+// row of any width; the table's row is read again for every pass.
+template <typename TW, typename TO>
+__global__ __launch_bounds__(256) void embed_norm_kernel(
+    const TW* __restrict__ table, const int* __restrict__ ids, float scale,
+    const float* __restrict__ gain, float eps, float* __restrict__ x,
+    const float* __restrict__ gain_b, float eps_b, TO* __restrict__ out, int W) {
+  __shared__ float red[16];
+  const TW* row = table + (size_t)ids[blockIdx.x] * W;
+  float* xr = x + (size_t)blockIdx.x * W;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float e = load_as_float<TW>(row + i) * scale;
+    ss = fmaf(e, e, ss);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)W + eps);
+  float sb = 0.f;
+  for (int i = threadIdx.x; i < W; i += blockDim.x) {
+    const float v = load_as_float<TW>(row + i) * scale * inv * gain[i];
+    xr[i] = v;
+    sb = fmaf(v, v, sb);
+  }
+  if (gain_b == nullptr) return;
+  const float inv_b = 1.0f / sqrtf(block_sum(sb, red) / (float)W + eps_b);
+  TO* o = out + (size_t)blockIdx.x * W;
+  for (int i = threadIdx.x; i < W; i += blockDim.x)
+    store_from_float<TO>(o + i, load_as_float<TW>(row + i) * scale * inv * gain[i] * inv_b * gain_b[i]);
+}
+
+extern "C" int zf_embed_norm(const void* table, int table_dtype, const int* ids, float scale,
+                             const float* gain, float eps, float* x, const float* gain_b,
+                             float eps_b, void* out, int out_dtype, int T, int W,
+                             hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (W <= 0 || (gain_b != nullptr && out == nullptr)) return -2;
+#define EMBED_NORM(TW, TO)                                                                       \
+  hipLaunchKernelGGL((embed_norm_kernel<TW, TO>), dim3(T), dim3(256), 0, stream,                 \
+                     (const TW*)table, ids, scale, gain, eps, x, gain_b, eps_b, (TO*)out, W)
+  if (table_dtype == ZF_F32) {
+    if (out_dtype == ZF_F32) EMBED_NORM(float, float); else EMBED_NORM(float, bf16_t);
+  } else {
+    if (out_dtype == ZF_F32) EMBED_NORM(bf16_t, float); else EMBED_NORM(bf16_t, bf16_t);
   }
   ZF_CHECK_LAUNCH();
 }

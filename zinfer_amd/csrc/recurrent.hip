@@ -691,3 +691,95 @@ extern "C" int zf_head_norm_gate(const float* o, const float* gain, int gain_per
   else { if (wide) HNG(bf16_t, true); else HNG(bf16_t, false); }
   ZF_CHECK_LAUNCH();
 }
+
+// ---------------------------------------------------------------- gate, then a norm over equal parts
+// u = o * gate(g); out[t, p, :] = u / sqrt(mean(u^2) + eps) * gain over the P parts of dv columns a
+// row has; gain [P dv].  Otherwise as above: a wave a (token, part), or (WIDE) a workgroup of four
+// waves.  With `quads` a thread keeps its R groups of four u in registers between the two passes.
+template <typename T, bool WIDE>
+__global__ __launch_bounds__(256) void gate_norm_kernel(
+    const float* __restrict__ o, const float* __restrict__ gain, const T* __restrict__ g,
+    long long g_stride, int gate_kind, T* __restrict__ out, long long out_stride, int n_rows, int P,
+    int dv, float eps, int quads) {
+  constexpr int R = WIDE ? 8 : 2, LANES = WIDE ? 256 : ZF_WAVE;
+  __shared__ float red[16];
+  const int r = WIDE ? blockIdx.x : (blockIdx.x * blockDim.x + threadIdx.x) / LANES;  // (token, part)
+  if (r >= n_rows) return;                // (WIDE: the whole workgroup; else the whole wave)
+  const int t = r / P, part = r % P, at = threadIdx.x % LANES;
+  const float* row = o + (size_t)r * dv;
+  const T* gr = g + (size_t)t * g_stride + (size_t)part * dv;
+  T* orow = out + (size_t)t * out_stride + (size_t)part * dv;
+  const float* gn = gain + (size_t)part * dv;
+  auto gated = [&](float x, float gv) {
+    const float s = 1.0f / (1.0f + expf(-gv));
+    return x * (gate_kind == 0 ? gv * s : s);
+  };
+  float ss = 0.f;
+  float4 u[R];
+  if (quads) {
+#pragma unroll
+    for (int k = 0; k < R; ++k) {
+      const int i = 4 * (at + k * LANES);
+      u[k] = float4{0.f, 0.f, 0.f, 0.f};
+      if (i < dv) {
+        const float4 x = *(const float4*)(row + i);
+        float4 w;
+        if constexpr (sizeof(T) == 2) {
+          const uint2 b = *(const uint2*)(gr + i);
+          w = float4{__uint_as_float(b.x << 16), __uint_as_float(b.x & 0xffff0000u),
+                     __uint_as_float(b.y << 16), __uint_as_float(b.y & 0xffff0000u)};
+        } else {
+          w = *(const float4*)(gr + i);
+        }
+        u[k] = float4{gated(x.x, w.x), gated(x.y, w.y), gated(x.z, w.z), gated(x.w, w.w)};
+        ss = fmaf(u[k].x, u[k].x, fmaf(u[k].y, u[k].y, fmaf(u[k].z, u[k].z, fmaf(u[k].w, u[k].w, ss))));
+      }
+    }
+  } else {
+    for (int i = at; i < dv; i += LANES) {
+      const float v = gated(row[i], load_as_float<T>(gr + i));
+      ss = fmaf(v, v, ss);
+    }
+  }
+  if constexpr (WIDE) ss = block_sum(ss, red);
+  else ss = wave_sum(ss);
+  const float inv = 1.0f / sqrtf(ss / (float)dv + eps);
+  if (quads) {
+#pragma unroll
+    for (int k = 0; k < R; ++k) {
+      const int i = 4 * (at + k * LANES);
+      if (i < dv) {
+        const float4 w = *(const float4*)(gn + i);
+        const float4 v = float4{u[k].x * inv * w.x, u[k].y * inv * w.y, u[k].z * inv * w.z,
+                                u[k].w * inv * w.w};
+        if constexpr (sizeof(T) == 2)
+          *(uint2*)(orow + i) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
+        else
+          *(float4*)(orow + i) = v;
+      }
+    }
+  } else {
+    for (int i = at; i < dv; i += LANES)
+      store_from_float<T>(orow + i, gated(row[i], load_as_float<T>(gr + i)) * inv * gn[i]);
+  }
+}
+
+extern "C" int zf_gate_norm(const float* o, const float* gain, const void* g, long long g_stride,
+                            int gate_kind, void* out, long long out_stride, int dtype, int T, int P,
+                            int dv, float eps, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (P <= 0 || dv <= 0 || gate_kind < 0 || gate_kind > 1) return -2;
+  const int rows = T * P;
+  const int esz = dtype == ZF_F32 ? 4 : 2;
+  const int quads = dv % 4 == 0 && dv <= 8192 && (uintptr_t)o % 16 == 0 &&
+                    (uintptr_t)gain % 16 == 0 && (uintptr_t)g % (4 * esz) == 0 &&
+                    (uintptr_t)out % (4 * esz) == 0 && g_stride % 4 == 0 && out_stride % 4 == 0;
+  const bool wide = dv > 512;
+  const dim3 grid(wide ? rows : (rows + 3) / 4), block(256);
+#define GN(TT, W)                                                                                \
+  hipLaunchKernelGGL((gate_norm_kernel<TT, W>), grid, block, 0, stream, o, gain, (const TT*)g,   \
+                     g_stride, gate_kind, (TT*)out, out_stride, rows, P, dv, eps, quads)
+  if (dtype == ZF_F32) { if (wide) GN(float, true); else GN(float, false); }
+  else { if (wide) GN(bf16_t, true); else GN(bf16_t, false); }
+  ZF_CHECK_LAUNCH();
+}

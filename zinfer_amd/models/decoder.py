@@ -12,6 +12,7 @@ from .. import ops
 from ..config.specs import ModelSpec
 from ..errors import ConfigError
 from ..parts import BuildContext, TensorDecl, build_part
+from ..parts.block import NormedRows
 from ..parts.linear import Linear, place_matrix
 
 
@@ -26,6 +27,16 @@ class DecoderModel:
         self.blocks = [build_part("block", b, ctx, spec.layer_prefix.format(n))
                        for n, b in zip(numbers, spec.layers)]
         self.final_norm = build_part("norm", spec.final_norm, ctx, spec.final_norm_prefix)
+        self.embedding_norm = None
+        if spec.embedding_norm is not None:
+            self.embedding_norm = build_part("norm", spec.embedding_norm, ctx,
+                                             spec.embedding_norm_prefix)
+            if not getattr(self.embedding_norm, "plain", False):
+                raise ConfigError("the norm of the embedding's rows is an RMS norm with a gain alone")
+            if spec.streams is not None or spec.position_table_name is not None \
+                    or spec.sinusoidal_positions is not None:
+                raise ConfigError("a norm of the embedding's rows stands with one stream and without "
+                                  "position vectors")
         self.graph_safe = self.final_norm.graph_safe and all(b.graph_safe for b in self.blocks)
         # (inspection) called with (schedule position, the stream) behind every run of a block
         self.layer_probe = None
@@ -35,6 +46,7 @@ class DecoderModel:
             | ({"norms"} if spec.position_table_name is not None or spec.streams is not None
                else set())
             | set(self.final_norm.kernel_modules)
+            | set(self.embedding_norm.kernel_modules if self.embedding_norm is not None else ())
             | {m for b in self.blocks for m in b.kernel_modules}))
         if spec.position_table_name is not None and spec.sinusoidal_positions is not None:
             raise ConfigError("a learned position table or computed position vectors, not both")
@@ -68,6 +80,8 @@ class DecoderModel:
         for b in self.blocks:
             d.update(b.declare())
         d.update(self.final_norm.declare())
+        if self.embedding_norm is not None:
+            d.update(self.embedding_norm.declare())
         d[s.head_name] = TensorDecl((s.vocab_size, s.hidden_size),
                                     optional=s.tie_word_embeddings)
         return d
@@ -94,6 +108,8 @@ class DecoderModel:
         for b in self.blocks:
             b.bind(tensors)
         self.final_norm.bind(tensors)
+        if self.embedding_norm is not None:
+            self.embedding_norm.bind(tensors)
         if s.head_name in tensors:
             self.head = Linear(place_matrix(tensors[s.head_name], self.ctx))
         else:
@@ -142,7 +158,17 @@ class DecoderModel:
             x = copies[0]
         else:
             x = step.scratch("residual", (T, s.hidden_size), torch.float32)
-        if self.position_table is not None:
+        step.norm_ready = None
+        if self.embedding_norm is not None:
+            # the rows through their norm, and through the first block's norm in the same kernel
+            first = None if s.schedule[0].reentry else \
+                getattr(self.blocks[s.schedule[0].layer], "entry_norm", None)
+            out = step.scratch("normed", (T, s.hidden_size), self.ctx.act_dtype) \
+                if first is not None else None
+            if self.embedding_norm.forward_embedding(self.embedding, step.token_ids,
+                                                     float(s.embedding_multiplier), x, first, out):
+                step.norm_ready = NormedRows(first, x, out)
+        elif self.position_table is not None:
             ops.embed_position(self.embedding, step.token_ids, self.position_table,
                                step.positions, x, float(s.embedding_multiplier))
         elif self.position_freq is not None:
@@ -159,7 +185,6 @@ class DecoderModel:
             for c in range(1, s.streams):
                 copies[c].copy_(x)
             x = copies
-        step.norm_ready = None
         for pos, e in enumerate(s.schedule):
             if e.reentry:
                 # x = W [x ; x0]: both streams side by side in the products' type, one product
@@ -172,8 +197,7 @@ class DecoderModel:
             if pos + 1 < len(s.schedule):
                 after = getattr(self.blocks[s.schedule[pos + 1].layer], "entry_norm", None)
             else:
-                after = self.final_norm if self.final_norm.defers and step.wants_all_rows \
-                    else None
+                after = self.final_norm if step.wants_all_rows else None
             if pos + 1 < len(s.schedule) and s.schedule[pos + 1].reentry:
                 after = None            # the stream is replaced before the next block reads it
             step.norm_after_block = after
@@ -195,7 +219,10 @@ class DecoderModel:
             ops.gather_rows(x, step.want_rows, rows)
         make = lambda: step.scratch("final_normed", (n_rows, s.hidden_size), self.ctx.act_dtype)
         with ops.kernel_class("head_sampling"):      # what a per-class measurement counts these as
-            normed = self.final_norm.deferred(rows, make, left)
+            if isinstance(left, NormedRows) and left.fits(self.final_norm, rows):
+                normed = left.normed          # the last block's closing kernel ran it
+            else:
+                normed = self.final_norm.deferred(rows, make, left)
             if normed is None:
                 normed = self.final_norm.forward(rows, make())
             self.head.forward(normed, logits)

@@ -1440,23 +1440,26 @@ def paged_attention(q, k_pool, v_pool, block_table, q_start, ctx_len, seq_index,
 # ------------------------------------------------------------------------- norms with a bias
 @_launches("norm_rope_write")
 def norm_rows(x: torch.Tensor, gain: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
-              out: torch.Tensor, centred: bool = True, add: bool = False) -> None:
-    """Row by row over float32 ``x`` [T, W], all in 32-bit: centred,
+              out: torch.Tensor, centred: bool = True, add: bool = False,
+              x_bias: Optional[torch.Tensor] = None) -> None:
+    """Row by row over float32 ``x`` [T, W] (plus ``x_bias`` float32 [W], if given), all in
+    32-bit: centred,
     n = (x - mean) / sqrt(mean((x - mean)^2) + eps) * gain + bias (a layer norm); not centred,
     n = x / sqrt(mean(x^2) + eps) * gain (+ bias).  ``out`` = n (float32 or bfloat16), or with
     ``add`` out += n (float32: a branch's normed output joins the residual stream)."""
-    _need_gpu(x, gain, bias, out)
+    _need_gpu(x, gain, bias, out, x_bias)
     T, W = x.shape
     if x.dtype != torch.float32 or gain.dtype != torch.float32 or gain.shape != (W,) \
-            or out.shape != x.shape or (bias is not None and (bias.dtype != torch.float32
-                                                              or bias.shape != (W,))) \
+            or out.shape != x.shape \
+            or any(b is not None and (b.dtype != torch.float32 or b.shape != (W,))
+                   for b in (bias, x_bias)) \
             or (add and out.dtype != torch.float32):
         raise KernelUnavailable(f"norm_rows: x {tuple(x.shape)} {x.dtype}, gain "
                                 f"{tuple(gain.shape)} {gain.dtype}, out {tuple(out.shape)} "
                                 f"{out.dtype} (float32 when added to)")
     lib = build.load("norms")
-    _check(lib.zf_norm_rows(_ptr(x), _ptr(gain), _ptr(bias), _ptr(out), _dt(out), T, W,
-                            ctypes.c_float(eps), 1 if centred else 0, 1 if add else 0,
+    _check(lib.zf_norm_rows(_ptr(x), _ptr(x_bias), _ptr(gain), _ptr(bias), _ptr(out), _dt(out), T,
+                            W, ctypes.c_float(eps), 1 if centred else 0, 1 if add else 0,
                             _stream()), "norm_rows")
 
 
@@ -1470,13 +1473,14 @@ def norm_add_norm_covers(width: int) -> bool:
 @_launches("norm_rope_write")
 def norm_add_norm(y: torch.Tensor, gain_a, bias_a, eps_a: float, centred_a: bool,
                   x: torch.Tensor, gain_b, bias_b, eps_b: float, centred_b: bool,
-                  out: torch.Tensor) -> None:
+                  out: torch.Tensor, y_bias: Optional[torch.Tensor] = None) -> None:
     """x += norm_a(y); out = norm_b(x), row by row in 32-bit (``norm_rows`` with ``add`` and then
     ``norm_rows``, in one kernel, the same numbers): the norm behind a sublayer and the norm
-    before the next one.  ``y`` and ``x`` float32 [T, W], W a multiple of 4 up to 8192."""
-    _need_gpu(y, gain_a, bias_a, x, gain_b, bias_b, out)
+    before the next one.  ``y`` and ``x`` float32 [T, W], W a multiple of 4 up to 8192.
+    ``y_bias`` float32 [W]: a row added to y first."""
+    _need_gpu(y, gain_a, bias_a, x, gain_b, bias_b, out, y_bias)
     T, W = x.shape
-    vecs = [v for v in (gain_a, bias_a, gain_b, bias_b) if v is not None]
+    vecs = [v for v in (gain_a, bias_a, gain_b, bias_b, y_bias) if v is not None]
     if y.shape != x.shape or out.shape != x.shape or y.dtype != torch.float32 \
             or x.dtype != torch.float32 or gain_a is None or gain_b is None \
             or any(v.dtype != torch.float32 or v.shape != (W,) for v in vecs) \
@@ -1485,10 +1489,34 @@ def norm_add_norm(y: torch.Tensor, gain_a, bias_a, eps_a: float, centred_a: bool
                                 f"{tuple(x.shape)}, float32 [W] gains and biases, W a multiple "
                                 f"of 4 up to {NORM_ADD_NORM_MAX_WIDTH}")
     lib = build.load("norms")
-    _check(lib.zf_norm_add_norm(_ptr(y), _ptr(gain_a), _ptr(bias_a), ctypes.c_float(eps_a),
+    _check(lib.zf_norm_add_norm(_ptr(y), _ptr(y_bias), _ptr(gain_a), _ptr(bias_a),
+                                ctypes.c_float(eps_a),
                                 1 if centred_a else 0, _ptr(x), _ptr(gain_b), _ptr(bias_b),
                                 ctypes.c_float(eps_b), 1 if centred_b else 0, _ptr(out), _dt(out),
                                 T, W, _stream()), "norm_add_norm")
+
+
+@_launches("other")
+def embed_norm(table: torch.Tensor, ids: torch.Tensor, gain: torch.Tensor, eps: float,
+               x: torch.Tensor, scale: float = 1.0, gain_then: Optional[torch.Tensor] = None,
+               eps_then: float = 0.0, out: Optional[torch.Tensor] = None) -> None:
+    """x[t, :] = e / sqrt(mean(e^2) + eps) * gain with e = table[ids[t], :] * scale, in 32-bit into
+    float32 ``x`` [T, W]; with ``gain_then`` the norm that reads x next runs in the same kernel,
+    ``out`` [T, W] = x / sqrt(mean(x^2) + eps_then) * gain_then.  Gains float32 [W]."""
+    _need_gpu(table, ids, gain, x, gain_then, out)
+    _i32(ids, "ids")
+    T, W = x.shape
+    if table.shape[1] != W or ids.shape[0] != T or x.dtype != torch.float32 \
+            or any(g is not None and (g.shape != (W,) or g.dtype != torch.float32)
+                   for g in (gain, gain_then)) \
+            or (gain_then is not None and (out is None or out.shape != (T, W))):
+        raise KernelUnavailable(f"embed_norm: table {tuple(table.shape)} {table.dtype}, {ids.shape[0]} "
+                                f"ids -> {tuple(x.shape)} {x.dtype}")
+    lib = build.load("norms")
+    _check(lib.zf_embed_norm(_ptr(table), _dt(table), _ptr(ids), ctypes.c_float(scale), _ptr(gain),
+                             ctypes.c_float(eps), _ptr(x), _ptr(gain_then),
+                             ctypes.c_float(eps_then), _ptr(out if gain_then is not None else None),
+                             _dt(out) if gain_then is not None else 0, T, W, _stream()), "embed_norm")
 
 
 @_launches("other")
@@ -2032,6 +2060,25 @@ def bias_act_rows(x: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tens
     _check(lib.zf_bias_act_rows(_ptr(x), _dt(x), ctypes.c_longlong(xs), _ptr(bias), _ptr(out),
                                 ctypes.c_longlong(os_), T, n, ACTIVATIONS[kind], int(tail),
                                 int(ones), _stream()), "bias_act_rows")
+
+
+@_launches("norm_rope_write")
+def gated_rows(x: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor, kind: str) -> None:
+    """out = act(x[:, :n] + bias[:n]) * (x[:, n:2 n] + bias[n:]) in 32-bit: ``x`` [T, >= 2 n] (any
+    row stride), the rows of a product over a gate's and an up projection's stacked rows,
+    ``bias`` float32 [2 n] or None, ``out`` [T, n] in x's type; ``kind`` as for ``activation``."""
+    _need_gpu(bias, out)
+    if not x.is_cuda:
+        raise KernelUnavailable("the HIP kernels run on GPU tensors only")
+    T, n = out.shape
+    if kind not in ACTIVATIONS or x.shape[0] != T or x.shape[1] < 2 * n or out.dtype != x.dtype \
+            or (bias is not None and (bias.shape != (2 * n,) or bias.dtype != torch.float32)):
+        raise KernelUnavailable(f"gated_rows: {tuple(x.shape)} {x.dtype} -> {tuple(out.shape)} "
+                                f"{out.dtype}, kind {kind!r} of {sorted(ACTIVATIONS)}")
+    lib = build.load("elementwise")
+    _check(lib.zf_gated_rows(_ptr(x), _dt(x), ctypes.c_longlong(_columns(x, "gated_rows: x")),
+                             _ptr(bias), _ptr(out), T, n, ACTIVATIONS[kind], _stream()),
+           "gated_rows")
 
 
 @_launches("norm_rope_write")
@@ -2652,6 +2699,32 @@ def head_norm_gate(o: torch.Tensor, gain: Optional[torch.Tensor], gate: torch.Te
                                  T, H, dv, ctypes.c_float(eps), _stream()), "head_norm_gate")
 
 
+@_launches("norm_rope_write")
+def gate_norm(o: torch.Tensor, gain: torch.Tensor, gate: torch.Tensor, out: torch.Tensor,
+              parts: int, eps: float, gate_kind: str = "silu") -> None:
+    """The gate first, then the norm: u = o * act(gate), and every one of ``parts`` equal parts of
+    a row over its own root mean square, times ``gain`` float32 [width].  ``o`` float32 [T,
+    width]; ``gate`` and ``out`` [T, width] (contiguous rows, any row stride) in the products'
+    type; ``gate_kind`` as for ``head_norm_gate``.  All in 32-bit."""
+    _need_gpu(o, gain)
+    if not gate.is_cuda or not out.is_cuda:
+        raise KernelUnavailable("the HIP kernels run on GPU tensors only")
+    T, width = o.shape
+    P = int(parts)
+    if P < 1 or width % P != 0 or o.dtype != torch.float32 or gate_kind not in GATE_KINDS \
+            or gain.dtype != torch.float32 or gain.shape != (width,) \
+            or gate.shape != (T, width) or out.shape != (T, width) or gate.dtype != out.dtype:
+        raise KernelUnavailable(f"gate_norm: o {tuple(o.shape)} {o.dtype}, gain "
+                                f"{tuple(gain.shape)}, gate {tuple(gate.shape)} {gate.dtype}, out "
+                                f"{tuple(out.shape)} {out.dtype}, {P} parts, gate {gate_kind!r}")
+    lib = build.load("recurrent")
+    _check(lib.zf_gate_norm(_ptr(o), _ptr(gain), _ptr(gate),
+                            ctypes.c_longlong(_columns(gate, "gate_norm: gate")),
+                            GATE_KINDS[gate_kind], _ptr(out),
+                            ctypes.c_longlong(_columns(out, "gate_norm: out")), _dt(out), T, P,
+                            width // P, ctypes.c_float(eps), _stream()), "gate_norm")
+
+
 # ------------------------------------------------------------------------- linear attention with a fixed decay a head
 FIXED_DECAY_MAX_KEY_DIM = 256
 FIXED_DECAY_CHUNK = 128          # FC_C in fixed_decay.hip
@@ -2879,16 +2952,18 @@ def delta_state_matrix(state: torch.Tensor, n_heads: int, key_dim: int,
 def short_conv(src: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, state_offset: int,
                state_slots: torch.Tensor, seq_index: torch.Tensor, q_start: torch.Tensor,
                out: torch.Tensor, unit_heads: int = 0, head_dim: int = 1, scaled_heads: int = 0,
-               scale: float = 1.0, unit_eps: float = 0.0, single_tokens: bool = False) -> None:
-    """out[t, c] = silu(sum_j taps[c, j] * x_(t - n + 1 + j)[c]) over the rows of a step: ``src``
-    [T, >= C] (contiguous rows, any row stride), ``taps`` float32 [C, n] (the last column is the
-    token's own), ``out`` float32 [T, C].  Rows before a sequence's portion come from its state:
+               scale: float = 1.0, unit_eps: float = 0.0, single_tokens: bool = False,
+               bias: Optional[torch.Tensor] = None) -> None:
+    """out[t, c] = silu(sum_j taps[c, j] * x_(t - n + 1 + j)[c] + bias[c]) over the rows of a
+    step: ``src`` [T, >= C] (contiguous rows, any row stride), ``taps`` float32 [C, n] (the last
+    column is the token's own), ``bias`` float32 [C] or None, ``out`` [T, C] in float32 or the
+    rows' type.  Rows before a sequence's portion come from its state:
     [n - 1, C] floats from ``state_offset`` on in row state_slots[s] of ``state`` (float32
     [slots, width]), oldest first; zeros for a new request.  After the step the state holds the
     last n - 1 rows seen.  The leading ``unit_heads`` * ``head_dim`` channels are heads that
     leave as unit vectors x / sqrt(sum x^2 + unit_eps), the first ``scaled_heads`` of them times
     ``scale``.  ``single_tokens``: every sequence brings one token (one launch instead of two)."""
-    _need_gpu(taps, state, state_slots, seq_index, q_start, out)
+    _need_gpu(taps, state, state_slots, seq_index, q_start, out, bias)
     if not src.is_cuda:
         raise KernelUnavailable("the HIP kernels run on GPU tensors only")
     for t, name in ((state_slots, "state_slots"), (seq_index, "seq_index"), (q_start, "q_start")):
@@ -2897,7 +2972,8 @@ def short_conv(src: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, state
     C, n = taps.shape
     n_seqs = state_slots.shape[0]
     if taps.dtype != torch.float32 or not taps.is_contiguous() or src.shape[1] < C \
-            or out.shape != (T, C) or out.dtype != torch.float32 or not out.is_contiguous() \
+            or out.shape != (T, C) or out.dtype not in (torch.float32, src.dtype) \
+            or (bias is not None and (bias.shape != (C,) or bias.dtype != torch.float32)) \
             or state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 \
             or state_offset < 0 or state_offset + (n - 1) * C > state.shape[1] \
             or seq_index.shape[0] != T or q_start.shape[0] != n_seqs + 1 \
@@ -2909,9 +2985,10 @@ def short_conv(src: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, state
                                 f"{tuple(state.shape)} from {state_offset}")
     lib = build.load("delta")
     _check(lib.zf_short_conv(_ptr(src), _dt(src), ctypes.c_longlong(_columns(src, "short_conv: src")),
-                             _ptr(taps), n, _ptr(state), ctypes.c_longlong(state.stride(0)),
-                             ctypes.c_longlong(state_offset), _ptr(state_slots), _ptr(seq_index),
-                             _ptr(q_start), _ptr(out), T, n_seqs, C, int(unit_heads),
+                             _ptr(taps), n, _ptr(bias), _ptr(state),
+                             ctypes.c_longlong(state.stride(0)), ctypes.c_longlong(state_offset),
+                             _ptr(state_slots), _ptr(seq_index), _ptr(q_start), _ptr(out),
+                             _dt(out), T, n_seqs, C, int(unit_heads),
                              int(head_dim), int(scaled_heads), ctypes.c_float(scale),
                              ctypes.c_float(unit_eps), 1 if single_tokens else 0, _stream()),
            "short_conv")
@@ -2964,3 +3041,106 @@ def delta_recurrence(qkv: torch.Tensor, q_off: int, k_off: int, v_off: int, ab: 
                                    ctypes.c_longlong(state.stride(0)), _ptr(state_slots),
                                    _ptr(q_start), _ptr(out), n_seqs, H, KH, d, dv, r, lanes, cols,
                                    _stream()), "delta_recurrence")
+
+
+# ------------------------------------------------------------------------- a state space with one decay a head and token
+STATE_SPACE_MAX_STATE = 256      # channels of a head's state (the lanes that share a value column)
+STATE_SPACE_HEADS_MAX = 4        # SS_HEADS_MAX in state_space.hip
+STATE_SPACE_WORKGROUPS = 512     # a workgroup takes more heads while at least this many are left
+
+
+def state_space_state_size(n_heads: int, state_dim: int, value_dim: int) -> int:
+    """32-bit numbers a request's matrices take: [head][value column][channels padded to 4]."""
+    return n_heads * value_dim * ((state_dim + 3) // 4 * 4)
+
+
+def state_space_state_matrix(state: torch.Tensor, n_heads: int, state_dim: int,
+                             value_dim: int) -> torch.Tensor:
+    """The matrices S [.., head, channel, value column] of states as the kernels keep them (tests
+    and inspection)."""
+    return fixed_decay_state_matrix(state, n_heads, state_dim, value_dim)
+
+
+def state_space_heads(n_chunks: int, n_heads: int, n_groups: int, value_dim: int) -> int:
+    """Heads of a group that a workgroup of the chunked form takes one after the other (they share
+    the group's staged rows): the largest of 1, 2 and 4 that divides them and leaves enough
+    workgroups."""
+    blocks = (value_dim + 63) // 64
+    best = 1
+    for heads in (2, STATE_SPACE_HEADS_MAX):
+        if (n_heads // n_groups) % heads == 0 \
+                and n_chunks * (n_heads // heads) * blocks >= STATE_SPACE_WORKGROUPS:
+            best = heads
+    return best
+
+
+@_launches("attention")
+def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, steps: torch.Tensor,
+                decay_log: torch.Tensor, step_bias: torch.Tensor, skip: torch.Tensor,
+                state: torch.Tensor, state_slots: torch.Tensor, q_start: torch.Tensor,
+                out: torch.Tensor, n_heads: int, n_groups: int, state_dim: int, value_dim: int, *,
+                lists=None, heads: Optional[int] = None) -> None:
+    """dt_t = softplus(steps_t + step_bias), S_t = exp(-exp(decay_log) dt_t) S_(t-1) + dt_t b_t
+    x_t^T, out_t = S_t^T c_t + skip x_t a head, in 32-bit, over the rows of a step: ``x`` [T, >= H
+    * dv], ``b`` and ``c`` [T, >= G * N] (contiguous rows, any row stride, that of b and c the
+    same; head h reads group floor(h / (H / G))), ``steps`` float32 [T, H], ``decay_log``,
+    ``step_bias`` and ``skip`` float32 [H], ``out`` float32 [T, H * dv].  Sequence s owns the rows
+    q_start[s] .. q_start[s + 1] - 1; its matrices (the leading ``state_space_state_size`` floats
+    of row state_slots[s] of ``state``) are read before its first row and written behind its last.
+
+    ``lists`` (bfloat16 only): the int32 tensors of ``fixed_decay_chunk_lists``; long sequences
+    then run in chunks side by side through MFMAs, where an operand that is a 32-bit number
+    enters as two bfloat16 terms (``heads``: how many heads a workgroup takes, None: by
+    ``state_space_heads``).  None: token by token, all 32-bit, every size and both types (the
+    same bits however a sequence is cut into steps)."""
+    _need_gpu(steps, decay_log, step_bias, skip, state_slots, q_start, out)
+    for t in (x, b, c, state):
+        if not t.is_cuda:
+            raise KernelUnavailable("the HIP kernels run on GPU tensors only")
+    _i32(state_slots, "state_slots")
+    _i32(q_start, "q_start")
+    T = x.shape[0]
+    H, G, N, dv = int(n_heads), int(n_groups), int(state_dim), int(value_dim)
+    n_seqs = state_slots.shape[0]
+    if min(H, G, N, dv) < 1 or H % G != 0 or N > STATE_SPACE_MAX_STATE:
+        raise KernelUnavailable(f"state_space: {H} heads of {dv} in {G} groups with {N} channels "
+                                f"(up to {STATE_SPACE_MAX_STATE})")
+    need = state_space_state_size(H, N, dv)
+    xs, bs = _columns(x, "state_space: x"), _columns(b, "state_space: b")
+    if x.shape[1] < H * dv or b.shape[1] < G * N or c.shape[1] < G * N or b.shape[0] != T \
+            or c.shape[0] != T or b.dtype != x.dtype or c.dtype != x.dtype \
+            or (T > 1 and _columns(c, "state_space: c") != bs) \
+            or steps.shape != (T, H) or steps.dtype != torch.float32 \
+            or any(v.shape != (H,) or v.dtype != torch.float32 for v in (decay_log, step_bias, skip)) \
+            or out.shape != (T, H * dv) or out.dtype != torch.float32 \
+            or state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 \
+            or state.shape[1] < need or state.stride(0) % 4 != 0 or state.data_ptr() % 16 != 0 \
+            or q_start.shape[0] != n_seqs + 1 \
+            or (lists is not None and x.dtype != torch.bfloat16):
+        raise KernelUnavailable(f"state_space: x {tuple(x.shape)}, b {tuple(b.shape)}, c "
+                                f"{tuple(c.shape)} {x.dtype}, steps {tuple(steps.shape)}, out "
+                                f"{tuple(out.shape)} {out.dtype}, state {tuple(state.shape)} "
+                                f"{state.dtype} (rows a multiple of 4 floats, at least {need})")
+    lib = build.load("state_space")
+    rows = (_ptr(x), ctypes.c_longlong(xs), _ptr(b), _ptr(c), ctypes.c_longlong(bs))
+    head = (_ptr(steps), _ptr(decay_log), _ptr(step_bias), _ptr(skip), _ptr(state),
+            ctypes.c_longlong(state.stride(0)), _ptr(state_slots))
+    shorts, n_short = None, n_seqs
+    if lists is not None:
+        chunks, firsts, shorts = lists
+        for t in (chunks, firsts, shorts):
+            if t is not None:
+                _i32(t, "state_space: lists")
+        n_chunks, n_long = chunks.shape[0], firsts.shape[0]
+        n_short = 0 if shorts is None else shorts.shape[0]
+        states = _workspace("state_space_states", n_chunks * need, torch.float32, x.device)
+        decays = _workspace("state_space_decays", n_chunks * H * FIXED_DECAY_CHUNK * 2,
+                            torch.float32, x.device)
+        hb = int(heads) if heads is not None else state_space_heads(n_chunks, H, G, dv)
+        _check(lib.zf_state_space_chunks(*rows, *head, _ptr(chunks), n_chunks, _ptr(firsts), n_long,
+                                         _ptr(states), _ptr(decays), _ptr(out), H, G, N, dv, hb,
+                                         _stream()), "state_space (chunks)")
+    if n_short:
+        _check(lib.zf_state_space_walk(
+            *rows, _dt(x), *head, _ptr(q_start), _ptr(shorts), _ptr(out), n_short, H, G, N, dv,
+            _stream()), "state_space (token by token)")

@@ -25,9 +25,10 @@ from ..errors import KernelUnavailable
 
 CSRC = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file__))), "csrc")
 MODULES = ("elementwise", "gemm", "attention", "sampling", "randinit", "norms",
-           "sink_attention", "moe", "masked_attention", "recurrent", "delta", "fixed_decay")
+           "sink_attention", "moe", "masked_attention", "recurrent", "delta", "fixed_decay",
+           "state_space")
 HOST_MODULES = ("cache_core",)
-HEADERS = ("zf_common.h", "zf_no_alloc.h")
+HEADERS = ("zf_common.h", "zf_no_alloc.h", "zf_chunks.h")
 HOST_FLAGS = ["-O2", "-std=c++17", "-fPIC", "-shared", "-Wall"]
 # -packed-fp32-ops off: hipcc must not form packed 32-bit float instructions by itself
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared",

@@ -12,6 +12,7 @@ from typing import Callable, Dict
 from . import (gated_act, moe_grouped, norm_add_norm, tied_attention_mfma)
 from . import delta_recurrence, short_conv, streams_step
 from . import add_row, bias_act_rows, fixed_decay, rotation_table
+from . import embed_norm, gate_norm, gated_rows, state_space
 from . import (concat_rows, decay_recurrence, embed_sinusoid, head_norm_gate, token_shift_mix)
 from . import (activation, head_products, masked_attention, masked_attention_mfma,
                norm_add_store, project_rows)
@@ -125,6 +126,13 @@ KERNELS: Dict[str, KernelEntry] = {
     "bias_act_rows": KernelEntry(bias_act_rows, "elementwise", "own: an activation behind a bias "
                                  "a column, over slices of wider rows"),
     "add_row": KernelEntry(add_row, "elementwise", "own: one row added to every row"),
+    "embed_norm": KernelEntry(embed_norm, "norms", "own: embedding rows through an RMS norm, and "
+                              "the norm that reads them next"),
+    "gated_rows": KernelEntry(gated_rows, "elementwise", "own: a gated activation behind biases"),
+    "gate_norm": KernelEntry(gate_norm, "recurrent", "own: a gate, then an RMS norm over equal "
+                             "parts of a row"),
+    "state_space": KernelEntry(state_space, "state_space", "own: a matrix a head with one decay a "
+                               "head and token, token by token or in chunks side by side"),
     "mfma_loop": KernelEntry(mfma_loop, "gemm",
                              "own: MFMAs alone, the rate the tiled products are measured against"),
 }

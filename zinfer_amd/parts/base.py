@@ -21,7 +21,10 @@ Roles and what each must provide:
                   ``accumulate=False`` and then stores it there instead; optionally ``step_hints`` (what its kernels want
                   to know about a step's shape, packed with the step's metadata),
                   ``graph_table_pages`` and ``accept_cache``
-* feed_forward    ``forward(h[T, H], residual_f32[T, H], step)`` adds its output to ``residual``
+* feed_forward    ``forward(h[T, H], residual_f32[T, H], step)`` adds its output to ``residual``; a
+                  part whose output has a bias may say ``leaves_bias``: with ``accumulate=False,
+                  leave_bias=True`` it stores the output without it and returns it, for a norm
+                  behind it that takes it in (``Norm.adds_input_bias``)
 * block           ``forward(x_f32[T, H], step, cache)`` in place on the residual stream
 """
 from __future__ import annotations
@@ -185,6 +188,8 @@ class Norm(Part):
       returns True, or returns False and does nothing."""
     role = "norm"
     defers = False         # whether ``deferred`` can ever give a stand-in
+    # whether ``forward_add`` takes ``x_bias`` [W], a row added to what the norm reads
+    adds_input_bias = False
 
     def forward(self, x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
         raise NotImplementedError

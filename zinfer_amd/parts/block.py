@@ -80,7 +80,8 @@ class SandwichNormBlock(Block):
     one behind it, ahead of the residual sum.  A sublayer's output is a float32 branch of its
     own (a part that says ``stores_output`` stores it there; any other part adds it to a
     branch that was cleared first); the norm behind it reads the branch and adds its result to
-    the stream in one kernel, in 32-bit.  Without a feed-forward the block is its first line."""
+    the stream in one kernel, in 32-bit (a part that ``leaves_bias`` leaves its output's bias to
+    that kernel).  Without a feed-forward the block is its first line."""
 
     def __init__(self, spec: SandwichNormBlockSpec, ctx, prefix):
         super().__init__(spec, ctx, prefix)
@@ -133,7 +134,11 @@ class SandwichNormBlock(Block):
         else:
             h = norm.forward(x, step.scratch("normed", x.shape, self.ctx.act_dtype))
         branch = step.scratch("branch", x.shape, torch.float32)
-        if getattr(part, "stores_output", False):
+        given = {}
+        if getattr(part, "leaves_bias", False) and post.adds_input_bias:
+            given["x_bias"] = part.forward(h, branch, step, *args, accumulate=False,
+                                           leave_bias=True)
+        elif getattr(part, "stores_output", False):
             part.forward(h, branch, step, *args, accumulate=False)
         else:
             branch.zero_()
@@ -143,9 +148,9 @@ class SandwichNormBlock(Block):
         if then is not None and fused is not None:
             # (the mixer or feed-forward is done with the buffer its input lay in)
             out = step.scratch("normed", x.shape, self.ctx.act_dtype)
-            if fused(branch, x, then, out):
+            if fused(branch, x, then, out, **given):
                 return out
-        post.forward_add(branch, x)
+        post.forward_add(branch, x, **given)
         return None
 
     def forward(self, x, step, cache) -> None:

@@ -5,7 +5,8 @@ from typing import Dict
 import torch
 
 from .. import ops
-from ..config.specs import DenseMlpSpec, SwiGluSpec
+from ..config.specs import DenseMlpSpec, GatedMlpSpec, SwiGluSpec
+from ..errors import ConfigError
 from .base import FeedForward, TensorDecl, register_part
 from .linear import Linear, place_gain, place_matrix
 
@@ -96,7 +97,6 @@ class DenseMlp(FeedForward):
     def bind_joined(self, tensors) -> None:
         s, p = self.spec, self.prefix
         if s.activation not in ops.ACTIVATIONS:
-            from ..errors import ConfigError
             raise ConfigError(f"activation {s.activation!r}: known are {sorted(ops.ACTIVATIONS)}")
         self.up_bias = place_gain(tensors[p + s.up_name + s.bias_suffix], self.ctx) \
             if s.bias else None
@@ -128,5 +128,65 @@ class DenseMlp(FeedForward):
         ops.bias_act_rows(rows, self.up_bias, out, self.spec.activation, tail=tail, ones=ones)
 
 
+class GatedMlp(FeedForward):
+    """d = W_down (act(W_gate m) * W_up m) with any of ``ops.ACTIVATIONS`` and, if the
+    specification says so, biases on all three.  gate and up rows are stacked into one matrix at
+    load: each output keeps its own dot product; biases, activation and the product of the two
+    run in 32-bit on the product's rows.  The output's bias may be left to a norm behind the
+    part."""
+    graph_safe = True
+    stores_output = True
+    leaves_bias = True
+    kernel_modules = ("elementwise", "gemm")
+
+    def __init__(self, spec: GatedMlpSpec, ctx, prefix):
+        super().__init__(spec, ctx, prefix)
+        if spec.activation not in ops.ACTIVATIONS:
+            raise ConfigError(f"activation {spec.activation!r}: known are {sorted(ops.ACTIVATIONS)}")
+
+    def declare(self) -> Dict[str, TensorDecl]:
+        s, p = self.spec, self.prefix
+        d = {p + s.gate_name: TensorDecl((s.intermediate_size, s.hidden_size)),
+             p + s.up_name: TensorDecl((s.intermediate_size, s.hidden_size)),
+             p + s.down_name: TensorDecl((s.hidden_size, s.intermediate_size))}
+        if s.bias:
+            for name, width in ((s.gate_name, s.intermediate_size),
+                                (s.up_name, s.intermediate_size), (s.down_name, s.hidden_size)):
+                d[p + name + s.bias_suffix] = TensorDecl((width,))
+        return d
+
+    def bind(self, tensors) -> None:
+        s, p = self.spec, self.prefix
+        g, u = tensors[p + s.gate_name], tensors[p + s.up_name]
+        if g.dtype != u.dtype:
+            g, u = g.float(), u.float()
+        self.gate_up = Linear(place_matrix(torch.cat([g, u], dim=0), self.ctx))
+        self.down = Linear(place_matrix(tensors[p + s.down_name], self.ctx))
+        self.bias = self.down_bias = None
+        if s.bias:
+            self.bias = place_gain(torch.cat([tensors[p + n + s.bias_suffix].to(torch.float32)
+                                              for n in (s.gate_name, s.up_name)]), self.ctx)
+            self.down_bias = place_gain(tensors[p + s.down_name + s.bias_suffix], self.ctx)
+
+    def forward(self, h, residual, step, accumulate: bool = True, leave_bias: bool = False):
+        T, I = h.shape[0], self.spec.intermediate_size
+        act = self.ctx.act_dtype
+        if hasattr(h, "materialize"):
+            h = h.materialize()
+        a = step.scratch("ff_act", (T, I), act)
+        gu = step.scratch("gate_up", (T, 2 * I), act)
+        self.gate_up.forward(h, gu)
+        ops.gated_rows(gu, self.bias, a, self.spec.activation)
+        last = self.down_bias is None
+        self.down.forward(a, residual, accumulate=accumulate,
+                          step=step if accumulate and last else None)
+        if leave_bias:
+            return self.down_bias
+        if not last:
+            ops.add_row(residual, self.down_bias)
+        return None
+
+
 register_part("feed_forward", SwiGluSpec, SwiGluMlp)
+register_part("feed_forward", GatedMlpSpec, GatedMlp)
 register_part("feed_forward", DenseMlpSpec, DenseMlp)

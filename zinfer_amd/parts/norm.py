@@ -129,8 +129,9 @@ class LayerNorm(Norm):
     """n = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b, all in 32-bit; reads the float32
     residual stream (or a branch's float32 output), writes the activation dtype, or adds its
     result to a float32 destination (``forward_add``: a norm after a sublayer, ahead of the
-    residual sum).  Not centred it is an RMS norm with a bias."""
+    residual sum; the sublayer's output bias, if it leaves one, joins on the way in).  Not centred it is an RMS norm with a bias."""
     graph_safe = True
+    adds_input_bias = True
     kernel_modules = ("norms",)
 
     def declare(self) -> Dict[str, TensorDecl]:
@@ -155,10 +156,25 @@ class LayerNorm(Norm):
         ops.norm_rows(x, self.gain, self.bias, float(self.spec.eps), out, bool(self.spec.centred))
         return out
 
-    def forward_add(self, x: torch.Tensor, residual: torch.Tensor) -> None:
-        """residual += norm(x), in 32-bit."""
+    def forward_add(self, x: torch.Tensor, residual: torch.Tensor, x_bias=None) -> None:
+        """residual += norm(x + x_bias), in 32-bit."""
         ops.norm_rows(x, self.gain, self.bias, float(self.spec.eps), residual,
-                      bool(self.spec.centred), add=True)
+                      bool(self.spec.centred), add=True, x_bias=x_bias)
+
+    def forward_embedding(self, table: torch.Tensor, ids: torch.Tensor, scale: float,
+                          x: torch.Tensor, then: "Norm" = None, out: torch.Tensor = None) -> bool:
+        """x = norm(table[ids] * scale) in one kernel, and where ``then`` is a norm of this kind
+        (neither centred nor with a bias) out = then(x) in the same; says whether it was."""
+        fused = out is not None and isinstance(then, LayerNorm) and then.plain
+        ops.embed_norm(table, ids, self.gain, float(self.spec.eps), x, scale,
+                       then.gain if fused else None, float(then.spec.eps) if fused else 0.0,
+                       out if fused else None)
+        return fused
+
+    @property
+    def plain(self) -> bool:
+        """An RMS norm with a gain and nothing else."""
+        return not self.spec.centred and self.spec.bias_name is None
 
     def forward_add_store(self, x: torch.Tensor, residual: torch.Tensor,
                           out: torch.Tensor) -> bool:
@@ -172,15 +188,15 @@ class LayerNorm(Norm):
         return True
 
     def forward_add_then(self, x: torch.Tensor, residual: torch.Tensor, then: "Norm",
-                         out: torch.Tensor) -> bool:
-        """residual += norm(x) and out = then(residual) in one kernel, if ``then`` is a norm of
-        this kind and the width allows; False (and nothing done) otherwise."""
+                         out: torch.Tensor, x_bias=None) -> bool:
+        """residual += norm(x + x_bias) and out = then(residual) in one kernel, if ``then`` is a
+        norm of this kind and the width allows; False (and nothing done) otherwise."""
         if not isinstance(then, LayerNorm) or not residual.is_cuda \
                 or not ops.norm_add_norm_covers(residual.shape[1]):
             return False
         ops.norm_add_norm(x, self.gain, self.bias, float(self.spec.eps), bool(self.spec.centred),
                           residual, then.gain, then.bias, float(then.spec.eps),
-                          bool(then.spec.centred), out)
+                          bool(then.spec.centred), out, y_bias=x_bias)
         return True
 
 
