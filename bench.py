@@ -1871,11 +1871,330 @@ def main_fumanex(args) -> int:
     return 0
 
 
+# --------------------------------------------------------------------------- Tigesun beside Qwen3
+# Layer sizes that resemble served hybrids: attention heads of 128 with a stretched rotation, latent
+# attention behind a window of 1024, state-space layers of twice the width in heads of 64 with 128
+# channels and 4 taps and no feed-forward of their own, gated feed-forwards four times the width.
+# Every shape is run beside the dense Qwen3 decoder of the same width, depth, vocabulary and
+# attention heads whose feed-forward makes the matrix work a token equal; the kernels alone stand
+# beside the like kernels of that decoder and of the closest designs: Lodenex (attention, latent
+# attention), Fumanex (a decayed recurrence in chunks, the norm with a gate), Kugisun (convolutions).
+def _tg_attention(heads, kv):
+    return ("attention", dict(heads=heads, kv_heads=kv, dim=128, vdim=128, scale=128 ** -0.5,
+                              rot=dict(base=10000.0, dims=128,
+                                       scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0))))
+
+
+def _tg_latent(heads, window=1024):
+    return ("latent_attention", dict(heads=heads, dim=128, vdim=128, kv_rank=128,
+                                     scale=128 ** -0.5, mask=dict(size=window)))
+
+
+def _tg_space(heads, groups):
+    return ("mamba2", dict(heads=heads, vdim=64, state=128, groups=groups, conv=4,
+                           norm_groups=groups))
+
+
+TIGESUN_SHAPES = {
+    "medium": dict(width=2048, vocab=32768, heads=16, kv_heads=4, ff=8192, layers=[
+        _tg_attention(16, 4), _tg_space(64, 1), _tg_latent(16), _tg_space(64, 1)]),
+    "wide": dict(width=4096, vocab=32768, heads=32, kv_heads=8, ff=14336, layers=[
+        _tg_attention(32, 8), _tg_space(128, 8), _tg_latent(32), _tg_space(128, 8)]),
+}
+
+
+def tigesun_config(sh: dict) -> dict:
+    return {"architecture": "Tigesun", "vocab": sh["vocab"], "width": sh["width"],
+            "norm": {"eps": 1e-6}, "logit_softcap": 30.0,
+            "layers": [{"type": kind, "mixer": dict(m), "mlp": None if kind == "mamba2" else
+                        {"kind": "dense", "ff": sh["ff"]}} for kind, m in sh["layers"]]}
+
+
+def tigesun_matrix_numbers(sh: dict) -> int:
+    """Numbers in the matrices that every token meets, all layers together."""
+    W, total = sh["width"], 0
+    for kind, m in sh["layers"]:
+        if kind == "mamba2":
+            inner = m["heads"] * m["vdim"]
+            total += W * (3 * inner + 2 * m["groups"] * m["state"] + m["heads"])
+            continue
+        q, v = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+        if kind == "attention":
+            total += W * (q + v + m["kv_heads"] * (m["dim"] + m["vdim"]))
+        else:
+            total += W * (q + v + m["kv_rank"]) + m["kv_rank"] * (q + v)
+        total += 3 * W * sh["ff"]
+    return total
+
+
+def tigesun_twin(sh: dict, max_positions: int) -> dict:
+    W, n = sh["width"], len(sh["layers"])
+    attn = 2 * W * (sh["heads"] + sh["kv_heads"]) * 128
+    ff = (tigesun_matrix_numbers(sh) // n - attn) // (3 * W) // 64 * 64
+    return dict(architectures=["Qwen3ForCausalLM"], model_type="qwen3", num_hidden_layers=n,
+                hidden_size=W, num_attention_heads=sh["heads"], num_key_value_heads=sh["kv_heads"],
+                head_dim=128, intermediate_size=ff, vocab_size=sh["vocab"], rope_theta=1000000.0,
+                rms_norm_eps=1e-6, tie_word_embeddings=True,
+                max_position_embeddings=max_positions, torch_dtype="bfloat16")
+
+
+def tigesun_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float) -> dict:
+    """The design's kernels alone beside the like kernels of other designs, at ``T`` tokens of one
+    sequence that holds ``ctx`` tokens (T = ctx: a prompt; T = 1 x 8 sequences: a decode step).
+    Every figure has the fraction of its roofline it reaches: the larger of the matrix work at the
+    MFMA loop's rate and the bytes at the measured read stream, over the time."""
+    import torch
+    import zinfer_amd.ops as ops
+    dev = "cuda:0"
+    W, nH, nKV, hd, ff = sh["width"], sh["heads"], sh["kv_heads"], 128, sh["ff"]
+    bf = torch.bfloat16
+    decode = T == 1
+    n_seqs = 8 if decode else 1
+    rows = n_seqs * T
+    g = torch.Generator(device=dev).manual_seed(1)
+    rnd = lambda *shape: (torch.randn(shape, generator=g, device=dev) * 0.05).to(bf)
+    f32 = lambda *shape: torch.randn(shape, generator=g, device=dev)
+    i32 = lambda a: torch.tensor(a, dtype=torch.int32, device=dev)
+    pages = (ctx + PAGE - 1) // PAGE
+    table = torch.arange(n_seqs * pages, dtype=torch.int32, device=dev).view(n_seqs, pages)
+    q_start = i32([i * T for i in range(n_seqs + 1)])
+    ctx_len = i32([ctx] * n_seqs)
+    seq_index = i32([i for i in range(n_seqs) for _ in range(T)])
+    positions = i32([ctx - T + t for _ in range(n_seqs) for t in range(T)])
+    slots = i32([(s * pages) * PAGE + ctx - T + t for s in range(n_seqs) for t in range(T)])
+    state_slots = i32(list(range(n_seqs)))
+    out = {}
+
+    def roof(t, flops, nbytes):
+        return round(max(flops / mfma_rate, nbytes / read_bw) / t, 4)
+
+    def row(name, t_new, flops, nbytes, **like):
+        r = {"tigesun_us": round(t_new * 1e6, 1), "tigesun_frac": roof(t_new, flops, nbytes)}
+        for label, (t, fl, nb) in like.items():
+            r[label + "_us"] = round(t * 1e6, 1)
+            r[label + "_frac"] = roof(t, fl, nb)
+        out[name] = r
+
+    # ---- attention over every earlier key
+    q = rnd(rows, nH * hd)
+    k_pool, v_pool = rnd(n_seqs * pages, nKV * PAGE * hd), rnd(n_seqs * pages, nKV * PAGE * hd)
+    o = torch.empty((rows, nH * hd), dtype=bf, device=dev)
+    sink, gate = torch.zeros((nH,), device=dev), rnd(rows, nH)
+    work = (0.0, n_seqs * ctx * nKV * 2 * hd * 2) if decode else \
+        (2.0 * T * (T + 1) * hd * nH, rows * (nH + nKV) * 2 * hd * 2)
+    attend = lambda cap, snk, gt: _timed_graph(lambda: ops.attend_masked(
+        q, gt, "head" if gt is not None else None, k_pool, v_pool, snk, table, q_start, ctx_len,
+        seq_index, o, hd ** -0.5, cap, 0, 0, nH, nKV, hd, hd, PAGE, T, ctx))
+    t_new, t_lx = attend(0.0, None, None), attend(30.0, sink, gate)
+    t_q3 = _timed_graph(lambda: ops.paged_attention(
+        q, k_pool, v_pool, table, q_start, ctx_len, seq_index, o, hd ** -0.5, 0, nH, nKV, hd, PAGE,
+        T, ctx))
+    row("attention", t_new, *work, lodenex=(t_lx, *work), qwen3=(t_q3, *work))
+    # ---- its projection's rows: a norm a head, the rotation, into the cache
+    width = (nH + 2 * nKV) * hd
+    proj = rnd(rows, width)
+    ones = torch.ones((hd,), device=dev)
+    freq = torch.rand((hd // 2,), generator=g, device=dev)
+    per = dict(gain=ones, eps=1e-6, hd=hd, per_head=True, rot_dims=hd, freq=freq)
+    segs = [ops.RowSegment(0, nH * hd, q, **per),
+            ops.RowSegment(nH * hd, nKV * hd, k_pool, pool_heads=nKV, **per),
+            ops.RowSegment((nH + nKV) * hd, nKV * hd, v_pool, hd=hd, pool_heads=nKV)]
+    t_new = _timed_graph(lambda: ops.project_rows(proj, positions, slots, PAGE, segs))
+    gq, gk = torch.ones((nH * hd,), device=dev), torch.ones((nKV * hd,), device=dev)
+    lx = dict(eps=1e-6, hd=hd, rot_dims=hd // 2, freq=freq[:hd // 4].contiguous())
+    lsegs = [ops.RowSegment(0, nH * hd, q, gain=gq, **lx),
+             ops.RowSegment(nH * hd, nKV * hd, k_pool, gain=gk, pool_heads=nKV, **lx), segs[2]]
+    t_lx = _timed_graph(lambda: ops.project_rows(proj, positions, slots, PAGE, lsegs))
+    cos = torch.rand((ctx + 1, hd // 2), generator=g, device=dev)
+    t_q3 = _timed_graph(lambda: ops.qk_norm_rope_kv_write(
+        proj, ones, ones, 1e-6, cos, cos, positions, slots, k_pool, v_pool, q, nH, nKV, hd, PAGE))
+    work = (0.0, rows * width * 4)
+    row("norm_rotate_store", t_new, *work, lodenex=(t_lx, *work), qwen3=(t_q3, *work))
+    # ---- latent attention behind its window (Lodenex's: a rotated part of 32 beside the latent)
+    latent = dict(sh["layers"])["latent_attention"]
+    H, R, window = latent["heads"], latent["kv_rank"], latent["mask"]["size"]
+    for label, KW in (("latent_attention", R), ("lodenex", R + 32)):
+        qa, pool = rnd(rows, H * KW), rnd(n_seqs * pages, PAGE * KW)
+        mixed = torch.empty((rows, H * R), dtype=bf, device=dev)
+        t = _timed_graph(lambda: ops.attend_masked(
+            qa, None, None, pool, None, None, table, q_start, ctx_len, seq_index, mixed, 0.09, 0.0,
+            window, 0, H, 1, KW, R, PAGE, T, ctx))
+        w = min(window, T)
+        seen = n_seqs * min(ctx, window) if decode else w * (w + 1) // 2 + (T - w) * w
+        work = (0.0, seen * KW * 2) if decode else \
+            (2.0 * seen * (KW + R) * H, rows * (H * (KW + R) + KW) * 2)
+        if label == "latent_attention":
+            t_new, w_new = t, work
+        else:
+            row("latent_attention", t_new, *w_new, lodenex=(t, *work))
+    # ---- the state space: convolution, recurrence, gate and norm
+    m = dict(sh["layers"])["mamba2"]
+    H, dv, N, G, taps = m["heads"], m["vdim"], m["state"], m["groups"], m["conv"]
+    I, BC = H * dv, G * N
+    C = I + 2 * BC
+    wide = rnd(rows, I + C)
+    size = (ops.state_space_state_size(H, N, dv) + (taps - 1) * C + 3) // 4 * 4
+    state = torch.zeros((n_seqs, size), dtype=torch.float32, device=dev)
+    tp, cb = f32(C, taps), f32(C)
+    xbc = torch.empty((rows, C), dtype=bf, device=dev)
+    t_new = _timed_graph(lambda: ops.short_conv(
+        wide[:, I:], tp, state, size - (taps - 1) * C, state_slots, seq_index, q_start, xbc,
+        single_tokens=decode, bias=cb))
+    xf = torch.empty((rows, C), dtype=torch.float32, device=dev)
+    unit = C // 2 // 128                          # (half the channels q and k heads of 128)
+    t_kg = _timed_graph(lambda: ops.short_conv(
+        wide[:, I:], tp, state, size - (taps - 1) * C, state_slots, seq_index, q_start, xf,
+        unit_heads=unit, head_dim=128, scaled_heads=unit // 2, scale=0.09, unit_eps=1e-6,
+        single_tokens=decode))
+    kept = 2.0 * n_seqs * (taps - 1) * C * 4
+    row("short_conv", t_new, 0.0, rows * C * 4 + kept, kugisun=(t_kg, 0.0, rows * C * 6 + kept))
+    lists = ops.fixed_decay_chunk_lists([T] * n_seqs)
+    if lists is not None:
+        lists = tuple(torch.from_numpy(t).to(dev) if t.size else None for t in lists)
+    steps = f32(rows, H)
+    al, db, sk = torch.zeros((H,), device=dev), torch.full((H,), -4.0, device=dev), f32(H)
+    y = torch.empty((rows, I), dtype=torch.float32, device=dev)
+    t_new = _timed_graph(lambda: ops.state_space(
+        xbc[:, :I], xbc[:, I:I + BC], xbc[:, I + BC:], steps, al, db, sk, state, state_slots, q_start,
+        y, H, G, N, dv, lists=lists))
+    fq, fk = rnd(rows, H * N), rnd(rows, H * N)
+    old = torch.zeros((n_seqs, ops.fixed_decay_state_size(H, N, dv)), device=dev)
+    decay = torch.stack([torch.full((H,), 0.99), torch.full((H,), 0.99).log2()]).to(dev)
+    t_fx = _timed_graph(lambda: ops.fixed_decay(
+        fq, fk, xbc[:, :I], decay, old, state_slots, q_start, y, H, N, dv, silu=True, k_scale=0.09,
+        lists=lists))
+    if decode:
+        work = old_work = (0.0, 2.0 * n_seqs * H * N * dv * 4)
+    else:
+        # state read and grown (4 N dv a token and head), a chunk of 128's own pairs (the scores
+        # once a group here, once a head there)
+        work = (rows * (H * (4.0 * N * dv + 128.0 * dv) + G * 128.0 * N),
+                rows * (C * 2 + I * 4 + H * 4))
+        old_work = (rows * H * (4.0 * N * dv + 128.0 * (N + dv)), rows * H * ((2 * N + dv) * 2 + dv * 4))
+    row("state_space", t_new, *work, fumanex=(t_fx, *old_work))
+    mixed = torch.empty((rows, I), dtype=bf, device=dev)
+    gain = torch.ones((I,), device=dev)
+    t_new = _timed_graph(lambda: ops.gate_norm(y, gain, wide[:, :I], mixed, m["norm_groups"], 1e-6))
+    t_fx = _timed_graph(lambda: ops.head_norm_gate(y, gain, wide[:, :I], mixed, m["norm_groups"], 1e-6))
+    work = (0.0, rows * I * 8)
+    row("gate_norm", t_new, *work, fumanex=(t_fx, *work))
+    # ---- products: the state space's (with the one for its step sizes) and the feed-forward
+    h = rnd(rows, W)
+    w_in, w_s, w_o = (ops.pretile_weight(rnd(*shape)) for shape in ((I + C, W), (H, W), (W, I)))
+    wide2, x = torch.empty((rows, I + C), dtype=bf, device=dev), torch.zeros((rows, W), device=dev)
+
+    def space_products():
+        ops.gemm(h, w_in, wide2, w_tiled=True)
+        ops.gemm(h, w_s, steps, w_tiled=True)
+        ops.gemm(mixed, w_o, x, w_tiled=True)
+    t_new = _timed_graph(space_products)
+    t_steps = _timed_graph(lambda: ops.gemm(h, w_s, steps, w_tiled=True))
+    gate_w, up_w, w_d = rnd(ff, W), rnd(ff, W), ops.pretile_weight(rnd(W, ff))
+    w_gu = ops.pretile_weight(ops.interleave_gate_up(gate_w, up_w))
+    act = torch.empty((rows, ff), dtype=bf, device=dev)
+    both = f32(2 * ff)
+
+    def swiglu_ff():
+        ops.gemm_swiglu(h, w_gu, act, w_tiled=True)
+        ops.gemm(act, w_d, x, w_tiled=True)
+    t_q3 = _timed_graph(swiglu_ff)
+    n_q3, n_new = 3 * W * ff, W * (2 * I + C + H)
+    row("space_products", t_new, 2.0 * rows * n_new, 2.0 * n_new,
+        qwen3=(t_q3, 2.0 * rows * n_q3, 2.0 * n_q3))
+    row("step_product", t_steps, 2.0 * rows * W * H, 2.0 * (W * H + rows * W) + 4.0 * rows * H)
+    t_new = _timed_graph(tigesun_ff(ops, h, gate_w, up_w, w_d, both, act, x))
+    row("feed_forward", t_new, 2.0 * rows * n_q3, 2.0 * n_q3,
+        qwen3=(t_q3, 2.0 * rows * n_q3, 2.0 * n_q3))
+    # ---- the norm behind a sublayer and the next one's, with the output's bias (Fezupel's: without)
+    gw, br = torch.ones((W,), device=dev), f32(rows, W)
+    res, normed, bias = f32(rows, W), torch.empty((rows, W), dtype=bf, device=dev), f32(W)
+    add = lambda yb: _timed_graph(lambda: ops.norm_add_norm(
+        br, gw, None, 1e-6, False, res, gw, None, 1e-6, False, normed, y_bias=yb))
+    work = (0.0, rows * W * 14)
+    row("norm_add_norm", add(bias), *work, fezupel=(add(None), *work))
+    ids = torch.randint(0, sh["vocab"], (rows,), generator=g, device=dev).to(torch.int32)
+    emb = rnd(sh["vocab"], W)
+    t_new = _timed_graph(lambda: ops.embed_norm(emb, ids, gw, 1e-6, res, 1.0, gw, 1e-6, normed))
+
+    def plain_embed():
+        ops.embed(emb, ids, res)
+        ops.rmsnorm(res, gw, 1e-6, normed)
+    t_q3 = _timed_graph(plain_embed)
+    row("embed_norm", t_new, 0.0, rows * W * 8, qwen3=(t_q3, 0.0, rows * W * 12))
+    return out
+
+
+def tigesun_ff(ops, h, gate_w, up_w, w_d, both, act, x):
+    """The gated feed-forward with biases as the model's part runs it, as one call."""
+    import torch
+    w = ops.pretile_weight(torch.cat([gate_w, up_w]).contiguous())
+    gu = torch.empty((h.shape[0], w.shape[0]), dtype=h.dtype, device=h.device)
+
+    def run():
+        ops.gemm(h, w, gu, w_tiled=True)
+        ops.gated_rows(gu, both, act, "gelu_tanh")
+        ops.gemm(act, w_d, x, w_tiled=True)
+    return run
+
+
+def main_tigesun(args) -> int:
+    """Prefill and decode throughput of Tigesun shapes beside the dense Qwen3 decoder of equal
+    size, and the design's kernels alone beside the like kernels of other designs."""
+    import torch
+    import zinfer_amd.ops as ops
+    from zinfer_amd.config import entry_for
+    T, batch, prompt = args.prefill_tokens, args.batch, args.prompt_len
+    max_positions = max(T, prompt + args.steps + args.warmup + 64) + 64
+    read_bw = ops.measure_read_bandwidth("cuda:0")
+    mfma_rate = ops.measure_mfma_rate("cuda:0")
+    names = [args.tigesun_shape] if args.tigesun_shape else list(TIGESUN_SHAPES)
+    shapes = {}
+    for name in names:
+        sh = TIGESUN_SHAPES[name]
+        row = {"sizes": {"width": sh["width"], "vocab": sh["vocab"], "ff": sh["ff"],
+                         "layers": [[k, dict(m)] for k, m in sh["layers"]]}}
+        for label, raw in (("tigesun", tigesun_config(sh)), ("qwen3", tigesun_twin(sh, max_positions))):
+            cfg = entry_for(raw).config_type.from_dict(raw)
+            pool = batch * (prompt + args.steps + args.warmup + 64) + T + 256
+            llm = build_llm(raw, args.dtype, args.seed, pool, max(batch, 8),
+                            max_step_tokens=max(T, 2048), multi_step=args.multi_step)
+            t_pre = run_prefill(llm, cfg, T, args.seed + 1)
+            dt, mean_ctx = run_decode(llm, cfg, batch, prompt, args.steps, args.warmup, args.seed + 2)
+            row[label] = {"prefill_tokens_per_s": round(T / t_pre, 1), "prefill_ms": round(t_pre * 1e3, 3),
+                          "decode_tokens_per_s": round(batch * args.steps / dt, 1),
+                          "decode_ms_per_step": round(dt / args.steps * 1e3, 4),
+                          "decode_mean_context": round(mean_ctx, 1)}
+            drop(llm)
+        row["prefill_vs_qwen3"] = round(row["tigesun"]["prefill_tokens_per_s"]
+                                        / row["qwen3"]["prefill_tokens_per_s"], 3)
+        row["decode_vs_qwen3"] = round(row["tigesun"]["decode_tokens_per_s"]
+                                       / row["qwen3"]["decode_tokens_per_s"], 3)
+        if args.dtype == "bfloat16":
+            row["kernels_prefill"] = tigesun_kernels(sh, T, T, mfma_rate, read_bw)
+            row["kernels_decode"] = tigesun_kernels(sh, 1, prompt, mfma_rate, read_bw)
+        ops._workspaces.clear()
+        torch.cuda.empty_cache()
+        shapes[name] = row
+    first = shapes[names[0]]
+    print(json.dumps({
+        "metric": "tigesun_decode_tokens_per_s", "value": first["tigesun"]["decode_tokens_per_s"],
+        "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": first["tigesun"]["decode_ms_per_step"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+        "data": "synthetic", "config": {"model": f"Tigesun {names[0]} shape beside the dense Qwen3 "
+                                                 "decoder of equal size, random weights",
+                                        "batch": batch, "prompt_len": prompt, "prefill_tokens": T,
+                                        "parallelism": "single GPU"},
+        "measured_read_gbs": round(read_bw / 1e9, 1), "mfma_loop_tflops": round(mfma_rate / 1e12, 1),
+        "shapes": shapes}))
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--workload", default="decode", choices=["decode", "continuous", "long-context", "fezupel", "lodenex", "nupovik",
-                             "kugisun", "fumanex"])
+                             "kugisun", "fumanex", "tigesun"])
     ap.add_argument("--shape", default=None, choices=sorted(SHAPES),
                     help="layer sizes (default: 8b for decode, 14b for continuous, 32b for "
                          "long-context)")
@@ -1919,6 +2238,8 @@ def main() -> int:
                     help="kugisun: only this shape (default: all of them)")
     ap.add_argument("--fumanex-shape", default=None, choices=sorted(FUMANEX_SHAPES),
                     help="fumanex: only this shape (default: all of them)")
+    ap.add_argument("--tigesun-shape", default=None, choices=sorted(TIGESUN_SHAPES),
+                    help="tigesun: only this shape (default: all of them)")
     ap.add_argument("--no-run-graphs", action="store_true",
                     help="decode steps in a row replay one graph per step instead of one for the run")
     args = ap.parse_args()
@@ -1929,7 +2250,7 @@ def main() -> int:
     return {"decode": main_decode, "continuous": main_continuous,
             "long-context": main_long_context, "fezupel": main_fezupel,
             "lodenex": main_lodenex, "nupovik": main_nupovik,
-            "kugisun": main_kugisun, "fumanex": main_fumanex}[args.workload](args)
+            "kugisun": main_kugisun, "fumanex": main_fumanex, "tigesun": main_tigesun}[args.workload](args)
 
 
 if __name__ == "__main__":
