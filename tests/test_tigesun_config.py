@@ -99,7 +99,7 @@ def test_what_the_configuration_refuses():
     broken(lambda r: r["layers"][0]["mixer"]["rot"]["scaling"].pop("slow"))
     broken(lambda r: r["layers"][0]["mixer"]["rot"].update(scaling=3))
     broken(lambda r: r["layers"][1]["mixer"].update(groups=2))              # of 3 heads
-    broken(lambda r: r["layers"][1]["mixer"].update(norm_groups=5))         # of 24 values
+    broken(lambda r: r["layers"][1]["mixer"].update(norm_groups=5))         # of 48 values
     broken(lambda r: r["layers"][1]["mixer"].update(state=0))
     broken(lambda r: r["layers"][1]["mixer"].pop("conv"))
     broken(lambda r: r["layers"][2]["mixer"]["mask"].update(size=0))

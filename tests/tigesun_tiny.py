@@ -48,15 +48,15 @@ def _again(layers, j):
 
 
 # every mixer; a state space without a feed-forward and one with it; the first three run again
-_A = [_attention(6, 3, 12, 20, 40, 8, 100.0, (3.0, 40, 4.0, 0.5)), _space(3, 8, 10, 1, 4, 3),
+_A = [_attention(6, 3, 12, 20, 40, 8, 100.0, (3.0, 40, 4.0, 0.5)), _space(3, 16, 10, 1, 4, 3),
       _latent(4, 10, 12, 18, 36, 9), _space(4, 6, 12, 2, 2, 1, 28), _latent(2, 16, 5, 24, None, 30)]
 TG_A = {"architecture": "Tigesun", "vocab": 203, "width": 48, "norm": {"eps": 1e-5},
         "logit_softcap": 25.0,
         "layers": _A + [_again(_A, 0), _again(_A, 1), _again(_A, 2)]}
 
 # a state space first, tensors of a layer that comes later, and a chain of such layers; no cap; a
-# window of one token and none; rotations whole and not at all; one tap; a norm part of half a head
-_B = [_space(6, 4, 8, 6, 1, 12, 24), _attention(5, 5, 8, 12, 24, 8, 50.0), _latent(3, 8, 16, 20, 44, 1),
+# window of one token and none; rotations whole and not at all; one tap; norm parts of a head and a half
+_B = [_space(6, 4, 8, 6, 1, 4, 24), _attention(5, 5, 8, 12, 24, 8, 50.0), _latent(3, 8, 16, 20, 44, 1),
       _attention(10, 5, 24, 12, 32), _latent(5, 24, 8, 16, None, None), _space(4, 16, 40, 1, 5, 2)]
 TG_B = {"architecture": "Tigesun", "vocab": 310, "width": 72, "norm": {"eps": 1e-6},
         "layers": [dict(_B[5], weights_of=6)] + _B + [dict(_B[1], weights_of=2),
@@ -65,8 +65,8 @@ TG_B = {"architecture": "Tigesun", "vocab": 310, "width": 72, "norm": {"eps": 1e
 # a width no vector kernel takes, sizes that are no multiple of 4, one head, one kv head, heads of
 # one value
 _C = [_latent(1, 7, 3, 5, 14, 7), _space(5, 3, 7, 5, 3, 1), _attention(5, 1, 10, 5, 30, 6, 7.0),
-      _space(7, 1, 1, 1, 4, 7, 18), _attention(3, 1, 6, 11, None, 2, 20.0, (2.5, 100, 8.0, 2.0)),
-      _space(1, 9, 30, 1, 2, 3)]
+      _space(7, 1, 1, 1, 4, 1, 18), _attention(3, 1, 6, 11, None, 2, 20.0, (2.5, 100, 8.0, 2.0)),
+      _space(1, 12, 30, 1, 2, 2)]
 TG_C = {"architecture": "Tigesun", "vocab": 97, "width": 50, "norm": {"eps": 1e-3},
         "logit_softcap": 12.0, "layers": _C + [_again(_C, 1), _again(_C, 4)]}
 
