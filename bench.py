@@ -2089,8 +2089,8 @@ def tigesun_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float
         ops.gemm(mixed, w_o, x, w_tiled=True)
     t_new = _timed_graph(space_products)
     t_steps = _timed_graph(lambda: ops.gemm(h, w_s, steps, w_tiled=True))
-    gate_w, up_w, w_d = rnd(ff, W), rnd(ff, W), ops.pretile_weight(rnd(W, ff))
-    w_gu = ops.pretile_weight(ops.interleave_gate_up(gate_w, up_w))
+    w_gu = ops.pretile_weight(ops.interleave_gate_up(rnd(ff, W), rnd(ff, W)))
+    w_d = ops.pretile_weight(rnd(W, ff))
     act = torch.empty((rows, ff), dtype=bf, device=dev)
     both = f32(2 * ff)
 
@@ -2102,7 +2102,11 @@ def tigesun_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float
     row("space_products", t_new, 2.0 * rows * n_new, 2.0 * n_new,
         qwen3=(t_q3, 2.0 * rows * n_q3, 2.0 * n_q3))
     row("step_product", t_steps, 2.0 * rows * W * H, 2.0 * (W * H + rows * W) + 4.0 * rows * H)
-    t_new = _timed_graph(tigesun_ff(ops, h, gate_w, up_w, w_d, both, act, x))
+
+    def geglu_ff():
+        ops.gemm_geglu(h, w_gu, both, act)
+        ops.gemm(act, w_d, x, w_tiled=True)
+    t_new = _timed_graph(geglu_ff)
     row("feed_forward", t_new, 2.0 * rows * n_q3, 2.0 * n_q3,
         qwen3=(t_q3, 2.0 * rows * n_q3, 2.0 * n_q3))
     # ---- the norm behind a sublayer and the next one's, with the output's bias (Fezupel's: without)
@@ -2122,19 +2126,6 @@ def tigesun_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float
     t_q3 = _timed_graph(plain_embed)
     row("embed_norm", t_new, 0.0, rows * W * 8, qwen3=(t_q3, 0.0, rows * W * 12))
     return out
-
-
-def tigesun_ff(ops, h, gate_w, up_w, w_d, both, act, x):
-    """The gated feed-forward with biases as the model's part runs it, as one call."""
-    import torch
-    w = ops.pretile_weight(torch.cat([gate_w, up_w]).contiguous())
-    gu = torch.empty((h.shape[0], w.shape[0]), dtype=h.dtype, device=h.device)
-
-    def run():
-        ops.gemm(h, w, gu, w_tiled=True)
-        ops.gated_rows(gu, both, act, "gelu_tanh")
-        ops.gemm(act, w_d, x, w_tiled=True)
-    return run
 
 
 def main_tigesun(args) -> int:

@@ -168,6 +168,7 @@ TESTED_AGAINST = {
     "delta_recurrence": "plain_kugisun.py:delta_rule",
     "rotation_table": "plain_fumanex.py:rotate", "fixed_decay": "plain_fumanex.py:decayed_sums",
     "embed_norm": "plain_tigesun.py:rms_norm", "gated_rows": "plain_tigesun.py:gelu_tanh",
+    "gemm_geglu": "plain_tigesun.py:feed_forward",
     "gate_norm": "plain_tigesun.py:gated_parts_norm", "state_space": "plain_tigesun.py:state_space",
     "bias_act_rows": "plain_fumanex.py:gelu_tanh", "add_row": "plain_fumanex.py:linear",
 }

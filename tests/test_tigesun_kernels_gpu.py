@@ -95,6 +95,26 @@ def test_gated_activation_behind_biases(dt, n):
         assert rel_err(out, P.gelu_tanh(x[:, :n]) * x[:, n:]) < tol(dt)
 
 
+@pytest.mark.parametrize("M", [1, 8, 16, 17, 33, 64, 100, 128, 129, 300, 1000, 2048])
+@pytest.mark.parametrize("I,K", [(64, 64), (96, 192), (2048, 512), (8192, 256), (5632, 2048)])
+def test_gated_activation_in_the_products_epilogue(M, I, K):
+    """Every kernel that the number of rows and the sizes lead to, with biases that differ from
+    column to column and without."""
+    if M > 300 and I * K > (1 << 20) and (M, I) not in ((2048, 8192), (1000, 5632)):
+        pytest.skip("one long product a size")
+    a = _rand((M, K), 1, 1.0, torch.bfloat16)
+    g, u = _rand((I, K), 2, K ** -0.5, torch.bfloat16), _rand((I, K), 3, K ** -0.5, torch.bfloat16)
+    bg, bu = _rand((I,), 4), _rand((I,), 5)
+    w = ops.pretile_weight(ops.interleave_gate_up(g, u).to(DEV))
+    out = torch.empty((M, I), dtype=torch.bfloat16, device=DEV)
+    # (32-bit products on the CPU: 64-bit ones of these sizes take seconds)
+    zg, zu = (a.float() @ g.float().T).double(), (a.float() @ u.float().T).double()
+    ops.gemm_geglu(a.to(DEV), w, ops.interleave_bias(bg, bu).to(DEV), out)
+    assert rel_err(out, P.gelu_tanh(zg + bg.double()) * (zu + bu.double())) < tol(torch.bfloat16)
+    ops.gemm_geglu(a.to(DEV), w, None, out)
+    assert rel_err(out, P.gelu_tanh(zg) * zu) < tol(torch.bfloat16)
+
+
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("parts,dv", [(1, 24), (3, 8), (2, 50), (4, 128), (2, 516), (1, 4096), (7, 1),
                                       (1, 9000)])

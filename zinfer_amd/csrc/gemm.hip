@@ -121,7 +121,21 @@ typedef __attribute__((__vector_size__(2 * sizeof(uint32_t)))) uint32_t u32x2_t;
 // silu(gate) * up as bfloat16 [M, N / 2]  (a_j = g_j / (1 + exp(-g_j)) * u_j, cpu.zig:130-147)
 #define EPI_SWIGLU 3
 
+// the same with the tanh form of gelu and a bias a row of W (float32 [N] in W's order, or null):
+// gelu(gate + b_gate) * (up + b_up)
+#define EPI_GEGLU 4
+#define EPI_GLU(E) ((E) == EPI_SWIGLU || (E) == EPI_GEGLU)
+
 __device__ __forceinline__ float swiglu_f(float g, float u) { return g / (1.0f + expf(-g)) * u; }
+// gelu(g) = g / 2 (1 + tanh(v)), the tanh through one exponential: 1 - 2 / (e^2v + 1)
+__device__ __forceinline__ float geglu_f(float g, float u) {
+  const float v = 0.79788456080286535588f * (g + 0.044715f * g * g * g);
+  const float e = __builtin_amdgcn_exp2f(v * 2.8853900817779268f);
+  return g * (1.0f - __builtin_amdgcn_rcpf(e + 1.0f)) * u;
+}
+template <int EPI> __device__ __forceinline__ float glu_f(float g, float u) {
+  return EPI == EPI_GEGLU ? geglu_f(g, u) : swiglu_f(g, u);
+}
 
 // ---------------------------------------------------------------- large M: LDS-tiled
 // Block tile BM x BN x 64, waves laid out (BM/WM) x (BN/WN), each wave WM x WN through
@@ -322,6 +336,10 @@ __global__ __launch_bounds__((BM / WM) * (BN / WN) * 64) void gemm_bf16_tile_ker
     }
 }
 
+__device__ __forceinline__ float4 sum4(const float4& a, const float4& b) {
+  return float4{a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w};
+}
+
 // Epilogue through LDS of the kernels whose waves hold 32-row x 32-column MFMA results: a
 // 32x32 result has a lane's 16 values in 16 different rows, so direct stores would be 2 or 4
 // bytes wide in runs of 64 bytes.  Each wave lays 32 rows of WN columns of its tile (the FN
@@ -330,7 +348,8 @@ __global__ __launch_bounds__((BM / WM) * (BN / WN) * 64) void gemm_bf16_tile_ker
 // workgroup call it together.
 template <int FM, int FN, int WN, int EPI, int J0 = 0, int FNALL = FN>
 __device__ __forceinline__ void store_through_slab(f32x16_t (&acc)[FM][FNALL], float* slab, int mw,
-                                                   int nw, int M, int N, void* Cv, int lane) {
+                                                   int nw, int M, int N, void* Cv, int lane,
+                                                   const float* glu_bias = nullptr) {
   static_assert(WN == 32 * FN && J0 + FN <= FNALL, "column blocks");
   constexpr int SLAB_ROW = WN + 4;
 #pragma unroll
@@ -341,7 +360,7 @@ __device__ __forceinline__ void store_through_slab(f32x16_t (&acc)[FM][FNALL], f
       for (int r = 0; r < 16; ++r)
         slab[(8 * (r / 4) + 4 * (lane / 32) + r % 4) * SLAB_ROW + j * 32 + lane % 32] = acc[i][J0 + j][r];
     __syncthreads();
-    if (EPI == EPI_SWIGLU) {
+    if (EPI_GLU(EPI)) {
       // 16 gate columns, then the 16 up columns that belong to them: 8 outputs per lane
       constexpr int LPR = WN / 16;                  // lanes per row
 #pragma unroll
@@ -352,13 +371,19 @@ __device__ __forceinline__ void store_through_slab(f32x16_t (&acc)[FM][FNALL], f
         const int n = nw + c;
         if (m < M && n < N) {
           const float* src = slab + row * SLAB_ROW + c;
-          const float4 g0 = *(const float4*)src, g1 = *(const float4*)(src + 4);
-          const float4 u0 = *(const float4*)(src + 16), u1 = *(const float4*)(src + 20);
+          float4 g0 = *(const float4*)src, g1 = *(const float4*)(src + 4);
+          float4 u0 = *(const float4*)(src + 16), u1 = *(const float4*)(src + 20);
+          if (EPI == EPI_GEGLU && glu_bias != nullptr) {
+            g0 = sum4(g0, *(const float4*)(glu_bias + n));
+            g1 = sum4(g1, *(const float4*)(glu_bias + n + 4));
+            u0 = sum4(u0, *(const float4*)(glu_bias + n + 16));
+            u1 = sum4(u1, *(const float4*)(glu_bias + n + 20));
+          }
           const u32x4_t v = u32x4_t{
-              pack_bf16x2(swiglu_f(g0.x, u0.x), swiglu_f(g0.y, u0.y)),
-              pack_bf16x2(swiglu_f(g0.z, u0.z), swiglu_f(g0.w, u0.w)),
-              pack_bf16x2(swiglu_f(g1.x, u1.x), swiglu_f(g1.y, u1.y)),
-              pack_bf16x2(swiglu_f(g1.z, u1.z), swiglu_f(g1.w, u1.w))};
+              pack_bf16x2(glu_f<EPI>(g0.x, u0.x), glu_f<EPI>(g0.y, u0.y)),
+              pack_bf16x2(glu_f<EPI>(g0.z, u0.z), glu_f<EPI>(g0.w, u0.w)),
+              pack_bf16x2(glu_f<EPI>(g1.x, u1.x), glu_f<EPI>(g1.y, u1.y)),
+              pack_bf16x2(glu_f<EPI>(g1.z, u1.z), glu_f<EPI>(g1.w, u1.w))};
           *(u32x4_t*)((bf16_t*)Cv + (size_t)m * (N / 2) + (n / 32) * 16 + (n % 32)) = v;
         }
       }
@@ -428,7 +453,7 @@ template <int BM, int BN, int WM, int WN, int EPI, int TKM = TK, bool W2 = false
 __global__ __launch_bounds__((BM / WM) * (BN / WN) * 64 * KG) void gemm_bf16_tile_wdirect_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, void* __restrict__ Cv, int M,
     int N, int K, int tiles_m, int tiles_n, int whole, int tail_split,
-    float* __restrict__ tail_ws) {
+    float* __restrict__ tail_ws, const float* __restrict__ glu_bias) {
   // (the host pass, which only needs the launch stub, does not know the buffer descriptor type)
 #if defined(__HIP_DEVICE_COMPILE__)
   constexpr int NWN = BN / WN, NT = (BM / WM) * NWN * 64;       // (NT: the threads of a group)
@@ -738,7 +763,7 @@ __global__ __launch_bounds__((BM / WM) * (BN / WN) * 64 * KG) void gemm_bf16_til
       for (int r = 0; r < 16; ++r) kept[i][0][r] = kgrp == 0 ? acc[i][0][r] : acc[i][1][r];
     float* slab32 = (float*)lds_raw + (size_t)(kgrp * (NT / 64) + wave) * 32 * (32 + 4);
     store_through_slab<FM, 1, 32, EPI>(kept, slab32, m0 + wm * WM, n0 + wn * WN + 32 * kgrp, M, N,
-                                       Cv, lane);
+                                       Cv, lane, glu_bias);
     return;
   }
   float* slab = (float*)lds_raw + (size_t)wave * 32 * (WN + 4);
@@ -749,7 +774,8 @@ __global__ __launch_bounds__((BM / WM) * (BN / WN) * 64 * KG) void gemm_bf16_til
       return;
     }
   }
-  store_through_slab<FM, FN, WN, EPI>(acc, slab, m0 + wm * WM, n0 + wn * WN, M, N, Cv, lane);
+  store_through_slab<FM, FN, WN, EPI>(acc, slab, m0 + wm * WM, n0 + wn * WN, M, N, Cv, lane,
+                                      glu_bias);
 #endif
 }
 
@@ -760,7 +786,7 @@ __global__ __launch_bounds__((BM / WM) * (BN / WN) * 64 * KG) void gemm_bf16_til
 template <int BM, int BN, int EPI>
 __global__ __launch_bounds__(BN) void tile_tail_reduce_kernel(
     const float* __restrict__ ws, void* __restrict__ Cv, int M, int N, int tiles_m, int tiles_n,
-    int whole, int split) {
+    int whole, int split, const float* __restrict__ glu_bias) {
   static_assert(BN % 32 == 0 && BM % 8 == 0, "a row is BN / 8 threads");
   constexpr int TPR = BN / 8;                        // threads per row
   const int t = blockIdx.x;
@@ -768,8 +794,8 @@ __global__ __launch_bounds__(BN) void tile_tail_reduce_kernel(
   tile_of_workgroup<(BM >= 128 ? 8 : 1024 / BM)>(whole + t, tiles_m, tiles_n, tm, tn);
   const int row = blockIdx.y * 8 + threadIdx.x / TPR, q = threadIdx.x % TPR;
   const int m = tm * BM + row;
-  const int c0 = EPI == EPI_SWIGLU ? (q / 4) * 32 + (q % 4) * 4 : q * 8;
-  const int c1 = EPI == EPI_SWIGLU ? c0 + 16 : c0 + 4;
+  const int c0 = EPI_GLU(EPI) ? (q / 4) * 32 + (q % 4) * 4 : q * 8;
+  const int c1 = EPI_GLU(EPI) ? c0 + 16 : c0 + 4;
   const int n = tn * BN + c0;
   if (m >= M || n >= N) return;
   const float* part = ws + ((size_t)t * split * BM + row) * BN;
@@ -780,9 +806,13 @@ __global__ __launch_bounds__(BN) void tile_tail_reduce_kernel(
     x0.x += p0.x; x0.y += p0.y; x0.z += p0.z; x0.w += p0.w;
     x1.x += p1.x; x1.y += p1.y; x1.z += p1.z; x1.w += p1.w;
   }
-  if (EPI == EPI_SWIGLU) {
-    const u32x2_t v = u32x2_t{pack_bf16x2(swiglu_f(x0.x, x1.x), swiglu_f(x0.y, x1.y)),
-                              pack_bf16x2(swiglu_f(x0.z, x1.z), swiglu_f(x0.w, x1.w))};
+  if (EPI_GLU(EPI)) {
+    if (EPI == EPI_GEGLU && glu_bias != nullptr) {
+      x0 = sum4(x0, *(const float4*)(glu_bias + n));
+      x1 = sum4(x1, *(const float4*)(glu_bias + n + 16));
+    }
+    const u32x2_t v = u32x2_t{pack_bf16x2(glu_f<EPI>(x0.x, x1.x), glu_f<EPI>(x0.y, x1.y)),
+                              pack_bf16x2(glu_f<EPI>(x0.z, x1.z), glu_f<EPI>(x0.w, x1.w))};
     *(u32x2_t*)((bf16_t*)Cv + (size_t)m * (N / 2) + (n / 32) * 16 + (n % 32)) = v;
   } else if (EPI == EPI_STORE_BF16) {
     *(u32x4_t*)((bf16_t*)Cv + (size_t)m * N + n) =
@@ -841,7 +871,7 @@ constexpr int reads_before(int m, int nm, int cnt, int nr) {
 template <int BN, int EPI>
 __global__ __launch_bounds__(256) void gemm_bf16_tile256_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ W, void* __restrict__ Cv, int M,
-    int N, int K, int tiles_m, int tiles_n) {
+    int N, int K, int tiles_m, int tiles_n, const float* __restrict__ glu_bias) {
   // (the host pass, which only needs the launch stub, does not know the buffer descriptor type)
 #if defined(__HIP_DEVICE_COMPILE__)
   constexpr int BM = 256, NT = 256, WM = 128, WN = BN / 2, FM = WM / 32, FN = WN / 32;
@@ -1060,26 +1090,28 @@ __global__ __launch_bounds__(256) void gemm_bf16_tile256_kernel(
   static_assert(32 * (WN + 4) * sizeof(float) <= (A_PLACES + W_PLACES) * 16 || FN == 3, "slab");
   const int mw = m0 + wm * WM, nw = n0 + wn * WN;
   if constexpr (FN == 3) {
-    store_through_slab<FM, 2, 64, EPI, 0, FN>(acc, slab, mw, nw, M, N, Cv, lane);
-    store_through_slab<FM, 1, 32, EPI, 2, FN>(acc, slab, mw, nw + 64, M, N, Cv, lane);
+    store_through_slab<FM, 2, 64, EPI, 0, FN>(acc, slab, mw, nw, M, N, Cv, lane, glu_bias);
+    store_through_slab<FM, 1, 32, EPI, 2, FN>(acc, slab, mw, nw + 64, M, N, Cv, lane, glu_bias);
   } else {
-    store_through_slab<FM, FN, WN, EPI>(acc, slab, mw, nw, M, N, Cv, lane);
+    store_through_slab<FM, FN, WN, EPI>(acc, slab, mw, nw, M, N, Cv, lane, glu_bias);
   }
 #endif
 }
 
 template <int BN>
 static int launch_tile256(const void* A, const void* W, void* C, int M, int N, int K, int epi,
-                          hipStream_t stream) {
+                          hipStream_t stream, const float* glu_bias = nullptr) {
   if (N % 16 != 0 || K % 128 != 0) return -3;
   const int tiles_m = (M + 255) / 256, tiles_n = (N + BN - 1) / BN;
   const dim3 grid(tiles_m * tiles_n), block(256);
 #define ZF_T256(E)                                                                             \
   hipLaunchKernelGGL((gemm_bf16_tile256_kernel<BN, E>), grid, block, 0, stream,                \
-                     (const bf16_t*)A, (const bf16_t*)W, C, M, N, K, tiles_m, tiles_n)
+                     (const bf16_t*)A, (const bf16_t*)W, C, M, N, K, tiles_m, tiles_n,   \
+                     glu_bias)
   if (epi == EPI_STORE_BF16) ZF_T256(EPI_STORE_BF16);
   else if (epi == EPI_STORE_F32) ZF_T256(EPI_STORE_F32);
   else if (epi == EPI_SWIGLU) ZF_T256(EPI_SWIGLU);
+  else if (epi == EPI_GEGLU) ZF_T256(EPI_GEGLU);
   else ZF_T256(EPI_ACC_F32);
 #undef ZF_T256
   return (int)hipGetLastError();
@@ -1094,12 +1126,12 @@ template <int BM, int BN, int WM, int WN, int TKM = TK, bool W2 = false, bool AD
           int KG = 1>
 static int launch_tile_wdirect(const void* A, const void* W, void* C, int M, int N, int K, int epi,
                                hipStream_t stream, void* ws = nullptr, int ksplit = 1,
-                               bool reduce = true) {
+                               bool reduce = true, const float* glu_bias = nullptr) {
   if (N % 16 != 0 || K % TKM != 0) return -3;
   // every part (and every group of waves in it) an even number of k-tiles
   if (W2 && (K / TKM) % (2 * ksplit * KG) != 0) return -3;
   if (KG > 1 && (K / TKM) % (ksplit * KG) != 0) return -3;      // the groups meet step by step
-  if (ksplit > 1 && (ws == nullptr || epi == EPI_SWIGLU || ksplit > K / TKM)) return -3;
+  if (ksplit > 1 && (ws == nullptr || EPI_GLU(epi) || ksplit > K / TKM)) return -3;
   constexpr int NT = (BM / WM) * (BN / WN) * 64 * KG;
   const int tiles_m = (M + BM - 1) / BM, tiles_n = (N + BN - 1) / BN;
   const dim3 grid(tiles_m * tiles_n, ksplit), block(NT);
@@ -1121,7 +1153,7 @@ static int launch_tile_wdirect(const void* A, const void* W, void* C, int M, int
       if (e != hipSuccess) return (int)e;                                                     \
     }                                                                                         \
     hipLaunchKernelGGL(kern, grid, block, smem, stream, (const bf16_t*)A, (const bf16_t*)W, C, \
-                       M, N, K, tiles_m, tiles_n, 0, 1, (float*)nullptr);                     \
+                       M, N, K, tiles_m, tiles_n, 0, 1, (float*)nullptr, glu_bias);           \
   } while (0)
   void* const final_c = C;
   if (ksplit > 1) {
@@ -1131,6 +1163,7 @@ static int launch_tile_wdirect(const void* A, const void* W, void* C, int M, int
   if (epi == EPI_STORE_BF16) ZF_WD(EPI_STORE_BF16);
   else if (epi == EPI_STORE_F32) ZF_WD(EPI_STORE_F32);
   else if (epi == EPI_SWIGLU) ZF_WD(EPI_SWIGLU);
+  else if (epi == EPI_GEGLU) ZF_WD(EPI_GEGLU);
   else ZF_WD(EPI_ACC_F32);
 #undef ZF_WD
   if (ksplit > 1 && reduce) return launch_reduce(ws, final_c, M, N, ksplit, final_epi, stream);
@@ -1142,7 +1175,8 @@ static int launch_tile_wdirect(const void* A, const void* W, void* C, int M, int
 // partials; every epilogue.
 template <bool W2>
 static int launch_tile_tail(const void* A, const void* W, void* C, void* ws, int M, int N, int K,
-                            int epi, int whole, int split, hipStream_t stream) {
+                            int epi, int whole, int split, hipStream_t stream,
+                            const float* glu_bias = nullptr) {
   constexpr int BM = 128, BN = 256, WM = 128, WN = 64, NT = 256;
   const int tiles_m = (M + BM - 1) / BM, tiles_n = (N + BN - 1) / BN;
   const long long tiles = (long long)tiles_m * tiles_n;
@@ -1158,14 +1192,15 @@ static int launch_tile_tail(const void* A, const void* W, void* C, void* ws, int
   do {                                                                                        \
     hipLaunchKernelGGL((gemm_bf16_tile_wdirect_kernel<BM, BN, WM, WN, E, TK, W2, true, true>), \
                        grid, block, smem, stream, (const bf16_t*)A, (const bf16_t*)W, C, M, N, \
-                       K, tiles_m, tiles_n, whole, split, (float*)ws);                        \
+                       K, tiles_m, tiles_n, whole, split, (float*)ws, glu_bias);              \
     hipLaunchKernelGGL((tile_tail_reduce_kernel<BM, BN, E>), dim3((unsigned)tail, BM / 8),    \
                        dim3(BN), 0, stream, (const float*)ws, C, M, N, tiles_m, tiles_n,      \
-                       whole, split);                                                         \
+                       whole, split, glu_bias);                                               \
   } while (0)
   if (epi == EPI_STORE_BF16) ZF_WT(EPI_STORE_BF16);
   else if (epi == EPI_STORE_F32) ZF_WT(EPI_STORE_F32);
   else if (epi == EPI_SWIGLU) ZF_WT(EPI_SWIGLU);
+  else if (epi == EPI_GEGLU) ZF_WT(EPI_GEGLU);
   else ZF_WT(EPI_ACC_F32);
 #undef ZF_WT
   return (int)hipGetLastError();
@@ -1321,6 +1356,7 @@ struct SkinnyNorm {
   const float* gain_out;
   bf16_t* xg_out;
   float* sq_out;
+  const float* glu_bias;       // (EPI_GEGLU) a bias a row of W, or null
 };
 
 // The 128 x 128 tiled product on pre-tiled W with ksplit workgroups per tile along K, for
@@ -1420,7 +1456,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_bf16_skinny_kernel(
       sqv[i] = gidx < nrm.sq_groups ? nrm.sq_in[gidx * 16 + j] : 0.f;
     }
   }
-  if (WT && NORM != NORM_FOLD && (RG * MT == 1 || (RG * MT == 2 && EPI != EPI_SWIGLU))) {
+  if (WT && NORM != NORM_FOLD && (RG * MT == 1 || (RG * MT == 2 && !EPI_GLU(EPI)))) {
     // Pre-tiled weights (no bounds checks; K % 64 == 0), up to two MFMA tiles per k-step:
     // batches of UNR k-steps in two register sets, the next batch asked for before the
     // MFMAs of the one that has arrived, so that a wave always has loads in flight.  The
@@ -1580,7 +1616,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_bf16_skinny_kernel(
     for (int w = 0; w < NSS; ++w) tot += ssum[w][t][j];
     return 1.0f / sqrtf(tot / (float)K + eps);
   };
-  if (EPI == EPI_SWIGLU) {
+  if (EPI_GLU(EPI)) {
     // row groups alternate gate / up: the pair (2 p, 2 p + 1) gives 16 outputs per token
     for (int item = tid; item < (RG / 2) * MT * 64; item += NW * 64) {
       const int pt = item / 64, l = item % 64;
@@ -1599,9 +1635,15 @@ __global__ __launch_bounds__(NW * 64) void gemm_bf16_skinny_kernel(
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const int n = n0 / 2 + p * 16 + 4 * (l / 16) + e;      // column of the [M, N / 2] output
-          if (2 * n < N)
-            ((bf16_t*)Cv)[(size_t)token * (N / 2) + n] =
-                float_to_bf16(swiglu_f(g[e] * inv, u[e] * inv));
+          if (2 * n < N) {
+            float gv = g[e] * inv, uv = u[e] * inv;
+            if (EPI == EPI_GEGLU && nrm.glu_bias != nullptr) {
+              const float* b = nrm.glu_bias + n0 + p * 32 + 4 * (l / 16) + e;
+              gv += b[0];
+              uv += b[16];
+            }
+            ((bf16_t*)Cv)[(size_t)token * (N / 2) + n] = float_to_bf16(glu_f<EPI>(gv, uv));
+          }
         }
       }
     }
@@ -1836,6 +1878,15 @@ static int launch_skinny(const void* A, const void* W, void* C, void* ws, int M,
                        block, 0, stream, (const bf16_t*)A, (const bf16_t*)W, dst, M, N, K, nrm);
     return (int)hipGetLastError();
   }
+  if (epi == EPI_GEGLU) {
+    if constexpr (WT && NORM == NORM_NONE) {
+      if (RG < 2 || ksplit != 1 || N % 32 != 0) return -3;
+      hipLaunchKernelGGL((gemm_bf16_skinny_kernel<MT, (RG < 2 ? 2 : RG), EPI_GEGLU, WT, NORM, NW>),
+                         grid, block, 0, stream, (const bf16_t*)A, (const bf16_t*)W, dst, M, N, K, nrm);
+      return (int)hipGetLastError();
+    }
+    return -3;
+  }
   if (epi == EPI_SWIGLU) {
     if (RG < 2 || ksplit != 1 || N % 32 != 0) return -3;
     hipLaunchKernelGGL((gemm_bf16_skinny_kernel<MT, (RG < 2 ? 2 : RG), EPI_SWIGLU, WT, NORM, NW>), grid,
@@ -1902,6 +1953,61 @@ extern "C" int zf_gemm_bf16_skinny(const void* A, const void* W, void* C, void* 
   if (rg == 4) { if (mt == 1) ZF_SK(1, 4); if (mt == 2) ZF_SK(2, 4); if (mt == 3) ZF_SK(3, 4); ZF_SK(4, 4); }
 #undef ZF_SK
   return -4;
+}
+
+// out[M, N / 2] = gelu(A Wg^T + bg) * (A Wu^T + bu) with W's and bias's rows alternating in groups
+// of 16 (EPI_GEGLU), W pre-tiled.  way: 0 tiles (number: the variant of zf_gemm_bf16_tile), 1 the
+// 128 x 256 tiles with the last round split along K (number: whole, split), 2 for 17 to 128
+// tokens, 3 weight streaming (number: rg).
+extern "C" int zf_gemm_geglu(const void* A, const void* W, const float* bias, void* C, void* ws,
+                             int M, int N, int K, int way, int number, int split,
+                             hipStream_t stream) {
+  if (M <= 0 || N <= 0) return 0;
+  if (N % 32 != 0 || K % 64 != 0) return -3;
+  constexpr int E = EPI_GEGLU;
+  if (way == 1) {
+    if (K % (2 * TK) == 0 && (K / TK) % (2 * split) == 0)
+      return launch_tile_tail<true>(A, W, C, ws, M, N, K, E, number, split, stream, bias);
+    return launch_tile_tail<false>(A, W, C, ws, M, N, K, E, number, split, stream, bias);
+  }
+  if (way == 2) {
+    if (M > 128) return -3;
+    if (M <= 32)
+      return launch_tile_wdirect<32, 128, 32, 32, 256>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+    if (M <= 64)
+      return launch_tile_wdirect<64, 128, 64, 32, 128>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+    return launch_tile_wdirect<128, 128, 128, 32, 128>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+  }
+  if (way == 3) {
+    if (M > 64 || N % (16 * number) != 0) return -3;
+    const int mt = (M + 15) / 16;
+    SkinnyNorm nrm{};
+    nrm.glu_bias = bias;
+#define ZF_GSK(MT, RG) \
+  return launch_skinny<MT, RG, true>(A, W, C, nullptr, M, N, K, E, 1, stream, nrm)
+    if (number == 2) { if (mt == 1) ZF_GSK(1, 2); if (mt == 2) ZF_GSK(2, 2); if (mt == 3) ZF_GSK(3, 2); ZF_GSK(4, 2); }
+    if (number == 4) { if (mt == 1) ZF_GSK(1, 4); if (mt == 2) ZF_GSK(2, 4); if (mt == 3) ZF_GSK(3, 4); ZF_GSK(4, 4); }
+#undef ZF_GSK
+    return -4;
+  }
+  switch (number) {
+    case 6:
+      if ((long long)((M + 127) / 128) * ((N + 127) / 128) >= 384)
+        return launch_tile_wdirect<128, 128, 64, 64, TK, false, true>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+      return launch_tile_wdirect<128, 128, 64, 64>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+    case 10:
+      if (K % (2 * TK) == 0)
+        return launch_tile_wdirect<128, 256, 128, 64, TK, true, true>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+      return launch_tile_wdirect<128, 256, 128, 64, TK, false, true>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+    case 12:
+      return launch_tile_wdirect<128, 256, 128, 64, TK, true, true, 2>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+    case 16:
+      return launch_tile_wdirect<128, 128, 128, 32, 128>(A, W, C, M, N, K, E, stream, nullptr, 1, true, bias);
+    case 20: return launch_tile256<256>(A, W, C, M, N, K, E, stream, bias);
+    case 21: return launch_tile256<192>(A, W, C, M, N, K, E, stream, bias);
+    case 22: return launch_tile256<128>(A, W, C, M, N, K, E, stream, bias);
+    default: return -4;
+  }
 }
 
 // The same product with the RMSNorm before it folded in: X is the float32 residual stream

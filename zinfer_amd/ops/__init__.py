@@ -1256,6 +1256,56 @@ def gemm_swiglu(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, w_tiled: bo
                "gemm_swiglu (tiled)")
 
 
+def can_fuse_geglu(intermediate_size: int, hidden_size: int) -> bool:
+    """Whether ``gemm_geglu`` takes the stacked matrix of a gated feed-forward of these sizes."""
+    return intermediate_size % 32 == 0 and hidden_size % 64 == 0
+
+
+def interleave_bias(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+    """The two projections' biases in the order of ``interleave_gate_up``'s rows."""
+    I = gate.shape[0]
+    return torch.stack([gate.view(I // 16, 16), up.view(I // 16, 16)], dim=1).reshape(2 * I).contiguous()
+
+
+@_launches("products")
+def gemm_geglu(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor],
+               out: torch.Tensor) -> None:
+    """out[M, I] = gelu(a Wg^T + bg) * (a Wu^T + bu) as bfloat16 (the tanh form), with ``w`` [2 I, K]
+    from ``interleave_gate_up`` and ``pretile_weight`` and ``bias`` float32 [2 I] from
+    ``interleave_bias`` or None: biases and activation are applied to the 32-bit sums in the
+    product's epilogue, by the kernels that ``gemm_swiglu`` would choose."""
+    _need_gpu(a, w, bias, out)
+    M, K = a.shape
+    N = w.shape[0]
+    if w.shape[1] != K or out.shape != (M, N // 2) or out.dtype != torch.bfloat16 \
+            or a.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 \
+            or not can_fuse_geglu(N // 2, K) \
+            or (bias is not None and (bias.shape != (N,) or bias.dtype != torch.float32)):
+        raise KernelUnavailable(f"gemm_geglu: a {tuple(a.shape)} {a.dtype}, w {tuple(w.shape)} "
+                                f"{w.dtype}, out {tuple(out.shape)} {out.dtype}")
+    if M == 0:
+        return
+    lib = build.load("gemm")
+    plan = _small_plan(M, N, K, True, swiglu=True) if M > 16 else None
+    ws, number, split = None, 0, 1
+    if plan is not None and plan[0] == "mid":
+        way = 2
+    elif M <= SKINNY_MAX_M:
+        way, number = 3, (plan[1] if plan is not None else 2)
+    else:
+        way, number = 0, _tile256_variant(M, N, K)
+        if number is None:
+            number = _tile_variant(M, N, True, False, K)
+            tail = _tile_tail_split(M, N, K) if number == 10 else None
+            if tail is not None:
+                way, (number, split) = 1, tail
+                tiles = ((M + 127) // 128) * ((N + 255) // 256)
+                ws = _workspace("gemm_tile_tail", (tiles - number) * split * 128 * 256,
+                                torch.float32, a.device)
+    _check(lib.zf_gemm_geglu(_ptr(a), _ptr(w), _ptr(bias), _ptr(out), _ptr(ws), M, N, K, way, number,
+                             split, _stream()), "gemm_geglu")
+
+
 # ------------------------------------------------------------------------- attention
 MAX_HEAD_DIM = 512          # the wave kernel keeps a head in registers: 8 values a lane
 DECODE_SPLIT_KEYS = 256     # keys per split of the decode kernel (DEC_SPLIT in attention.hip)

@@ -12,7 +12,7 @@ from typing import Callable, Dict
 from . import (gated_act, moe_grouped, norm_add_norm, tied_attention_mfma)
 from . import delta_recurrence, short_conv, streams_step
 from . import add_row, bias_act_rows, fixed_decay, rotation_table
-from . import embed_norm, gate_norm, gated_rows, state_space
+from . import embed_norm, gate_norm, gated_rows, gemm_geglu, state_space
 from . import (concat_rows, decay_recurrence, embed_sinusoid, head_norm_gate, token_shift_mix)
 from . import (activation, head_products, masked_attention, masked_attention_mfma,
                norm_add_store, project_rows)
@@ -57,6 +57,8 @@ KERNELS: Dict[str, KernelEntry] = {
     "gemm": KernelEntry(gemm, "gemm", _LINEAR),
     "gemm_partials": KernelEntry(gemm_partials, "gemm", _LINEAR),
     "gemm_swiglu": KernelEntry(gemm_swiglu, "gemm", _LINEAR + "; src/kernel/core/cpu.zig:130-147"),
+    "gemm_geglu": KernelEntry(gemm_geglu, "gemm", "own: a gate's and an up projection's product with "
+                              "biases and the tanh form of gelu in its epilogue"),
     "norm_gemm": KernelEntry(norm_gemm, "gemm", _RMSNORM + "; " + _LINEAR),
     "gemm_emit": KernelEntry(gemm_emit, "gemm", _LINEAR + "; " + _RMSNORM),
     "gemm_given": KernelEntry(gemm_given, "gemm", _RMSNORM + "; " + _LINEAR),

@@ -131,9 +131,10 @@ class DenseMlp(FeedForward):
 class GatedMlp(FeedForward):
     """d = W_down (act(W_gate m) * W_up m) with any of ``ops.ACTIVATIONS`` and, if the
     specification says so, biases on all three.  gate and up rows are stacked into one matrix at
-    load: each output keeps its own dot product; biases, activation and the product of the two
-    run in 32-bit on the product's rows.  The output's bias may be left to a norm behind the
-    part."""
+    load: each output keeps its own dot product.  Biases, activation and the product of the two
+    run in 32-bit: for the tanh form of gelu in bfloat16, where the sizes allow, in the product's
+    epilogue (gate and up rows then alternate in groups of 16), else on the product's rows.
+    The output's bias may be left to a norm behind the part."""
     graph_safe = True
     stores_output = True
     leaves_bias = True
@@ -160,12 +161,19 @@ class GatedMlp(FeedForward):
         g, u = tensors[p + s.gate_name], tensors[p + s.up_name]
         if g.dtype != u.dtype:
             g, u = g.float(), u.float()
-        self.gate_up = Linear(place_matrix(torch.cat([g, u], dim=0), self.ctx))
+        g, u = place_matrix(g, self.ctx), place_matrix(u, self.ctx)
+        self.fused = s.activation == "gelu_tanh" and g.is_cuda and g.dtype == torch.bfloat16 \
+            and self.ctx.compute_dtype == torch.bfloat16 \
+            and ops.can_fuse_geglu(s.intermediate_size, s.hidden_size)
+        self.gate_up = Linear(ops.interleave_gate_up(g, u) if self.fused
+                              else torch.cat([g, u], dim=0))
+        del g, u
         self.down = Linear(place_matrix(tensors[p + s.down_name], self.ctx))
         self.bias = self.down_bias = None
         if s.bias:
-            self.bias = place_gain(torch.cat([tensors[p + n + s.bias_suffix].to(torch.float32)
-                                              for n in (s.gate_name, s.up_name)]), self.ctx)
+            both = [tensors[p + n + s.bias_suffix].to(torch.float32) for n in (s.gate_name, s.up_name)]
+            self.bias = place_gain(ops.interleave_bias(*both) if self.fused else torch.cat(both),
+                                   self.ctx)
             self.down_bias = place_gain(tensors[p + s.down_name + s.bias_suffix], self.ctx)
 
     def forward(self, h, residual, step, accumulate: bool = True, leave_bias: bool = False):
@@ -174,9 +182,12 @@ class GatedMlp(FeedForward):
         if hasattr(h, "materialize"):
             h = h.materialize()
         a = step.scratch("ff_act", (T, I), act)
-        gu = step.scratch("gate_up", (T, 2 * I), act)
-        self.gate_up.forward(h, gu)
-        ops.gated_rows(gu, self.bias, a, self.spec.activation)
+        if self.fused:
+            ops.gemm_geglu(h, self.gate_up.weight, self.bias, a)
+        else:
+            gu = step.scratch("gate_up", (T, 2 * I), act)
+            self.gate_up.forward(h, gu)
+            ops.gated_rows(gu, self.bias, a, self.spec.activation)
         last = self.down_bias is None
         self.down.forward(a, residual, accumulate=accumulate,
                           step=step if accumulate and last else None)
