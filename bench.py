@@ -2054,9 +2054,10 @@ def tigesun_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float
     steps = f32(rows, H)
     al, db, sk = torch.zeros((H,), device=dev), torch.full((H,), -4.0, device=dev), f32(H)
     y = torch.empty((rows, I), dtype=torch.float32, device=dev)
+    given = (rnd(rows, W), rnd(H, W)) if decode else steps      # (formed by the kernel itself)
     t_new = _timed_graph(lambda: ops.state_space(
-        xbc[:, :I], xbc[:, I:I + BC], xbc[:, I + BC:], steps, al, db, sk, state, state_slots, q_start,
-        y, H, G, N, dv, lists=lists))
+        xbc[:, :I], xbc[:, I:I + BC], xbc[:, I + BC:], given, al, db, sk, state, state_slots, q_start,
+        y, H, G, N, dv, lists=lists, single_tokens=decode))
     fq, fk = rnd(rows, H * N), rnd(rows, H * N)
     old = torch.zeros((n_seqs, ops.fixed_decay_state_size(H, N, dv)), device=dev)
     decay = torch.stack([torch.full((H,), 0.99), torch.full((H,), 0.99).log2()]).to(dev)
@@ -2085,10 +2086,10 @@ def tigesun_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float
 
     def space_products():
         ops.gemm(h, w_in, wide2, w_tiled=True)
-        ops.gemm(h, w_s, steps, w_tiled=True)
+        if not decode:
+            ops.gemm(h, w_s, steps, w_tiled=True)
         ops.gemm(mixed, w_o, x, w_tiled=True)
     t_new = _timed_graph(space_products)
-    t_steps = _timed_graph(lambda: ops.gemm(h, w_s, steps, w_tiled=True))
     w_gu = ops.pretile_weight(ops.interleave_gate_up(rnd(ff, W), rnd(ff, W)))
     w_d = ops.pretile_weight(rnd(W, ff))
     act = torch.empty((rows, ff), dtype=bf, device=dev)
@@ -2101,7 +2102,9 @@ def tigesun_kernels(sh: dict, T: int, ctx: int, mfma_rate: float, read_bw: float
     n_q3, n_new = 3 * W * ff, W * (2 * I + C + H)
     row("space_products", t_new, 2.0 * rows * n_new, 2.0 * n_new,
         qwen3=(t_q3, 2.0 * rows * n_q3, 2.0 * n_q3))
-    row("step_product", t_steps, 2.0 * rows * W * H, 2.0 * (W * H + rows * W) + 4.0 * rows * H)
+    if not decode:
+        t_steps = _timed_graph(lambda: ops.gemm(h, w_s, steps, w_tiled=True))
+        row("step_product", t_steps, 2.0 * rows * W * H, 2.0 * (W * H + rows * W) + 4.0 * rows * H)
 
     def geglu_ff():
         ops.gemm_geglu(h, w_gu, both, act)

@@ -338,6 +338,26 @@ def test_recurrence_in_chunks(H, G, N, dv):
             assert all(torch.equal(a, b) for a, b in zip(seen, (first, second, state)))
 
 
+@pytest.mark.parametrize("H,G,N,dv,K", [(4, 2, 12, 10, 72), (64, 1, 128, 64, 2048), (3, 3, 24, 7, 4104)])
+def test_step_sizes_formed_where_they_are_used(H, G, N, dv, K):
+    """Single tokens of five sequences in bfloat16, from states that are not zero: step sizes from
+    the rows they are products of against the same given as numbers."""
+    T = 5
+    size = ops.state_space_state_size(H, N, dv)
+    rows, _ = _space_inputs(T, H, G, N, dv, 3, torch.bfloat16)
+    h, w = _rand((T, K), 4, 1.0, torch.bfloat16), _rand((H, K), 5, K ** -0.5, torch.bfloat16)
+    weights = [t.to(DEV) for t in _space_weights(H)]
+    rows, I, got = rows.to(DEV), H * dv, []
+    steps = (h.double() @ w.double().T).float().to(DEV)
+    for given in (steps, (h.to(DEV), w.to(DEV))):
+        state = _rand((T, size), 6).to(DEV)
+        out = torch.empty((T, I), dtype=torch.float32, device=DEV)
+        ops.state_space(rows[:, :I], rows[:, I:I + G * N], rows[:, I + G * N:], given, *weights, state,
+                        _i32(range(T)), _i32(range(T + 1)), out, H, G, N, dv, single_tokens=True)
+        got.append((out, state))
+    assert rel_err(got[1][0], got[0][0]) < 2e-5 and rel_err(got[1][1], got[0][1]) < 2e-5
+
+
 def test_a_token_far_back_is_kept_without_decay_and_lost_with_it():
     """Two heads, 600 tokens.  Token 3 alone writes (step size 1) along channel 0 with values that
     stand out; the last token asks for it.  The head whose decay is 1 to rounding returns them,

@@ -18,6 +18,14 @@ __device__ __forceinline__ void norm_store(TO* o, float v) {
   }
 }
 
+// four neighbouring results in one store
+template <typename TO> __device__ __forceinline__ void norm_store4(TO* o, const float4& v) {
+  if constexpr (sizeof(TO) == 2)
+    *(uint2*)o = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
+  else
+    *(float4*)o = v;
+}
+
 // any width: the row is read three times.  x_bias (or null): a row added to x first, what a
 // sublayer's output product leaves out
 template <typename TO, bool ADD>
@@ -141,38 +149,48 @@ extern "C" int zf_norm_rows(const float* x, const float* x_bias, const float* ga
 // still in registers (one kernel and one pass over the stream instead of two).  Widths that
 // are a multiple of 4 up to 8192.  Each norm as in norm_rows (32-bit, mean first, variance from
 // the deviations): the same numbers as the two kernels one after the other.
-template <typename TO>
+// NV groups of four columns a thread (256 NV * 4 >= W).  The stream's row and the gains are asked
+// for together with the branch's row, ahead of the sums that use them.
+template <typename TO, int NV>
 __global__ __launch_bounds__(256) void norm_add_norm_kernel(
-    const float* __restrict__ y, const float* __restrict__ y_bias, const float* __restrict__ gain_a, const float* __restrict__ bias_a,
-    float eps_a, int centred_a, float* __restrict__ x, const float* __restrict__ gain_b,
-    const float* __restrict__ bias_b, float eps_b, int centred_b, TO* __restrict__ out, int W) {
+    const float* __restrict__ y, const float* __restrict__ y_bias, const float* __restrict__ gain_a,
+    const float* __restrict__ bias_a, float eps_a, int centred_a, float* __restrict__ x,
+    const float* __restrict__ gain_b, const float* __restrict__ bias_b, float eps_b, int centred_b,
+    TO* __restrict__ out, int W) {
   __shared__ float red[16];
   const float4* yrow = (const float4*)(y + (size_t)blockIdx.x * W);
   float4* xrow = (float4*)(x + (size_t)blockIdx.x * W);
   TO* o = out + (size_t)blockIdx.x * W;
   const int n4 = W / 4;
-  float4 v[8];
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  float4 v[NV], r[NV], ga[NV], gb[NV];
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
+  for (int i = 0; i < NV; ++i) {
     const int c = threadIdx.x + i * 256;
-    v[i] = c < n4 ? yrow[c] : make_float4(0.f, 0.f, 0.f, 0.f);
-    if (y_bias != nullptr && c < n4) {
-      const float4 b = ((const float4*)y_bias)[c];
-      v[i].x += b.x; v[i].y += b.y; v[i].z += b.z; v[i].w += b.w;
+    v[i] = r[i] = ga[i] = gb[i] = zero;
+    if (c < n4) {
+      v[i] = yrow[c];
+      r[i] = xrow[c];
+      ga[i] = ((const float4*)gain_a)[c];
+      gb[i] = ((const float4*)gain_b)[c];
+      if (y_bias != nullptr) {
+        const float4 b = ((const float4*)y_bias)[c];
+        v[i].x += b.x; v[i].y += b.y; v[i].z += b.z; v[i].w += b.w;
+      }
     }
   }
   // one norm over the row held in v: v = (v - mean) * inv * gain + bias, in place
-  auto norm = [&](const float* gain, const float* bias, float eps, int centred) {
+  auto norm = [&](const float4 (&gain)[NV], const float* bias, float eps, int centred) {
     float mean = 0.f;
     if (centred) {
       float s = 0.f;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) s += (v[i].x + v[i].y) + (v[i].z + v[i].w);
+      for (int i = 0; i < NV; ++i) s += (v[i].x + v[i].y) + (v[i].z + v[i].w);
       mean = block_sum(s, red) / (float)W;
     }
     float ss = 0.f;
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
+    for (int i = 0; i < NV; ++i) {
       const int c = threadIdx.x + i * 256;
       if (c < n4) {
         v[i].x -= mean; v[i].y -= mean; v[i].z -= mean; v[i].w -= mean;
@@ -182,11 +200,11 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
     ss = block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)W + eps);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
+    for (int i = 0; i < NV; ++i) {
       const int c = threadIdx.x + i * 256;
       if (c < n4) {
-        const float4 g = ((const float4*)gain)[c];
-        float4 b = make_float4(0.f, 0.f, 0.f, 0.f);
+        const float4 g = gain[i];
+        float4 b = zero;
         if (bias != nullptr) b = ((const float4*)bias)[c];
         v[i].x = v[i].x * inv * g.x + b.x;
         v[i].y = v[i].y * inv * g.y + b.y;
@@ -195,42 +213,41 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
       }
     }
   };
-  norm(gain_a, bias_a, eps_a, centred_a);
+  norm(ga, bias_a, eps_a, centred_a);
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
+  for (int i = 0; i < NV; ++i) {
     const int c = threadIdx.x + i * 256;
     if (c < n4) {
-      const float4 r = xrow[c];
-      v[i].x = r.x + v[i].x; v[i].y = r.y + v[i].y; v[i].z = r.z + v[i].z; v[i].w = r.w + v[i].w;
+      v[i].x = r[i].x + v[i].x; v[i].y = r[i].y + v[i].y;
+      v[i].z = r[i].z + v[i].z; v[i].w = r[i].w + v[i].w;
       xrow[c] = v[i];
     }
   }
-  norm(gain_b, bias_b, eps_b, centred_b);
+  norm(gb, bias_b, eps_b, centred_b);
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
+  for (int i = 0; i < NV; ++i) {
     const int c = threadIdx.x + i * 256;
-    if (c < n4) {
-      store_from_float<TO>(o + 4 * c + 0, v[i].x);
-      store_from_float<TO>(o + 4 * c + 1, v[i].y);
-      store_from_float<TO>(o + 4 * c + 2, v[i].z);
-      store_from_float<TO>(o + 4 * c + 3, v[i].w);
-    }
+    if (c < n4) norm_store4<TO>(o + 4 * c, v[i]);
   }
 }
 
-extern "C" int zf_norm_add_norm(const float* y, const float* y_bias, const float* gain_a, const float* bias_a,
-                                float eps_a, int centred_a, float* x, const float* gain_b,
-                                const float* bias_b, float eps_b, int centred_b, void* out,
-                                int out_dtype, int T, int W, hipStream_t stream) {
+extern "C" int zf_norm_add_norm(const float* y, const float* y_bias, const float* gain_a,
+                                const float* bias_a, float eps_a, int centred_a, float* x,
+                                const float* gain_b, const float* bias_b, float eps_b,
+                                int centred_b, void* out, int out_dtype, int T, int W,
+                                hipStream_t stream) {
   if (T <= 0) return 0;
   if (W <= 0 || W % 4 != 0 || W > 8192) return -2;
-  if (out_dtype == ZF_F32)
-    hipLaunchKernelGGL(norm_add_norm_kernel<float>, dim3(T), dim3(256), 0, stream, y, y_bias,
-                       gain_a, bias_a, eps_a, centred_a, x, gain_b, bias_b, eps_b, centred_b, (float*)out, W);
-  else
-    hipLaunchKernelGGL(norm_add_norm_kernel<bf16_t>, dim3(T), dim3(256), 0, stream, y, y_bias,
-                       gain_a, bias_a, eps_a, centred_a, x, gain_b, bias_b, eps_b, centred_b,
-                       (bf16_t*)out, W);
+#define NORM_ADD_NORM(TO, NV)                                                                    \
+  hipLaunchKernelGGL((norm_add_norm_kernel<TO, NV>), dim3(T), dim3(256), 0, stream, y, y_bias,   \
+                     gain_a, bias_a, eps_a, centred_a, x, gain_b, bias_b, eps_b, centred_b,      \
+                     (TO*)out, W)
+#define NORM_ADD_NORM_ANY(TO)                                                                    \
+  if (W <= 1024) NORM_ADD_NORM(TO, 1);                                                           \
+  else if (W <= 2048) NORM_ADD_NORM(TO, 2);                                                      \
+  else if (W <= 4096) NORM_ADD_NORM(TO, 4);                                                      \
+  else NORM_ADD_NORM(TO, 8)
+  if (out_dtype == ZF_F32) { NORM_ADD_NORM_ANY(float); } else { NORM_ADD_NORM_ANY(bf16_t); }
   ZF_CHECK_LAUNCH();
 }
 
@@ -502,19 +519,84 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(
     store_from_float<TO>(o + i, load_as_float<TW>(row + i) * scale * inv * gain[i] * inv_b * gain_b[i]);
 }
 
+// The same for widths that are a multiple of 4 up to 8192: a thread keeps NV groups of four columns
+// in registers, the gains are asked for together with the row.
+template <typename TW, typename TO, int NV>
+__global__ __launch_bounds__(256) void embed_norm_vec_kernel(
+    const TW* __restrict__ table, const int* __restrict__ ids, float scale,
+    const float* __restrict__ gain, float eps, float* __restrict__ x,
+    const float* __restrict__ gain_b, float eps_b, TO* __restrict__ out, int W) {
+  __shared__ float red[16];
+  const TW* row = table + (size_t)ids[blockIdx.x] * W;
+  float4* xr = (float4*)(x + (size_t)blockIdx.x * W);
+  const int n4 = W / 4;
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  float4 v[NV], ga[NV], gb[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = threadIdx.x + i * 256;
+    v[i] = ga[i] = gb[i] = zero;
+    if (c < n4) {
+      ga[i] = ((const float4*)gain)[c];
+      if (gain_b != nullptr) gb[i] = ((const float4*)gain_b)[c];
+      if constexpr (sizeof(TW) == 2) {
+        const uint2 w = *(const uint2*)(row + 4 * c);
+        v[i] = make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u),
+                           __uint_as_float(w.y << 16), __uint_as_float(w.y & 0xffff0000u));
+      } else {
+        v[i] = *(const float4*)(row + 4 * c);
+      }
+      v[i].x *= scale; v[i].y *= scale; v[i].z *= scale; v[i].w *= scale;
+      ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+    }
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)W + eps);
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = threadIdx.x + i * 256;
+    if (c < n4) {
+      v[i] = make_float4(v[i].x * inv * ga[i].x, v[i].y * inv * ga[i].y, v[i].z * inv * ga[i].z,
+                         v[i].w * inv * ga[i].w);
+      xr[c] = v[i];
+      ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+    }
+  }
+  if (gain_b == nullptr) return;
+  const float inv_b = 1.0f / sqrtf(block_sum(ss, red) / (float)W + eps_b);
+  TO* o = out + (size_t)blockIdx.x * W;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = threadIdx.x + i * 256;
+    if (c < n4)
+      norm_store4<TO>(o + 4 * c, make_float4(v[i].x * inv_b * gb[i].x, v[i].y * inv_b * gb[i].y,
+                                             v[i].z * inv_b * gb[i].z, v[i].w * inv_b * gb[i].w));
+  }
+}
+
 extern "C" int zf_embed_norm(const void* table, int table_dtype, const int* ids, float scale,
                              const float* gain, float eps, float* x, const float* gain_b,
                              float eps_b, void* out, int out_dtype, int T, int W,
                              hipStream_t stream) {
   if (T <= 0) return 0;
   if (W <= 0 || (gain_b != nullptr && out == nullptr)) return -2;
+#define EMBED_NORM_K(K)                                                                          \
+  hipLaunchKernelGGL(K, dim3(T), dim3(256), 0, stream, table_t, ids, scale, gain, eps, x, gain_b, \
+                     eps_b, out_t, W)
 #define EMBED_NORM(TW, TO)                                                                       \
-  hipLaunchKernelGGL((embed_norm_kernel<TW, TO>), dim3(T), dim3(256), 0, stream,                 \
-                     (const TW*)table, ids, scale, gain, eps, x, gain_b, eps_b, (TO*)out, W)
+  {                                                                                              \
+    const TW* table_t = (const TW*)table;                                                        \
+    TO* out_t = (TO*)out;                                                                        \
+    if (W % 4 != 0 || W > 8192) EMBED_NORM_K((embed_norm_kernel<TW, TO>));                       \
+    else if (W <= 2048) EMBED_NORM_K((embed_norm_vec_kernel<TW, TO, 2>));                        \
+    else if (W <= 4096) EMBED_NORM_K((embed_norm_vec_kernel<TW, TO, 4>));                        \
+    else EMBED_NORM_K((embed_norm_vec_kernel<TW, TO, 8>));                                       \
+  }
   if (table_dtype == ZF_F32) {
-    if (out_dtype == ZF_F32) EMBED_NORM(float, float); else EMBED_NORM(float, bf16_t);
+    if (out_dtype == ZF_F32) EMBED_NORM(float, float) else EMBED_NORM(float, bf16_t)
   } else {
-    if (out_dtype == ZF_F32) EMBED_NORM(bf16_t, float); else EMBED_NORM(bf16_t, bf16_t);
+    if (out_dtype == ZF_F32) EMBED_NORM(bf16_t, float) else EMBED_NORM(bf16_t, bf16_t)
   }
   ZF_CHECK_LAUNCH();
 }

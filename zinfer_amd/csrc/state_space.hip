@@ -30,7 +30,27 @@ struct StateSpace {
   const float* bias;           // b [H]
   const float* skip;           // D [H]
   int H, G, N, dv, NP;         // NP: N padded to 4
+  // single tokens, bfloat16: steps null, s_h = w_h . h instead, formed where it is used (h [T, K],
+  // w [H, K], K a multiple of 8, rows on 16 bytes)
+  const bf16_t* h;
+  const bf16_t* w;
+  int K;
 };
+
+// w . h over a workgroup's threads in every one of them
+__device__ __forceinline__ float ss_dot(const bf16_t* h, const bf16_t* w, int K, float* red) {
+  float a = 0.f;
+  for (int i = threadIdx.x * 8; i < K; i += blockDim.x * 8) {
+    const uint4 x = *(const uint4*)(h + i), y = *(const uint4*)(w + i);
+    const uint32_t xs[4] = {x.x, x.y, x.z, x.w}, ys[4] = {y.x, y.y, y.z, y.w};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      a = fmaf(__uint_as_float(xs[e] << 16), __uint_as_float(ys[e] << 16), a);
+      a = fmaf(__uint_as_float(xs[e] & 0xffff0000u), __uint_as_float(ys[e] & 0xffff0000u), a);
+    }
+  }
+  return block_sum(a, red);
+}
 
 __device__ __forceinline__ float ss_softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
@@ -53,7 +73,7 @@ __global__ __launch_bounds__(256) void state_space_walk_kernel(
   constexpr int VBMAX = 4 * SS_NC * CPW;
   __shared__ __attribute__((aligned(16))) float bs[SS_TC * KW], cs[SS_TC * KW];
   __shared__ float xs[SS_TC * VBMAX];
-  __shared__ float gs[SS_TC];
+  __shared__ float gs[SS_TC], red[16];
   const int s = seqs != nullptr ? seqs[blockIdx.x] : blockIdx.x;
   const int hd = blockIdx.y, grp = hd / (p.H / p.G);
   const int t0 = q_start[s], t1 = q_start[s + 1];
@@ -73,6 +93,12 @@ __global__ __launch_bounds__(256) void state_space_walk_kernel(
       S[i] = *(const float4*)(st + (size_t)(v0 + col[i]) * p.NP + 4 * cg);
   }
   const float rate = expf(p.a_log[hd]), bias = p.bias[hd], skip = p.skip[hd];
+  const bool own = p.h != nullptr;                   // (then every sequence brings one token)
+  const float own_step = own && t0 < t1
+      ? ss_dot(p.h + (size_t)t0 * p.K, p.w + (size_t)hd * p.K, p.K, red) : 0.f;
+  auto step_size = [&](int t) {
+    return ss_softplus((own ? own_step : p.steps[(size_t)t * p.H + hd]) + bias);
+  };
   for (int tc = t0; tc < t1; tc += SS_TC) {
     const int n = min(SS_TC, t1 - tc);
     __syncthreads();                                 // the rows before are done with
@@ -81,7 +107,7 @@ __global__ __launch_bounds__(256) void state_space_walk_kernel(
       float bv = 0.f, cv = 0.f;
       if (c < p.N) {
         const size_t at = (size_t)(tc + t) * bc_stride + (size_t)grp * p.N + c;
-        const float dt = ss_softplus(p.steps[(size_t)(tc + t) * p.H + hd] + bias);
+        const float dt = step_size(tc + t);
         bv = dt * load_as_float<T>(br + at);
         cv = load_as_float<T>(cr + at);
       }
@@ -94,7 +120,7 @@ __global__ __launch_bounds__(256) void state_space_walk_kernel(
           ? load_as_float<T>(xr + (size_t)(tc + t) * x_stride + (size_t)hd * p.dv + v0 + x) : 0.f;
     }
     if (tid < n)
-      gs[tid] = expf(-(rate * ss_softplus(p.steps[(size_t)(tc + tid) * p.H + hd] + bias)));
+      gs[tid] = expf(-(rate * step_size(tc + tid)));
     __syncthreads();
     for (int t = 0; t < n; ++t) {
       const float4 b4 = *(const float4*)(bs + t * KW + 4 * cg);
@@ -135,16 +161,22 @@ static bool ss_sizes(const StateSpace& p, long long slot_stride) {
 }
 
 // seqs: the step's sequences to run (indices into q_start and state_slots), n_seqs of them; null:
-// 0 .. n_seqs - 1
+// 0 .. n_seqs - 1.  steps null (bfloat16, every sequence one token): h [T, K] and w [H, K] instead.
 extern "C" int zf_state_space_walk(const void* x, long long x_stride, const void* b, const void* c,
                                    long long bc_stride, int dtype, const float* steps,
                                    const float* a_log, const float* bias, const float* skip,
                                    float* state, long long slot_stride, const int* state_slots,
                                    const int* q_start, const int* seqs, float* out, int n_seqs,
-                                   int H, int G, int N, int dv, hipStream_t stream) {
+                                   int H, int G, int N, int dv, const void* h, const void* w, int K,
+                                   hipStream_t stream) {
   if (n_seqs <= 0) return 0;
-  const StateSpace p = {steps, a_log, bias, skip, H, G, N, dv, (N + 3) / 4 * 4};
+  const bool own = steps == nullptr;
+  const StateSpace p = {steps, a_log, bias, skip, H, G, N, dv, (N + 3) / 4 * 4,
+                        own ? (const bf16_t*)h : nullptr, own ? (const bf16_t*)w : nullptr, K};
   if (!ss_sizes(p, slot_stride)) return -2;
+  if (own && (dtype != ZF_BF16 || h == nullptr || w == nullptr || K % 8 != 0 || K <= 0 ||
+              (uintptr_t)h % 16 != 0 || (uintptr_t)w % 16 != 0))
+    return -2;
   int lpc = 4;
   while (4 * lpc < p.NP) lpc *= 2;
   const int per_wave = SS_NC * (ZF_WAVE / lpc);
@@ -519,7 +551,7 @@ extern "C" int zf_state_space_chunks(const void* x, long long x_stride, const vo
                                      float* states, float* decays, float* out, int H, int G, int N,
                                      int dv, int heads, hipStream_t stream) {
   if (n_chunks <= 0 || n_long <= 0) return 0;
-  const StateSpace p = {steps, a_log, bias, skip, H, G, N, dv, (N + 3) / 4 * 4};
+  const StateSpace p = {steps, a_log, bias, skip, H, G, N, dv, (N + 3) / 4 * 4, nullptr, nullptr, 0};
   if (!ss_sizes(p, slot_stride) || states == nullptr || decays == nullptr || heads < 1 ||
       heads > SS_HEADS_MAX || (H / G) % heads != 0)
     return -2;

@@ -3124,12 +3124,17 @@ def state_space_heads(n_chunks: int, n_heads: int, n_groups: int, value_dim: int
     return best
 
 
+def state_space_forms_steps(hidden_size: int) -> bool:
+    """Whether ``state_space`` takes the step sizes of single tokens as rows of that width."""
+    return hidden_size % 8 == 0
+
+
 @_launches("attention")
-def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, steps: torch.Tensor,
+def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, steps,
                 decay_log: torch.Tensor, step_bias: torch.Tensor, skip: torch.Tensor,
                 state: torch.Tensor, state_slots: torch.Tensor, q_start: torch.Tensor,
                 out: torch.Tensor, n_heads: int, n_groups: int, state_dim: int, value_dim: int, *,
-                lists=None, heads: Optional[int] = None) -> None:
+                lists=None, heads: Optional[int] = None, single_tokens: bool = False) -> None:
     """dt_t = softplus(steps_t + step_bias), S_t = exp(-exp(decay_log) dt_t) S_(t-1) + dt_t b_t
     x_t^T, out_t = S_t^T c_t + skip x_t a head, in 32-bit, over the rows of a step: ``x`` [T, >= H
     * dv], ``b`` and ``c`` [T, >= G * N] (contiguous rows, any row stride, that of b and c the
@@ -3142,7 +3147,22 @@ def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, steps: torch.
     then run in chunks side by side through MFMAs, where an operand that is a 32-bit number
     enters as two bfloat16 terms (``heads``: how many heads a workgroup takes, None: by
     ``state_space_heads``).  None: token by token, all 32-bit, every size and both types (the
-    same bits however a sequence is cut into steps)."""
+    same bits however a sequence is cut into steps).
+
+    ``single_tokens`` (bfloat16, no ``lists``): every sequence brings one token, and ``steps`` may
+    be a pair (h [T, K], w [H, K]) of bfloat16 rows instead: the numbers w . h are then formed
+    where they are used (``state_space_forms_steps`` says whether the sizes allow it)."""
+    pair = isinstance(steps, tuple)
+    h, w = steps if pair else (None, None)
+    if pair:
+        _need_gpu(h, w)
+        steps = None
+        if not single_tokens or lists is not None or x.dtype != torch.bfloat16 \
+                or h.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 \
+                or h.shape[0] != x.shape[0] or w.shape != (int(n_heads), h.shape[1]) \
+                or h.shape[0] != state_slots.shape[0] or not state_space_forms_steps(h.shape[1]):
+            raise KernelUnavailable(f"state_space: step sizes from rows {tuple(h.shape)} {h.dtype} "
+                                    f"and {tuple(w.shape)} {w.dtype}: single tokens in bfloat16 only")
     _need_gpu(steps, decay_log, step_bias, skip, state_slots, q_start, out)
     for t in (x, b, c, state):
         if not t.is_cuda:
@@ -3160,7 +3180,7 @@ def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, steps: torch.
     if x.shape[1] < H * dv or b.shape[1] < G * N or c.shape[1] < G * N or b.shape[0] != T \
             or c.shape[0] != T or b.dtype != x.dtype or c.dtype != x.dtype \
             or (T > 1 and _columns(c, "state_space: c") != bs) \
-            or steps.shape != (T, H) or steps.dtype != torch.float32 \
+            or (not pair and (steps.shape != (T, H) or steps.dtype != torch.float32)) \
             or any(v.shape != (H,) or v.dtype != torch.float32 for v in (decay_log, step_bias, skip)) \
             or out.shape != (T, H * dv) or out.dtype != torch.float32 \
             or state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 \
@@ -3168,7 +3188,7 @@ def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, steps: torch.
             or q_start.shape[0] != n_seqs + 1 \
             or (lists is not None and x.dtype != torch.bfloat16):
         raise KernelUnavailable(f"state_space: x {tuple(x.shape)}, b {tuple(b.shape)}, c "
-                                f"{tuple(c.shape)} {x.dtype}, steps {tuple(steps.shape)}, out "
+                                f"{tuple(c.shape)} {x.dtype}, steps {None if pair else tuple(steps.shape)}, out "
                                 f"{tuple(out.shape)} {out.dtype}, state {tuple(state.shape)} "
                                 f"{state.dtype} (rows a multiple of 4 floats, at least {need})")
     lib = build.load("state_space")
@@ -3193,4 +3213,4 @@ def state_space(x: torch.Tensor, b: torch.Tensor, c: torch.Tensor, steps: torch.
     if n_short:
         _check(lib.zf_state_space_walk(
             *rows, _dt(x), *head, _ptr(q_start), _ptr(shorts), _ptr(out), n_short, H, G, N, dv,
-            _stream()), "state_space (token by token)")
+            _ptr(h), _ptr(w), h.shape[1] if pair else 0, _stream()), "state_space (token by token)")

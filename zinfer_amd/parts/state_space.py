@@ -15,7 +15,8 @@ class StateSpace(Mixer):
     """The mixer of ``StateSpaceSpec``.  z, x, B and C come from one product (the input matrix's
     rows without its last ones, filled up to the multiple of 64 the MFMA kernels' own order
     takes), the step sizes' numbers from a second one over those last rows that leaves its
-    accumulators as 32-bit numbers.  One kernel runs the short convolutions with bias and silu
+    accumulators as 32-bit numbers (single tokens in bfloat16: the recurrence's kernel forms them
+    itself, one launch less).  One kernel runs the short convolutions with bias and silu
     from the product's rows and the request's last rows; the recurrence's kernels form step size
     and decay a head and token and keep every request's matrices in its state slot (32-bit), the
     convolution's last rows behind them (32-bit); one more kernel applies the gate and norms the
@@ -73,7 +74,12 @@ class StateSpace(Mixer):
         if rows % self.ALIGN:
             wide = torch.cat([wide, wide.new_zeros((-rows % self.ALIGN, wide.shape[1]))], dim=0)
         self.proj = Linear(place_matrix(wide.contiguous(), self.ctx))
-        self.step_proj = Linear(place_matrix(w[rows:].contiguous(), self.ctx))
+        steps = place_matrix(w[rows:].contiguous(), self.ctx)
+        self.step_proj = Linear(steps)
+        # the rows as they lie, for the kernel that forms single tokens' step sizes itself
+        self.step_rows = steps if steps.dtype == torch.bfloat16 and \
+            self.ctx.compute_dtype == torch.bfloat16 and \
+            ops.state_space_forms_steps(s.hidden_size) else None
         self.taps = place_gain(tensors[p + s.conv_name], self.ctx)
         self.conv_bias = place_gain(tensors[p + s.conv_bias_name], self.ctx)
         self.step_bias = place_gain(tensors[p + s.step_bias_name], self.ctx)
@@ -100,11 +106,15 @@ class StateSpace(Mixer):
         I, BC = self.inner, self.bc_width
         proj = step.scratch("space_proj", (T, self.proj.out_features), act)
         self.proj.forward(h, proj)
-        sizes = step.scratch("space_steps", (T, s.n_heads), torch.float32)
-        self.step_proj.forward(h, sizes)
+        single = step.max_q_len == 1
+        if single and self.step_rows is not None:
+            sizes = (h, self.step_rows)
+        else:
+            sizes = step.scratch("space_steps", (T, s.n_heads), torch.float32)
+            self.step_proj.forward(h, sizes)
         xbc = step.scratch("space_xbc", (T, self.conv_width), act)
         ops.short_conv(proj[:, I:], self.taps, cache.state, self.matrix_size, step.state_slots,
-                       step.seq_index, step.q_start, xbc, single_tokens=step.max_q_len == 1,
+                       step.seq_index, step.q_start, xbc, single_tokens=single,
                        bias=self.conv_bias)
         hints = step.hints.get(self.hint_key) if self.hint_key is not None else None
         lists = None
@@ -113,7 +123,8 @@ class StateSpace(Mixer):
         y = step.scratch("space_out", (T, I), torch.float32)
         ops.state_space(xbc[:, :I], xbc[:, I:I + BC], xbc[:, I + BC:], sizes, self.decay_log,
                         self.step_bias, self.skip, cache.state, step.state_slots, step.q_start, y,
-                        s.n_heads, s.n_groups, s.state_dim, s.value_dim, lists=lists)
+                        s.n_heads, s.n_groups, s.state_dim, s.value_dim, lists=lists,
+                        single_tokens=single)
         mixed = step.scratch("space_mixed", (T, I), act)
         ops.gate_norm(y, self.gain, proj[:, :I], mixed, s.norm_groups, float(s.norm_eps))
         self.o.forward(mixed, residual, accumulate=accumulate, step=step if accumulate else None)
