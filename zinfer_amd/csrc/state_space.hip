@@ -37,19 +37,15 @@ struct StateSpace {
   int K;
 };
 
-// w . h over a workgroup's threads in every one of them
-__device__ __forceinline__ float ss_dot(const bf16_t* h, const bf16_t* w, int K, float* red) {
-  float a = 0.f;
-  for (int i = threadIdx.x * 8; i < K; i += blockDim.x * 8) {
-    const uint4 x = *(const uint4*)(h + i), y = *(const uint4*)(w + i);
-    const uint32_t xs[4] = {x.x, x.y, x.z, x.w}, ys[4] = {y.x, y.y, y.z, y.w};
+// 8 neighbouring products of w . h
+__device__ __forceinline__ float ss_dot8(const uint4& x, const uint4& y, float a) {
+  const uint32_t xs[4] = {x.x, x.y, x.z, x.w}, ys[4] = {y.x, y.y, y.z, y.w};
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      a = fmaf(__uint_as_float(xs[e] << 16), __uint_as_float(ys[e] << 16), a);
-      a = fmaf(__uint_as_float(xs[e] & 0xffff0000u), __uint_as_float(ys[e] & 0xffff0000u), a);
-    }
+  for (int e = 0; e < 4; ++e) {
+    a = fmaf(__uint_as_float(xs[e] << 16), __uint_as_float(ys[e] << 16), a);
+    a = fmaf(__uint_as_float(xs[e] & 0xffff0000u), __uint_as_float(ys[e] & 0xffff0000u), a);
   }
-  return block_sum(a, red);
+  return a;
 }
 
 __device__ __forceinline__ float ss_softplus(float z) { return z > 20.f ? z : log1pf(expf(z)); }
@@ -83,6 +79,36 @@ __global__ __launch_bounds__(256) void state_space_walk_kernel(
   const int cg = lane % LPC, cl = lane / LPC;
   const bool live = 4 * cg < p.NP;
   float* st = state + (size_t)state_slots[s] * slot_stride + (size_t)hd * p.dv * p.NP;
+  // a single token: its rows, and what its step size is the product of, are asked for ahead of the
+  // matrix (which takes longest to come)
+  const bool own = p.h != nullptr;                   // (then every sequence brings one token)
+  const bool one = t1 - t0 == 1 && KW <= (int)blockDim.x && VB <= (int)blockDim.x;
+  float b1 = 0.f, c1 = 0.f, x1 = 0.f, s1 = 0.f;
+  constexpr int DOTS = 2;
+  uint4 hv[DOTS], wv[DOTS];
+  const bf16_t* hrow = p.h + (size_t)t0 * p.K;
+  const bf16_t* wrow = p.w + (size_t)hd * p.K;
+  if (one) {
+    if (tid < p.N) {
+      const size_t at = (size_t)t0 * bc_stride + (size_t)grp * p.N + tid;
+      b1 = load_as_float<T>(br + at);
+      c1 = load_as_float<T>(cr + at);
+    }
+    if (tid < VB && v0 + tid < p.dv)
+      x1 = load_as_float<T>(xr + (size_t)t0 * x_stride + (size_t)hd * p.dv + v0 + tid);
+    if (!own) s1 = p.steps[(size_t)t0 * p.H + hd];
+  }
+  if (own && t0 < t1) {
+#pragma unroll
+    for (int u = 0; u < DOTS; ++u) {
+      const int i = (tid + u * blockDim.x) * 8;
+      hv[u] = wv[u] = make_uint4(0u, 0u, 0u, 0u);
+      if (i < p.K) {
+        hv[u] = *(const uint4*)(hrow + i);
+        wv[u] = *(const uint4*)(wrow + i);
+      }
+    }
+  }
   float4 S[SS_NC];
   int col[SS_NC];
 #pragma unroll
@@ -93,34 +119,46 @@ __global__ __launch_bounds__(256) void state_space_walk_kernel(
       S[i] = *(const float4*)(st + (size_t)(v0 + col[i]) * p.NP + 4 * cg);
   }
   const float rate = expf(p.a_log[hd]), bias = p.bias[hd], skip = p.skip[hd];
-  const bool own = p.h != nullptr;                   // (then every sequence brings one token)
-  const float own_step = own && t0 < t1
-      ? ss_dot(p.h + (size_t)t0 * p.K, p.w + (size_t)hd * p.K, p.K, red) : 0.f;
+  if (own && t0 < t1) {
+    float a = 0.f;
+#pragma unroll
+    for (int u = 0; u < DOTS; ++u) a = ss_dot8(hv[u], wv[u], a);
+    for (int i = (tid + DOTS * blockDim.x) * 8; i < p.K; i += blockDim.x * 8)
+      a = ss_dot8(*(const uint4*)(hrow + i), *(const uint4*)(wrow + i), a);
+    s1 = block_sum(a, red);
+  }
   auto step_size = [&](int t) {
-    return ss_softplus((own ? own_step : p.steps[(size_t)t * p.H + hd]) + bias);
+    return ss_softplus((own || one ? s1 : p.steps[(size_t)t * p.H + hd]) + bias);
   };
   for (int tc = t0; tc < t1; tc += SS_TC) {
     const int n = min(SS_TC, t1 - tc);
     __syncthreads();                                 // the rows before are done with
-    for (int i = tid; i < n * KW; i += blockDim.x) {
-      const int t = i / KW, c = i % KW;
-      float bv = 0.f, cv = 0.f;
-      if (c < p.N) {
-        const size_t at = (size_t)(tc + t) * bc_stride + (size_t)grp * p.N + c;
-        const float dt = step_size(tc + t);
-        bv = dt * load_as_float<T>(br + at);
-        cv = load_as_float<T>(cr + at);
+    if (one) {
+      const float dt = step_size(t0);
+      if (tid < KW) {
+        bs[tid] = dt * b1;
+        cs[tid] = c1;
       }
-      bs[i] = bv;
-      cs[i] = cv;
+      if (tid < VB) xs[tid] = x1;
+    } else {
+      for (int i = tid; i < n * KW; i += blockDim.x) {
+        const int t = i / KW, c = i % KW;
+        float bv = 0.f, cv = 0.f;
+        if (c < p.N) {
+          const size_t at = (size_t)(tc + t) * bc_stride + (size_t)grp * p.N + c;
+          bv = step_size(tc + t) * load_as_float<T>(br + at);
+          cv = load_as_float<T>(cr + at);
+        }
+        bs[i] = bv;
+        cs[i] = cv;
+      }
+      for (int i = tid; i < n * VB; i += blockDim.x) {
+        const int t = i / VB, x = i % VB;
+        xs[t * VBMAX + x] = v0 + x < p.dv
+            ? load_as_float<T>(xr + (size_t)(tc + t) * x_stride + (size_t)hd * p.dv + v0 + x) : 0.f;
+      }
     }
-    for (int i = tid; i < n * VB; i += blockDim.x) {
-      const int t = i / VB, x = i % VB;
-      xs[t * VBMAX + x] = v0 + x < p.dv
-          ? load_as_float<T>(xr + (size_t)(tc + t) * x_stride + (size_t)hd * p.dv + v0 + x) : 0.f;
-    }
-    if (tid < n)
-      gs[tid] = expf(-(rate * step_size(tc + tid)));
+    if (tid < n) gs[tid] = expf(-(rate * step_size(tc + tid)));
     __syncthreads();
     for (int t = 0; t < n; ++t) {
       const float4 b4 = *(const float4*)(bs + t * KW + 4 * cg);
