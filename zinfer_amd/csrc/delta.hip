@@ -18,7 +18,15 @@
 // four lines above with one pass over S less.
 #include "zf_common.h"
 
+#include <type_traits>
+
 __device__ __forceinline__ float dl_silu(float z) { return z / (1.0f + expf(-z)); }
+// silu of what leaves in TO (for bfloat16 through the bare exponential and reciprocal)
+template <typename TO> __device__ __forceinline__ float dl_silu_to(float z) {
+  if constexpr (sizeof(TO) == 2)
+    return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+  return dl_silu(z);
+}
 __device__ __forceinline__ float dl_softplus(float z) {
   return z > 20.f ? z : log1pf(expf(z));
 }
@@ -65,6 +73,7 @@ __device__ __forceinline__ float dl_lanes_sum(float v) {
 // only reader of its channel's kept rows): the state is moved on by this kernel.
 #define DL_CONV_THREADS 256
 #define DL_CONV_MAX_TAPS 8
+#define DL_CONV_ROWS_AHEAD 8     // tokens whose rows a thread of the rows' form asks for at once
 #define DL_CONV_PER_THREAD 4     // channels a thread takes of a head wider than the workgroup
 
 template <typename T, typename TO>
@@ -102,7 +111,7 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_kernel(
       for (int j = 1; j < DL_CONV_MAX_TAPS; ++j)
         if (j < n_taps) st[(size_t)(j - 1) * C + c] = x[j];
     }
-    return dl_silu(bias != nullptr ? acc + bias[c] : acc);
+    return dl_silu_to<TO>(bias != nullptr ? acc + bias[c] : acc);
   };
   TO* o = out + (size_t)t * C;
   const int b = blockIdx.y;
@@ -187,9 +196,10 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_rows_kernel(
     if (bias != nullptr) f = *(const float4*)(bias + c + v);
     b[v] = f.x; b[v + 1] = f.y; b[v + 2] = f.z; b[v + 3] = f.w;
   }
-  auto load_row = [&](int t, float (&x)[V]) {
+  typedef typename std::conditional<sizeof(T) == 2, uint4, float4>::type raw_t;      // V channels
+  auto raw_row = [&](int t) { return *(const raw_t*)(src + (size_t)t * src_stride + c); };
+  auto open_row = [&](const raw_t& r, float (&x)[V]) {
     if constexpr (sizeof(T) == 2) {
-      const uint4 r = *(const uint4*)(src + (size_t)t * src_stride + c);
       const uint32_t u[4] = {r.x, r.y, r.z, r.w};
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -197,45 +207,38 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_rows_kernel(
         x[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u);
       }
     } else {
-      const float4 f = *(const float4*)(src + (size_t)t * src_stride + c);
-      x[0] = f.x; x[1] = f.y; x[2] = f.z; x[3] = f.w;
+      x[0] = r.x; x[1] = r.y; x[2] = r.z; x[3] = r.w;
     }
   };
-  const int first = blockIdx.x * TT, last = min(n_tokens, first + TT);
-  int seq = -1;
-  for (int t = first; t < last; ++t) {
-    const int s = seq_index[t];
-    float* st = state + (size_t)state_slots[s] * state_stride + state_off;
-    if (s != seq) {
-      // the rows before this token: of its portion, or of the request's state
-      const int i0 = t - q_start[s];
+  // the rows before token t: of its portion, or of the request's state
+  auto rows_before = [&](int t, int s, const float* st) {
+    const int i0 = t - q_start[s];
 #pragma unroll
-      for (int k = 0; k < NT - 1; ++k) {
-        const int back = NT - 1 - k;
+    for (int k = 0; k < NT - 1; ++k) {
+      const int back = NT - 1 - k;
 #pragma unroll
-        for (int v = 0; v < V; ++v) w[k][v] = 0.f;
-        if (back <= hist) {
-          if (back <= i0) {
-            load_row(t - back, w[k]);
-          } else {
+      for (int v = 0; v < V; ++v) w[k][v] = 0.f;
+      if (back <= hist) {
+        if (back <= i0) {
+          open_row(raw_row(t - back), w[k]);
+        } else {
 #pragma unroll
-            for (int v = 0; v < V; v += 4) {
-              const float4 f = *(const float4*)(st + (size_t)(hist + i0 - back) * C + c + v);
-              w[k][v] = f.x; w[k][v + 1] = f.y; w[k][v + 2] = f.z; w[k][v + 3] = f.w;
-            }
+          for (int v = 0; v < V; v += 4) {
+            const float4 f = *(const float4*)(st + (size_t)(hist + i0 - back) * C + c + v);
+            w[k][v] = f.x; w[k][v + 1] = f.y; w[k][v + 2] = f.z; w[k][v + 3] = f.w;
           }
         }
       }
-      seq = s;
     }
-    load_row(t, w[NT - 1]);
+  };
+  auto emit = [&](int t) {
     float acc[V];
 #pragma unroll
     for (int v = 0; v < V; ++v) {
       acc[v] = 0.f;
 #pragma unroll
       for (int k = 0; k < NT; ++k) acc[v] = acc[v] + tp[k][v] * w[k][v];
-      acc[v] = dl_silu(bias != nullptr ? acc[v] + b[v] : acc[v]);
+      acc[v] = dl_silu_to<TO>(bias != nullptr ? acc[v] + b[v] : acc[v]);
     }
     TO* o = out + (size_t)t * C + c;
     if constexpr (sizeof(TO) == 2) {
@@ -246,6 +249,37 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_rows_kernel(
       for (int v = 0; v < V; v += 4)
         *(float4*)(o + v) = make_float4(acc[v], acc[v + 1], acc[v + 2], acc[v + 3]);
     }
+  };
+  auto move_on = [&]() {
+#pragma unroll
+    for (int k = 0; k + 1 < NT; ++k)
+#pragma unroll
+      for (int v = 0; v < V; ++v) w[k][v] = w[k + 1][v];
+  };
+  const int first = blockIdx.x * TT, last = min(n_tokens, first + TT);
+  const int s0 = seq_index[first];
+  if (TT == DL_CONV_ROWS_AHEAD && last - first == TT && seq_index[last - 1] == s0) {
+    // tokens of one sequence: their rows are asked for all at once
+    raw_t raw[DL_CONV_ROWS_AHEAD];
+#pragma unroll
+    for (int u = 0; u < DL_CONV_ROWS_AHEAD; ++u) raw[u] = raw_row(first + u);
+    rows_before(first, s0, state + (size_t)state_slots[s0] * state_stride + state_off);
+#pragma unroll
+    for (int u = 0; u < DL_CONV_ROWS_AHEAD; ++u) {
+      open_row(raw[u], w[NT - 1]);
+      emit(first + u);
+      move_on();
+    }
+    return;
+  }
+  int seq = -1;
+  for (int t = first; t < last; ++t) {
+    const int s = seq_index[t];
+    float* st = state + (size_t)state_slots[s] * state_stride + state_off;
+    if (s != seq) rows_before(t, s, st);
+    seq = s;
+    open_row(raw_row(t), w[NT - 1]);
+    emit(t);
     if (update_state) {
       // the kept rows move on by one: the last n_taps - 1 rows of the window
 #pragma unroll
@@ -257,10 +291,7 @@ __global__ __launch_bounds__(DL_CONV_THREADS) void short_conv_rows_kernel(
                 make_float4(w[k][v], w[k][v + 1], w[k][v + 2], w[k][v + 3]);
         }
     }
-#pragma unroll
-    for (int k = 0; k + 1 < NT; ++k)
-#pragma unroll
-      for (int v = 0; v < V; ++v) w[k][v] = w[k + 1][v];
+    move_on();
   }
 }
 
